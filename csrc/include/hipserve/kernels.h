@@ -175,6 +175,9 @@ constexpr int PG_EPI_STORE = 0, PG_EPI_ADD = 1, PG_EPI_GLU = 2, PG_EPI_GEGLU = 3
 constexpr int PW_EPI_STORE = 0, PW_EPI_ADD = 1, PW_EPI_GLU = 2, PW_EPI_GEGLU = 3;
 // PW_EPI_RELU2: as STORE with C = bf16(max(acc, 0)^2) (the squared-ReLU experts of the table-routed MoE)
 constexpr int PW_EPI_RELU2 = 4;
+// PW_EPI_CGLU (grouped gather form only): as GLU with g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
+// u = clamp(up, -limit, limit), the products first multiplied by their pair's row_scale
+constexpr int PW_EPI_CGLU = 5;
 // grid_req <= 0: persistent (one workgroup per CU walking the tiles), else that many workgroups.
 // rw: weight register sets in flight (2 or 4 32-deep slots ahead; 5 = 4 with each reload
 // issued one MFMA group later).
@@ -189,6 +192,9 @@ struct PwGroup {
   const int* gather_slots = nullptr;
   int gather_k = 1;
   int x_rows = 0;
+  // PW_EPI_CGLU (gather form): products of slot row s times row_scale[gather_slots[s]] (null: 1), clamped at limit
+  const float* row_scale = nullptr;
+  float limit = 0.f;
 };
 bool launch_prefill_gemm_packed(int epi, void* C, long ldc, const void* X, long ldx, const void* Wp, int M, int N,
                                 int K, const void* bias, int wm, int grid_req, hipStream_t s,

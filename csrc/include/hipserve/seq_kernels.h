@@ -50,10 +50,11 @@ void launch_mingru_scan(void* y, float* state, const void* proj, const float* b_
 
 // out[slot, N] = act(W[e(tile)] [N, K] . x[row(slot)]) over moe_align tiles of `tile` slots; tiles whose
 // expert is < 0 or >= E (no weights) are skipped. act 0: none, 1: squared ReLU, 2: W[e] = [gate rows; up rows]
-// and out[slot, N / 2] = silu(gate) * up.
+// and out[slot, N / 2] = silu(gate) * up, 3: the same with g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
+// u = clamp(up, -limit, limit). row_scale (may be null): the products of pair p are multiplied by row_scale[p] first.
 void launch_expert_gemm(void* out, const void* x, long x_ld, const void* w, const int* slots, const int* tile_expert,
-                        int ntiles_cap, int tile, int gather_k, int N, int K, int act, int E, bool f32,
-                        hipStream_t s);
+                        int ntiles_cap, int tile, int gather_k, int N, int K, int act, int E, const float* row_scale,
+                        float limit, bool f32, hipStream_t s);
 
 // Residual update with the norm on the sublayer's output (group_norm.hip): residual[T, H] (fp32, in place) +=
 // y / sqrt(mean(y^2) + eps) * w; out = residual in the activation type. y null: the addend is a mixture's output,
@@ -62,28 +63,30 @@ void launch_add_normed(void* out, float* residual, const float* w, int T, int H,
                        const void* ye, const int* pair_slot, const int* ids, const float* wts, int top, int E,
                        const void* h, const void* shared, bool f32, hipStream_t s);
 
-// Softmax router (router.hip): s = softmax(logits[T, n]); the `top` largest s + correction are chosen (ties: the
-// lower index); ids[T, top] = min(index, E), wts[T, top] = s * scale. groups > 1: only outputs of the `keep`
+// Router (router.hip): s = softmax(logits[T, n]) or the sigmoid of each (rows of stride ld); the `top` largest
+// s + correction are chosen (ties: the lower index; correction null: the largest logits); ids[T, top] = min(index, E), wts[T, top] = s * scale. groups > 1: only outputs of the `keep`
 // groups (of n / groups neighbours) with the largest s + correction can be chosen; renorm: the chosen s are
 // divided by their sum + 1e-20 first.
 int route_topk_max_outputs();
-void launch_route_topk(int* ids, float* wts, const float* logits, const float* correction, int T, int n, int top,
-                       float scale, int E, int groups, int keep, bool renorm, hipStream_t s);
+void launch_route_topk(int* ids, float* wts, const float* logits, long ld, const float* correction, int T, int n,
+                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s);
 
 // Window attention on a paged cache [blocks, block_size, kv_heads * dim | kv_heads * vdim] (window_attention.hip).
 // attn_prepare: per row of proj = [q | k | v | ...]: optional RMS norm of q and k (norm_mode 0: none; 1: over the
 // whole projection, weights per element; 2: per head - and map - of `dim` elements, one weight of `dim` elements),
-// rotate-half rotation of the first 2 * nfreq dims per head, optional per-head unit-rms values; q in place, k / v
+// rotate-half rotation of the first 2 * nfreq dims per head (cos and sin times amp; norm_mode 3: every rotated head
+// divided by its root mean square), optional per-head unit-rms values; q in place, k / v
 // into cache row slots[t] (>= 0). `maps` query / key maps per head (rows hold heads * maps * dim query and
 // kv_heads * maps * dim key elements). cache null: the rows are [q | ...] and only q is prepared.
 void launch_attn_prepare(void* proj, long ld, void* cache, const long* positions, const long* slots,
                          const float* inv_freq, int nfreq, int T, int heads, int kv_heads, int maps, int dim, int vdim,
-                         const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, bool f32,
-                         hipStream_t s);
+                         const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, float amp,
+                         bool f32, hipStream_t s);
 // Sequences seq0 .. seq1-1 of the step, `tq` tokens per workgroup: keys 0 <= pos - j < window (0: all) or
 // j < keep, scores q . k * scale, through softcap * tanh(. / softcap) when softcap > 0,
 // weights exp(s_j) / (sink + sum exp) with sink = exp(sink_w[h]) (1 when sink_w is null),
-// head output times sigmoid(proj[t, gate_off + h]) (gate_off >= 0) and
+// head output times sigmoid(proj[t, gate_off + h]) (gate_off >= 0; channel_gate: element e of the concatenated
+// heads times sigmoid(proj[t, gate_off + e])) and
 // out_scale into out[t * out_ld + h * vdim ..]. maps = 2 (differential attention): queries and keys hold
 // [map 1 | map 2] per head; the head output is o = a1 - lam a2, o / sqrt(mean(o^2) + eps) * post.
 int window_attention_max_vdim();
@@ -91,7 +94,8 @@ void launch_window_attention(void* out, long out_ld, const void* proj, long proj
                              const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                              int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off,
                              float scale, int window, bool sink, float out_scale, int maps, float lam, float post,
-                             float eps, int keep, float softcap, const float* sink_w, bool f32, hipStream_t s);
+                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, bool f32,
+                             hipStream_t s);
 
 // bf16 on the matrix cores (window_attention_mfma.hip): 64 (token, head) rows of one key/value head per
 // workgroup, 32-key tiles. nparts > 1 (rows of one token each, rows_bound of them from batch row row_base on):
@@ -105,7 +109,7 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
                                   int vdim, int gate_off, float scale, int window, bool sink, float out_scale,
                                   int nparts, int part_keys, float* ws_acc, float* ws_ml, int row_base, int maps,
                                   float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                                  hipStream_t s);
+                                  bool channel_gate, hipStream_t s);
 
 // Delta-rule recurrences over state slots (delta_scan.hip). scratch: fp32, T * (2 * kv_heads * dim +
 // 2 * heads * vdim + 2 * heads) floats for the gated rule, T * 7 * heads * dim for the generalized one.
@@ -135,7 +139,8 @@ void launch_wkv_step(void* out, float* S, const void* proj, long T, const void* 
                      const float* w0, const float* u, const float* norm_w, const int* seq_cu, const int* seq_ctx,
                      const int* seq_state, int nseq, int heads, int dim, float eps, bool f32, hipStream_t s);
 // kind 0: tanh; 1: c0 z^2 + z/2 (z > 0), c1 (exp(z) - 1 - z) + z/2 (z <= 0); 2: max(z, 0)^2;
-// 3: x rows = [gate | up] of `cols` each, out = silu(gate) * up.
+// 3: x rows = [gate | up] of `cols` each, out = silu(gate) * up; 4: the same with the gate clamped at c0 (act 3 of
+// the expert GEMMs).
 void launch_activation(void* out, long out_ld, const void* x, long x_ld, int rows, int cols, int kind, float c0,
                        float c1, bool f32, hipStream_t s);
 
@@ -163,5 +168,28 @@ void launch_mlstm(void* out, float* S, float* N, float* M, const void* proj, lon
                   const float* b_if, const float* norm_w, const int* seq_cu, const int* seq_ctx, const int* seq_state,
                   int nseq, int T, float* scratch, int heads, int dim, int vdim, float cap, float eps,
                   bool one_row_seqs, bool f32, hipStream_t s);
+
+// Residual streams (streams.hip): src fp32 [T, S, H] (one_row: [T, H], all streams equal to it), coef =
+// [M (S x S, from x to) | p1 | p2 | c]: x_t = sum_s M[s, t] src_s + p1[t] y1 + p2[t] y2; out = norm(sum_t c[t] x_t) * w;
+// dst (may be src or null) = x. y2: a row, or (y2 null, ye not) sum_j wts[t, j] ye[pair_slot[t top + j]] (wts null:
+// ones) + sigmoid(gate[t * gate_ld]) * shared (gate null: one).
+int stream_update_max_streams();
+int stream_update_max_width();
+void launch_stream_update(void* out, float* dst, const float* src, bool one_row, const float* coef, int S,
+                          const float* w, int T, int H, float eps, const void* y1, const void* y2, const void* ye,
+                          const int* pair_slot, const float* wts, int top, const void* shared, const float* gate,
+                          long gate_ld, bool f32, hipStream_t s);
+
+// Lightning attention over state slots S [slots, heads, dim, vdim] (lightning.hip): proj rows = [q | k | v | gate | ..];
+// powers [heads, 65] = decay^0 .. decay^64; sequences 0 .. npf-1 are prompt portions (pf_rows rows in all, first in
+// the batch), the others bring one row each. scratch: T * heads * vdim floats, and without `mfma` another
+// pf_rows * heads * (2 dim + vdim).
+int lightning_max_dim();
+int lightning_powers();
+bool lightning_mfma_ok(int dim, int vdim, long ld, long offset);
+void launch_lightning(void* out, long out_ld, float* S, const void* proj, long ld, const float* powers,
+                      const float* norm_w, const int* seq_cu, const int* seq_ctx, const int* seq_state, int nseq,
+                      int npf, int T, int pf_rows, float* scratch, int heads, int dim, int vdim, float eps,
+                      float out_scale, bool mfma, bool f32, hipStream_t s);
 
 }  // namespace hipserve

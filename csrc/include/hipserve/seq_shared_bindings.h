@@ -47,7 +47,8 @@ inline void moe_align(const at::Tensor& ids, int64_t E, int64_t tile, at::Tensor
 }
 
 inline void expert_gemm(at::Tensor& out, const at::Tensor& x, const at::Tensor& w, const at::Tensor& slots,
-                        const at::Tensor& tile_expert, int64_t tile, int64_t gather_k, int64_t act) {
+                        const at::Tensor& tile_expert, int64_t tile, int64_t gather_k, int64_t act,
+                        const c10::optional<at::Tensor>& row_scale, double limit) {
   auto i32 = [](const at::Tensor& t) { return t.scalar_type() == at::kInt && t.is_contiguous(); };
   TORCH_CHECK(x.is_cuda() && out.is_contiguous() && w.is_contiguous() && i32(slots) && i32(tile_expert));
   TORCH_CHECK(x.scalar_type() == at::kFloat || x.scalar_type() == at::kBFloat16, "expert_gemm: bf16 or fp32 activations");
@@ -55,14 +56,31 @@ inline void expert_gemm(at::Tensor& out, const at::Tensor& x, const at::Tensor& 
   TORCH_CHECK(out.scalar_type() == x.scalar_type() && w.scalar_type() == x.scalar_type());
   TORCH_CHECK(w.dim() == 3 && x.dim() == 2 && x.stride(1) == 1 && out.dim() == 2);
   const long N = w.size(1), K = w.size(2), cap = slots.numel();
-  TORCH_CHECK(act >= 0 && act <= 2 && (act != 2 || N % 2 == 0), "expert_gemm: act 0 (none), 1 (relu^2), 2 (silu gate)");
-  TORCH_CHECK(x.size(1) == K && out.size(1) == (act == 2 ? N / 2 : N) && out.size(0) >= cap);
+  TORCH_CHECK(act >= 0 && act <= 3 && (act < 2 || N % 2 == 0),
+              "expert_gemm: act 0 (none), 1 (relu^2), 2 (silu gate), 3 (clamped gate)");
+  if (row_scale.has_value()) {
+    CHECK_F32(*row_scale);   // one number per (token, choice) pair: the slot table holds pair indices
+    TORCH_CHECK(gather_k > 0 && row_scale->numel() >= x.size(0) * gather_k, "expert_gemm: a scale per pair");
+  }
+  TORCH_CHECK(x.size(1) == K && out.size(1) == (act >= 2 ? N / 2 : N) && out.size(0) >= cap);
   TORCH_CHECK(tile % 32 == 0 && cap % tile == 0 && tile_expert.numel() * tile >= cap, "tiles of a multiple of 32 slots");
   TORCH_CHECK(gather_k > 0 || x.size(0) >= cap, "ungathered x needs one row per slot");
   c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
   hipserve::launch_expert_gemm(out.data_ptr(), x.data_ptr(), x.stride(0), w.data_ptr(), slots.data_ptr<int>(),
-                               tile_expert.data_ptr<int>(), cap / tile, tile, gather_k, N, K, act, w.size(0), f32,
+                               tile_expert.data_ptr<int>(), cap / tile, tile, gather_k, N, K, act, w.size(0),
+                               (const float*)opt_ptr(row_scale), (float)limit, f32,
                                c10::hip::getCurrentHIPStreamMasqueradingAsCUDA().stream());
+}
+
+inline void def_moe_ops(torch::Library& m) {
+  m.def("moe_align(Tensor ids, int E, int tile, Tensor(a!) slots, Tensor(b!) tile_expert, Tensor(c!) pair_slot) -> ()");
+  m.def("expert_gemm(Tensor(a!) out, Tensor x, Tensor w, Tensor slots, Tensor tile_expert, int tile, int gather_k, "
+        "int act, Tensor? row_scale=None, float limit=0.0) -> ()");
+}
+
+inline void impl_moe_ops(torch::Library& m) {
+  m.impl("moe_align", &moe_align);
+  m.impl("expert_gemm", &expert_gemm);
 }
 
 }  // namespace hipserve_shared

@@ -8,11 +8,11 @@ namespace hipserve_shared {
 inline void attn_prepare(at::Tensor& proj, const c10::optional<at::Tensor>& cache, const at::Tensor& positions,
                   const at::Tensor& slots, const at::Tensor& inv_freq, int64_t heads, int64_t kv_heads, int64_t maps,
                   int64_t dim, int64_t vdim, const c10::optional<at::Tensor>& q_norm,
-                  const c10::optional<at::Tensor>& k_norm, int64_t norm_mode, bool v_norm, double eps) {
+                  const c10::optional<at::Tensor>& k_norm, int64_t norm_mode, bool v_norm, double eps, double amp) {
   CHECK_DEV(proj); CHECK_F32(inv_freq);
   const bool f32 = is_f32(proj, "attn_prepare");
   TORCH_CHECK(heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 1 && vdim >= 1 && (maps == 1 || maps == 2));
-  TORCH_CHECK(norm_mode >= 0 && norm_mode <= 2 && (heads + kv_heads) * maps <= 8192);
+  TORCH_CHECK(norm_mode >= 0 && norm_mode <= 3 && (heads + kv_heads) * maps <= 8192);
   const long T = proj.size(0), nq = heads * maps * dim, nk = kv_heads * maps * dim, nv = kv_heads * vdim;
   const bool own_kv = cache.has_value();
   TORCH_CHECK(rows2d(proj) && proj.size(1) >= nq + (own_kv ? nk + nv : 0));
@@ -23,7 +23,7 @@ inline void attn_prepare(at::Tensor& proj, const c10::optional<at::Tensor>& cach
   TORCH_CHECK(positions.scalar_type() == at::kLong && slots.scalar_type() == at::kLong && positions.numel() >= T &&
               slots.numel() >= T && positions.is_contiguous() && slots.is_contiguous());
   TORCH_CHECK(2 * inv_freq.numel() <= dim, "rotated dims exceed the head size");
-  TORCH_CHECK((norm_mode != 0) == q_norm.has_value() && (!own_kv || q_norm.has_value() == k_norm.has_value()));
+  TORCH_CHECK((norm_mode == 1 || norm_mode == 2) == q_norm.has_value() && (!own_kv || q_norm.has_value() == k_norm.has_value()));
   if (q_norm.has_value()) {
     CHECK_F32(*q_norm);
     TORCH_CHECK(q_norm->numel() == (norm_mode == 2 ? dim : nq));
@@ -36,7 +36,7 @@ inline void attn_prepare(at::Tensor& proj, const c10::optional<at::Tensor>& cach
   hipserve::launch_attn_prepare(proj.data_ptr(), proj.stride(0), own_kv ? cache->data_ptr() : nullptr,
                                 positions.data_ptr<long>(), slots.data_ptr<long>(), inv_freq.data_ptr<float>(),
                                 inv_freq.numel(), T, heads, kv_heads, maps, dim, vdim, (const float*)opt_ptr(q_norm),
-                                own_kv ? (const float*)opt_ptr(k_norm) : nullptr, norm_mode, v_norm, (float)eps, f32,
+                                own_kv ? (const float*)opt_ptr(k_norm) : nullptr, norm_mode, v_norm, (float)eps, (float)amp, f32,
                                 cur_stream());
 }
 
@@ -45,7 +45,7 @@ inline void window_attention(at::Tensor& out, const at::Tensor& proj, const at::
                       int64_t rows_bound, int64_t tq, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
                       int64_t gate_off, double scale, int64_t window, bool sink, double out_scale, int64_t maps,
                       double lam, double post, double eps, int64_t keep, double softcap,
-                      const c10::optional<at::Tensor>& sink_w) {
+                      const c10::optional<at::Tensor>& sink_w, bool channel_gate) {
   CHECK_DEV(proj); CHECK_CONTIG(cache); CHECK_I32(seq_cu); CHECK_I32(seq_ctx); CHECK_I32(seq_bt);
   const bool f32 = is_f32(proj, "window_attention");
   TORCH_CHECK(maps == 1 || maps == 2);
@@ -53,7 +53,8 @@ inline void window_attention(at::Tensor& out, const at::Tensor& proj, const at::
   TORCH_CHECK(heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 1 && vdim >= 1 &&
               vdim <= hipserve::window_attention_max_vdim() && dim <= 1024, "window_attention: head sizes");
   const long T = proj.size(0);
-  TORCH_CHECK(rows2d(proj) && proj.size(1) >= heads * maps * dim && (gate_off < 0 || proj.size(1) >= gate_off + heads));
+  TORCH_CHECK(rows2d(proj) && proj.size(1) >= heads * maps * dim && (gate_off < 0 || proj.size(1) >= gate_off + heads * (channel_gate ? vdim : 1)) &&
+              (!channel_gate || (gate_off >= 0 && maps == 1)));
   TORCH_CHECK(rows2d(out) && out.size(0) == T && out.size(1) == heads * vdim);
   TORCH_CHECK(cache.dim() == 3 && cache.size(2) == kv_heads * (maps * dim + vdim));
   const long nseq = seq_ctx.numel();
@@ -70,8 +71,8 @@ inline void window_attention(at::Tensor& out, const at::Tensor& proj, const at::
                                     cache.size(1), seq_cu.data_ptr<int>(), seq_ctx.data_ptr<int>(),
                                     seq_bt.data_ptr<int>(), seq_bt.size(1), seq0, seq1, rows_bound, tq, heads, kv_heads,
                                     dim, vdim, gate_off, (float)scale, window, sink, (float)out_scale, maps, (float)lam,
-                                    (float)post, (float)eps, keep, (float)softcap, (const float*)opt_ptr(sink_w), f32,
-                                    cur_stream());
+                                    (float)post, (float)eps, keep, (float)softcap, (const float*)opt_ptr(sink_w),
+                                    channel_gate, f32, cur_stream());
 }
 
 inline bool window_attention_mfma_ok(int64_t dim, int64_t vdim, int64_t out_ld, int64_t out_off, int64_t maps) {
@@ -85,13 +86,14 @@ inline void window_attention_mfma(at::Tensor& out, const at::Tensor& proj, const
                            int64_t part_keys, const c10::optional<at::Tensor>& ws_acc,
                            const c10::optional<at::Tensor>& ws_ml, int64_t row_base, int64_t maps, double lam,
                            double post, double eps, int64_t keep, double softcap,
-                           const c10::optional<at::Tensor>& sink_w) {
+                           const c10::optional<at::Tensor>& sink_w, bool channel_gate) {
   CHECK_DEV(proj); CHECK_CONTIG(cache); CHECK_I32(seq_cu); CHECK_I32(seq_ctx); CHECK_I32(seq_bt);
   TORCH_CHECK(proj.scalar_type() == at::kBFloat16 && out.scalar_type() == at::kBFloat16 &&
               cache.scalar_type() == at::kBFloat16, "window_attention_mfma: bf16 only");
   TORCH_CHECK(heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0);
   const long T = proj.size(0);
-  TORCH_CHECK(rows2d(proj) && proj.size(1) >= heads * maps * dim && (gate_off < 0 || proj.size(1) >= gate_off + heads));
+  TORCH_CHECK(rows2d(proj) && proj.size(1) >= heads * maps * dim && (gate_off < 0 || proj.size(1) >= gate_off + heads * (channel_gate ? vdim : 1)) &&
+              (!channel_gate || (gate_off >= 0 && maps == 1)));
   TORCH_CHECK(rows2d(out) && out.size(0) == T && out.size(1) == heads * vdim);
   TORCH_CHECK(hipserve::window_attention_mfma_ok(dim, vdim, out.stride(0), out.storage_offset(), maps),
               "window_attention_mfma: unsupported head sizes or output alignment");
@@ -122,33 +124,37 @@ inline void window_attention_mfma(at::Tensor& out, const at::Tensor& proj, const
                                          rows_bound, heads, kv_heads, dim, vdim, gate_off, (float)scale, window, sink,
                                          (float)out_scale, nparts, part_keys, wa, wm, row_base, maps, (float)lam,
                                          (float)post, (float)eps, keep, (float)softcap, (const float*)opt_ptr(sink_w),
-                                         cur_stream());
+                                         channel_gate, cur_stream());
 }
 
 inline void activation(at::Tensor& out, const at::Tensor& x, int64_t kind, double c0, double c1) {
   CHECK_DEV(x);
   const bool f32 = is_f32(x, "activation");
-  TORCH_CHECK(kind >= 0 && kind <= 3, "activation: 0 = tanh, 1 = xielu, 2 = relu2, 3 = silu_mul");
+  TORCH_CHECK(kind >= 0 && kind <= 4, "activation: 0 = tanh, 1 = xielu, 2 = relu2, 3 = silu_mul, 4 = clamped_glu");
   TORCH_CHECK(out.scalar_type() == x.scalar_type() && rows2d(x) && rows2d(out) && out.size(0) == x.size(0));
-  TORCH_CHECK(kind == 3 ? (x.size(1) == 2 * out.size(1) && out.data_ptr() != x.data_ptr()) : out.size(1) == x.size(1));
+  TORCH_CHECK(kind >= 3 ? (x.size(1) == 2 * out.size(1) && out.data_ptr() != x.data_ptr()) : out.size(1) == x.size(1));
   c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
   hipserve::launch_activation(out.data_ptr(), out.stride(0), x.data_ptr(), x.stride(0), x.size(0), out.size(1), kind,
                               (float)c0, (float)c1, f32, cur_stream());
 }
 
-inline void route_topk(at::Tensor& ids, at::Tensor& wts, const at::Tensor& logits, const at::Tensor& correction, int64_t top,
-                double scale, int64_t E, int64_t groups, int64_t keep, bool renorm) {
-  CHECK_DEV(logits); CHECK_F32(logits); CHECK_F32(correction); CHECK_F32(wts); CHECK_I32(ids);
-  TORCH_CHECK(logits.dim() == 2);
+inline void route_topk(at::Tensor& ids, at::Tensor& wts, const at::Tensor& logits, const c10::optional<at::Tensor>& correction,
+                int64_t top, double scale, int64_t E, int64_t groups, int64_t keep, bool renorm, bool sigmoid) {
+  CHECK_DEV(logits); CHECK_F32(wts); CHECK_I32(ids);
+  TORCH_CHECK(logits.scalar_type() == at::kFloat && rows2d(logits), "route_topk: fp32 logits");
   const long T = logits.size(0), n = logits.size(1);
-  TORCH_CHECK(n >= 1 && n <= hipserve::route_topk_max_outputs() && correction.numel() == n && top >= 1 && top <= n);
+  TORCH_CHECK(n >= 1 && n <= hipserve::route_topk_max_outputs() && top >= 1 && top <= n);
+  if (correction.has_value()) {
+    CHECK_F32(*correction);
+    TORCH_CHECK(correction->numel() == n, "route_topk: a correction per output");
+  }
   TORCH_CHECK(ids.numel() == T * top && wts.numel() == T * top && E >= 0 && E <= n);
   TORCH_CHECK(groups >= 1 && groups <= 64 && n % groups == 0 && keep >= 1 && keep <= groups &&
               (groups == 1 || keep * (n / groups) >= top), "route_topk: groups of equal size that can hold the choice");
   c10::hip::HIPGuardMasqueradingAsCUDA g(logits.device());
-  hipserve::launch_route_topk(ids.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(),
-                              correction.data_ptr<float>(), T, n, top, (float)scale, E, groups, keep, renorm,
-                              cur_stream());
+  hipserve::launch_route_topk(ids.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(), logits.stride(0),
+                              (const float*)opt_ptr(correction), T, n, top, (float)scale, E, groups, keep, renorm,
+                              sigmoid, cur_stream());
 }
 
 inline void polynorm(at::Tensor& out, const at::Tensor& x, const at::Tensor& coef, double eps) {
@@ -170,6 +176,36 @@ inline void gate_mul(at::Tensor& out, const at::Tensor& x, const at::Tensor& gat
               "gate_mul: out and gate [T, heads * d] for x [heads, T, d]");
   c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
   hipserve::launch_gate_mul(out.data_ptr(), x.data_ptr(), gate.data_ptr(), gate.stride(0), T, heads, d, f32, cur_stream());
+}
+
+// The ops above and the experts', as every library with window attention registers them.
+inline void def_window_ops(torch::Library& m) {
+  m.def("attn_prepare(Tensor(a!) proj, Tensor(b!)? cache, Tensor positions, Tensor slots, Tensor inv_freq, int heads, "
+        "int kv_heads, int maps, int dim, int vdim, Tensor? q_norm, Tensor? k_norm, int norm_mode, bool v_norm, "
+        "float eps, float amp=1.0) -> ()");
+  m.def("window_attention(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
+        "int seq0, int seq1, int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, "
+        "float scale, int window, bool sink, float out_scale, int maps, float lam, float post, float eps, int keep, "
+        "float softcap, Tensor? sink_w, bool channel_gate=False) -> ()");
+  m.def("window_attention_mfma(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
+        "int seq0, int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, "
+        "int window, bool sink, float out_scale, int nparts, int part_keys, Tensor(b!)? ws_acc, Tensor(c!)? ws_ml, "
+        "int row_base, int maps, float lam, float post, float eps, int keep, float softcap, Tensor? sink_w, "
+        "bool channel_gate=False) -> ()");
+  m.def("window_attention_mfma_ok(int dim, int vdim, int out_ld, int out_off, int maps) -> bool", &window_attention_mfma_ok);
+  m.def("activation(Tensor(a!) out, Tensor x, int kind, float c0, float c1) -> ()");
+  m.def("route_topk(Tensor(a!) ids, Tensor(b!) wts, Tensor logits, Tensor? correction, int top, float scale, int E, "
+        "int groups, int keep, bool renorm, bool sigmoid=False) -> ()");
+  def_moe_ops(m);
+}
+
+inline void impl_window_ops(torch::Library& m) {
+  m.impl("attn_prepare", &attn_prepare);
+  m.impl("window_attention", &window_attention);
+  m.impl("window_attention_mfma", &window_attention_mfma);
+  m.impl("activation", &activation);
+  m.impl("route_topk", &route_topk);
+  impl_moe_ops(m);
 }
 
 }  // namespace hipserve_shared

@@ -40,6 +40,7 @@
 //                 act[m, 64 t + 16 rg + 4 (l >> 4) + j] = silu(gate) * up in registers
 //   PW_EPI_GEGLU  as GLU with tanh-GELU (Gemma)
 //   PW_EPI_RELU2  C = bf16(max(acc, 0)^2): the table-routed experts' squared ReLU
+//   PW_EPI_CGLU   as GLU with the clamped gate g sigmoid(1.702 g) (u + 1) and a scale per gathered row
 #include "hipserve/common.h"
 #include "hipserve/kernels.h"
 
@@ -262,18 +263,29 @@ __global__ __launch_bounds__(PW_T) __attribute__((amdgpu_waves_per_eu(1, 1))) vo
     asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 7\n\ts_nop 7" ::: "memory");  // last MFMA -> VALU reads
     const int t = cur.t, mb = cur.m0 + wm * 128 + fr;
     if (t < ntiles) {
-      if constexpr (EPI == PW_EPI_GLU || EPI == PW_EPI_GEGLU) {
+      if constexpr (EPI == PW_EPI_GLU || EPI == PW_EPI_GEGLU || EPI == PW_EPI_CGLU) {
         const int I = N >> 1;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           const int m = mb + 16 * i;
           if (m >= M) continue;
+          float rs = 1.f;
+          if constexpr (EPI == PW_EPI_CGLU) {
+            const int p = grp.gather_slots[m];
+            if (grp.row_scale != nullptr && p >= 0) rs = grp.row_scale[p];
+          }
 #pragma unroll
           for (int rg = 0; rg < 4; ++rg) {
             const int c = t * 64 + rg * 16 + 4 * fq;
             unsigned short o[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
+              if constexpr (EPI == PW_EPI_CGLU) {
+                const float g = fminf(acc[rg][i][j] * rs, grp.limit);
+                const float u = fminf(fmaxf(acc[rg + 4][i][j] * rs, -grp.limit), grp.limit);
+                o[j] = f32_to_bf16(g / (1.f + __expf(-1.702f * g)) * (u + 1.f));
+                continue;
+              }
               const unsigned short g = f32_to_bf16(acc[rg][i][j]), u = f32_to_bf16(acc[rg + 4][i][j]);
               o[j] = EPI == PW_EPI_GEGLU ? gelu_mul1(g, u) : silu_mul1(g, u);
             }
@@ -336,7 +348,8 @@ bool launch_prefill_gemm_packed(int epi, void* C, long ldc, const void* X, long 
   // (the gather form always runs rw = 4, PW_LAUNCH1: any rw knob value is accepted)
   if (gather && (grp.gather_k < 1 || (long)grp.x_rows * ldx * 2 >= (1L << 31) - 4096)) return false;
   if (M < 1 || N < 1 || K < 256 || K % 256 || (wm != 1 && wm != 2) || (rw != 2 && rw != 4 && rw != 5)) return false;
-  const bool glu = epi == PW_EPI_GLU || epi == PW_EPI_GEGLU;
+  const bool glu = epi == PW_EPI_GLU || epi == PW_EPI_GEGLU || epi == PW_EPI_CGLU;
+  if (epi == PW_EPI_CGLU && !gather) return false;
   if (glu && (N % 128 || bias != nullptr)) return false;
   if (epi == PW_EPI_ADD && bias != nullptr) return false;
   // 32-bit buffer offsets: the weight stream of one tile and one workgroup's X rows
@@ -376,6 +389,13 @@ bool launch_prefill_gemm_packed(int epi, void* C, long ldc, const void* X, long 
     else                                                                                                     \
       pgw_kernel<WM_, E_, false, 4, true><<<grid, PW_T, 0, s>>>(x, ldx, w, c, ldc, M, N, K, tiles_m, tiles_n, b, grp); \
   } while (0)
+  if (epi == PW_EPI_CGLU) {   // instantiated in the gather form only
+    if (wm == 1)
+      pgw_kernel<1, PW_EPI_CGLU, true, 4, false, true><<<grid, PW_T, 0, s>>>(x, ldx, w, c, ldc, M, N, K, tiles_m, tiles_n, b, grp);
+    else
+      pgw_kernel<2, PW_EPI_CGLU, true, 4, false, true><<<grid, PW_T, 0, s>>>(x, ldx, w, c, ldc, M, N, K, tiles_m, tiles_n, b, grp);
+    return true;
+  }
 #define PW_EPIS(WM_)                                          \
   switch (epi) {                                              \
     case PW_EPI_STORE: PW_LAUNCH(WM_, PW_EPI_STORE); return true; \

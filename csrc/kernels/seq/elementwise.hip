@@ -1,6 +1,6 @@
 // Elementwise and per-row activations of the layer-list decoders' feed-forwards and output gates
 // (bf16 or fp32 rows, fp32 arithmetic):
-//   activation  tanh, xIELU, squared ReLU, SiLU gate ([gate | up] rows)
+//   activation  tanh, xIELU, squared ReLU, SiLU gate and clamped gate ([gate | up] rows)
 //   polynorm    a N(z) + b N(z^2) + c N(z^3) + e per row, N(u) = u / sqrt(mean(u^2) + eps): one workgroup
 //               per row keeps its elements in registers between the three sums of powers and the output
 //   gate_mul    out[t, h * d + j] = x[h, t, j] * sigmoid(gate[t, h * d + j]): the heads of a head-major
@@ -22,6 +22,7 @@ __global__ __launch_bounds__(256) void activation_kernel(T* __restrict__ out, lo
   if (kind == 0) r = tanhf(z);
   else if (kind == 2) { r = fmaxf(z, 0.f); r *= r; }
   else if (kind == 3) r = z * sigmoid_f(z) * ldf<T>(x, t * x_ld + cols + c);   // x rows = [gate | up]
+  else if (kind == 4) r = clamped_glu_f(z, ldf<T>(x, t * x_ld + cols + c), c0);
   else r = z > 0.f ? c0 * z * z + 0.5f * z : c1 * (expm1f(z) - z) + 0.5f * z;
   stf<T>(out, t * out_ld + c, r);
 }
@@ -35,7 +36,7 @@ __global__ __launch_bounds__(256) void activation_vec_kernel(unsigned short* __r
   if (c >= cols8) return;
   const u16x8 z8 = *reinterpret_cast<const u16x8*>(x + t * x_ld + 8 * c);
   u16x8 u8 = z8;
-  if (kind == 3) u8 = *reinterpret_cast<const u16x8*>(x + t * x_ld + 8 * (cols8 + c));
+  if (kind >= 3) u8 = *reinterpret_cast<const u16x8*>(x + t * x_ld + 8 * (cols8 + c));
   u16x8 r8;
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
@@ -44,6 +45,7 @@ __global__ __launch_bounds__(256) void activation_vec_kernel(unsigned short* __r
     if (kind == 0) r = tanhf(z);
     else if (kind == 2) { r = fmaxf(z, 0.f); r *= r; }
     else if (kind == 3) r = z * sigmoid_f(z) * bf16_to_f32(u8[e]);
+    else if (kind == 4) r = clamped_glu_f(z, bf16_to_f32(u8[e]), c0);
     else r = z > 0.f ? c0 * z * z + 0.5f * z : c1 * (expm1f(z) - z) + 0.5f * z;
     r8[e] = f32_to_bf16(r);
   }

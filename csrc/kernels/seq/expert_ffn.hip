@@ -3,7 +3,9 @@
 // value >= E, a bucket of pairs whose expert has no weights, is skipped too),
 // row(slot) = slots[slot] / gather_k (the token row of the pair; first GEMM) or the slot itself
 // (second GEMM) and act = none (0), squared ReLU (1) or a SiLU gate (2): W[e] = [gate rows; up rows], N / 2 each,
-// and out[slot, c] = silu(gate_c . x) * (up_c . x) has N / 2 columns (a thread / lane holds a column's pair). Any N and K: edges are bounds-checked. A workgroup
+// and out[slot, c] = silu(gate_c . x) * (up_c . x) has N / 2 columns (a thread / lane holds a column's pair); act 3:
+// the same with g sigmoid(1.702 g) (u + 1), both clamped at `limit`. row_scale: every product of a pair's row is
+// multiplied by row_scale[pair] first (the pair's weight on its input: the products are linear in it). Any N and K: edges are bounds-checked. A workgroup
 // computes a [32 slots x 64 columns] block, x and W staged through LDS in K-chunks of 32, fp32
 // accumulation; bf16 and fp32 element types.
 #include "seq_common.h"
@@ -18,18 +20,21 @@ template <typename T>
 __global__ __launch_bounds__(256) void expert_gemm_kernel(T* __restrict__ out, const T* __restrict__ x, long x_ld,
                                                           const T* __restrict__ w, const int* __restrict__ slots,
                                                           const int* __restrict__ tile_expert, int tile, int gather_k,
-                                                          int N, int K, int act, int E) {
+                                                          int N, int K, int act, int E,
+                                                          const float* __restrict__ row_scale, float limit) {
+  __shared__ float xscale[kTM];
   __shared__ float xs[kTM][kTK + 1], ws[kTN][kTK + 1];
   __shared__ long xrow[kTM];
   const int e = tile_expert[(blockIdx.y * kTM) / tile];
   if (e < 0 || e >= E) return;
   const int tid = threadIdx.x;
-  const bool glu = act == 2;
+  const bool glu = act >= 2;
   const int No = glu ? N / 2 : N;   // output columns
   // gated: the block's 64 weight rows are 32 gate rows and the 32 up rows of the same output columns
   const int slot0 = blockIdx.y * kTM, n0 = blockIdx.x * (glu ? kTN / 2 : kTN);
   if (tid < kTM) {
     const int p = slots[slot0 + tid];
+    xscale[tid] = (row_scale != nullptr && p >= 0) ? row_scale[p] : 1.f;
     xrow[tid] = p < 0 ? -1 : (gather_k > 0 ? (long)(p / gather_k) : (long)(slot0 + tid)) * x_ld;
   }
   const T* we = w + (long)e * N * K;
@@ -64,11 +69,16 @@ __global__ __launch_bounds__(256) void expert_gemm_kernel(T* __restrict__ out, c
   for (int i = 0; i < 2; ++i) {
     const int r = ty * 2 + i;
     if (xrow[r] < 0) continue;
+    const float f = xscale[r];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] *= f;
     if (glu) {
 #pragma unroll
       for (int j = 0; j < 2; ++j) {   // columns tx, tx + 16: gates in acc[.][j], ups in acc[.][j + 2]
         const int c = n0 + tx + 16 * j;
-        if (c < No) stf<T>(out, (long)(slot0 + r) * No + c, acc[i][j] * sigmoid_f(acc[i][j]) * acc[i][j + 2]);
+        const float gv = acc[i][j], uv = acc[i][j + 2];
+        if (c < No)
+          stf<T>(out, (long)(slot0 + r) * No + c, act == 3 ? clamped_glu_f(gv, uv, limit) : gv * sigmoid_f(gv) * uv);
       }
       continue;
     }
@@ -91,23 +101,25 @@ template <int ST>
 __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(
     unsigned short* __restrict__ out, const unsigned short* __restrict__ x, long x_ld,
     const unsigned short* __restrict__ w, const int* __restrict__ slots, const int* __restrict__ tile_expert,
-    int gather_k, int N, int K, int act, int E) {
+    int gather_k, int N, int K, int act, int E, const float* __restrict__ row_scale, float limit) {
   const int e = tile_expert[blockIdx.y];
   if (e < 0 || e >= E) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int slot0 = blockIdx.y * 16 * ST;
-  const bool glu = act == 2;
+  const bool glu = act >= 2;
   const int No = glu ? N / 2 : N;
   // gated: the wave's two 16-column tiles are the gate rows and the up rows of the SAME 16 output columns
   const int n0 = glu ? blockIdx.x * 64 + 16 * wave : blockIdx.x * 128 + 32 * wave;
   if (n0 >= No) return;
   const unsigned short* xr[ST];
   bool live[ST];
+  float xscale[ST];
 #pragma unroll
   for (int st = 0; st < ST; ++st) {
     const int slot = slot0 + 16 * st + c;
     const int p = slots[slot];
+    xscale[st] = (row_scale != nullptr && p >= 0) ? row_scale[p] : 1.f;
     live[st] = p >= 0;
     xr[st] = x + (p < 0 ? 0 : (gather_k > 0 ? (long)(p / gather_k) : (long)slot)) * x_ld + 8 * g;
   }
@@ -147,12 +159,17 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(
   for (int st = 0; st < ST; ++st) {
     if (!live[st]) continue;
     const long slot = slot0 + 16 * st + c;
+    acc[0][st] *= xscale[st];
+    acc[1][st] *= xscale[st];
     if (glu) {
       const int n = n0 + 4 * g;
       if (n >= No) continue;  // No % 4 == 0: the four columns are inside together
       u16x4 o;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = f32_to_bf16(acc[0][st][j] * sigmoid_f(acc[0][st][j]) * acc[1][st][j]);
+      for (int j = 0; j < 4; ++j) {
+        const float gv = acc[0][st][j], uv = acc[1][st][j];
+        o[j] = f32_to_bf16(act == 3 ? clamped_glu_f(gv, uv, limit) : gv * sigmoid_f(gv) * uv);
+      }
       *reinterpret_cast<u16x4*>(out + slot * No + n) = o;
       continue;
     }
@@ -175,25 +192,26 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(
 }  // namespace
 
 void launch_expert_gemm(void* out, const void* x, long x_ld, const void* w, const int* slots, const int* tile_expert,
-                        int ntiles_cap, int tile, int gather_k, int N, int K, int act, int E, bool f32, hipStream_t s) {
+                        int ntiles_cap, int tile, int gather_k, int N, int K, int act, int E, const float* row_scale,
+                        float limit, bool f32, hipStream_t s) {
   if (ntiles_cap <= 0) return;
-  const int No = act == 2 ? N / 2 : N;
+  const int No = act >= 2 ? N / 2 : N;
   if (!f32 && K % 8 == 0 && No % 8 == 0 && x_ld % 8 == 0 && (tile == 32 || tile == 64)) {
-    dim3 mg(act == 2 ? (No + 63) / 64 : (N + 127) / 128, ntiles_cap);
+    dim3 mg(act >= 2 ? (No + 63) / 64 : (N + 127) / 128, ntiles_cap);
     auto o = (unsigned short*)out;
     auto xi = (const unsigned short*)x, wi = (const unsigned short*)w;
-    if (tile == 32) expert_gemm_mfma_kernel<2><<<mg, 256, 0, s>>>(o, xi, x_ld, wi, slots, tile_expert, gather_k, N, K, act, E);
-    else expert_gemm_mfma_kernel<4><<<mg, 256, 0, s>>>(o, xi, x_ld, wi, slots, tile_expert, gather_k, N, K, act, E);
+    if (tile == 32) expert_gemm_mfma_kernel<2><<<mg, 256, 0, s>>>(o, xi, x_ld, wi, slots, tile_expert, gather_k, N, K, act, E, row_scale, limit);
+    else expert_gemm_mfma_kernel<4><<<mg, 256, 0, s>>>(o, xi, x_ld, wi, slots, tile_expert, gather_k, N, K, act, E, row_scale, limit);
     return;
   }
-  dim3 grid(act == 2 ? (No + kTN / 2 - 1) / (kTN / 2) : (N + kTN - 1) / kTN, (long)ntiles_cap * tile / kTM);
+  dim3 grid(act >= 2 ? (No + kTN / 2 - 1) / (kTN / 2) : (N + kTN - 1) / kTN, (long)ntiles_cap * tile / kTM);
   if (f32)
     expert_gemm_kernel<float><<<grid, 256, 0, s>>>((float*)out, (const float*)x, x_ld, (const float*)w, slots,
-                                                   tile_expert, tile, gather_k, N, K, act, E);
+                                                   tile_expert, tile, gather_k, N, K, act, E, row_scale, limit);
   else
     expert_gemm_kernel<unsigned short><<<grid, 256, 0, s>>>((unsigned short*)out, (const unsigned short*)x, x_ld,
                                                             (const unsigned short*)w, slots, tile_expert, tile,
-                                                            gather_k, N, K, act, E);
+                                                            gather_k, N, K, act, E, row_scale, limit);
 }
 
 }  // namespace hipserve

@@ -1,11 +1,12 @@
-// Softmax router with a selection correction: per token, s = softmax(logits) over all n router
-// outputs (fp32); the `top` outputs with the largest s + correction are chosen (ties: the lower
+// Router with a selection correction: per token, s = softmax(logits) over all n router outputs, or the sigmoid
+// of each (fp32); the `top` outputs with the largest s + correction are chosen (ties: the lower
 // index); wts = s * scale of the chosen ones, ids = their index, where every index >= E (an
 // expert without weights) is written as E, so the expert alignment sees them as one bucket that
 // no GEMM tile serves. One wave per token, output e on lane e % 64, slot e / 64 (n <= 256).
 // groups > 1 (at most 64): the outputs form equal groups of neighbours; a group scores the largest
 // corrected score in it (group g's on lane g), and the outputs outside the `keep` best groups (ties:
-// the lower group) cannot be chosen. renorm: the chosen scores are divided by their sum + 1e-20.
+// the lower group) cannot be chosen. Without a correction the choice is made by the logits, which have the order of
+// s but do not saturate. renorm: the chosen scores are divided by their sum + 1e-20.
 #include "seq_common.h"
 #include "hipserve/seq_kernels.h"
 
@@ -15,33 +16,35 @@ namespace {
 constexpr int kSlots = 4;
 
 __global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, float* __restrict__ wts,
-                                                         const float* __restrict__ logits,
+                                                         const float* __restrict__ logits, long ld,
                                                          const float* __restrict__ correction, int T, int n, int top,
-                                                         float scale, int E, int groups, int keep, bool renorm) {
+                                                         float scale, int E, int groups, int keep, bool renorm,
+                                                         bool sigmoid) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (t >= T) return;
   float p[kSlots], c[kSlots];
+  float z[kSlots];
   float mx = -INFINITY;
 #pragma unroll
   for (int s = 0; s < kSlots; ++s) {
     const int e = lane + 64 * s;
-    p[s] = e < n ? logits[(long)t * n + e] : -INFINITY;
-    mx = fmaxf(mx, p[s]);
+    z[s] = e < n ? logits[(long)t * ld + e] : -INFINITY;
+    mx = fmaxf(mx, z[s]);
   }
   mx = wave_max(mx);
   float sum = 0.f;
 #pragma unroll
   for (int s = 0; s < kSlots; ++s) {
-    p[s] = lane + 64 * s < n ? expf(p[s] - mx) : 0.f;
+    p[s] = lane + 64 * s < n ? (sigmoid ? sigmoid_f(z[s]) : expf(z[s] - mx)) : 0.f;
     sum += p[s];
   }
-  sum = wave_sum(sum);
+  sum = sigmoid ? 1.f : wave_sum(sum);
 #pragma unroll
   for (int s = 0; s < kSlots; ++s) {
     const int e = lane + 64 * s;
     p[s] = p[s] / sum;
-    c[s] = e < n ? p[s] + correction[e] : -INFINITY;
+    c[s] = e < n ? (correction != nullptr ? p[s] + correction[e] : z[s]) : -INFINITY;
   }
   if (groups > 1) {
     const int per = n / groups;
@@ -105,10 +108,11 @@ __global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, 
 
 int route_topk_max_outputs() { return 64 * kSlots; }
 
-void launch_route_topk(int* ids, float* wts, const float* logits, const float* correction, int T, int n, int top,
-                       float scale, int E, int groups, int keep, bool renorm, hipStream_t s) {
+void launch_route_topk(int* ids, float* wts, const float* logits, long ld, const float* correction, int T, int n,
+                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s) {
   if (T <= 0) return;
-  route_topk_kernel<<<(T + 3) / 4, 256, 0, s>>>(ids, wts, logits, correction, T, n, top, scale, E, groups, keep, renorm);
+  route_topk_kernel<<<(T + 3) / 4, 256, 0, s>>>(ids, wts, logits, ld, correction, T, n, top, scale, E, groups, keep, renorm,
+                                               sigmoid);
 }
 
 }  // namespace hipserve

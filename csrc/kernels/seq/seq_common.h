@@ -12,4 +12,11 @@ template <> HS_DEVICE void stf<float>(float* p, long i, float v) { p[i] = v; }
 
 HS_DEVICE float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
 
+// g sigmoid(1.702 g) (u + 1) of g = min(gate, limit), u = clamp(up, -limit, limit)
+HS_DEVICE float clamped_glu_f(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * sigmoid_f(1.702f * g) * (u + 1.f);
+}
+
 }  // namespace hipserve

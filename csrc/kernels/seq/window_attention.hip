@@ -1,12 +1,13 @@
 // Grouped-query attention over a sliding window on a paged cache [blocks, block_size, keys | values]
 // (all key heads of a token, then all its value heads), with an optional softmax sink and an
-// optional per-head output gate.
+// optional sigmoid output gate (one per head, or one per channel of the concatenated heads).
 //
 // attn_prepare: per token, on the merged projection row [q | k | v | ...] (biases already added):
 // the optional RMS norm of q and k (over the WHOLE projection with a weight per element, or over
 // every head of `dim` elements with one weight of `dim` elements for all heads), the
 // rotate-half rotation of the first 2 * nfreq dims of every q / k head (angle = pos * inv_freq[i],
-// fp32), the optional division of every value head by its root mean square, q written back in
+// cos and sin times amp, fp32), the optional division of every rotated q / k head by its root mean
+// square (which the rotation changes only by amp, so it is taken from the unrotated head), the optional division of every value head by its root mean square, q written back in
 // place, k and v into the cache row. Without a cache (a layer that reads another layer's keys and
 // values) the row is [q | ...] and only q is prepared.
 //
@@ -38,7 +39,7 @@ namespace {
 template <typename T, typename F>
 HS_DEVICE void rotate_heads(const T* __restrict__ src, int nheads, int dim, int nfreq, float pos,
                             const float* __restrict__ inv_freq, float inv, const float* __restrict__ hinv,
-                            const float* __restrict__ w, int wmod, int tid, F&& store) {
+                            const float* __restrict__ w, int wmod, float amp, int tid, F&& store) {
   const int per = dim - nfreq;
   for (int it = tid; it < nheads * per; it += 256) {
     const int h = it / per, i = it % per;
@@ -53,6 +54,8 @@ HS_DEVICE void rotate_heads(const T* __restrict__ src, int nheads, int dim, int 
       if (w != nullptr) b *= w[wmod > 0 ? off + nfreq : e1];
       float sn, cs;
       sincosf(pos * inv_freq[i], &sn, &cs);
+      sn *= amp;
+      cs *= amp;
       store(e0, a * cs - b * sn);
       store(e1, b * cs + a * sn);
     } else {
@@ -62,14 +65,15 @@ HS_DEVICE void rotate_heads(const T* __restrict__ src, int nheads, int dim, int 
 }
 
 // heads / kv_heads count the maps (twice the head counts for two maps per head). norm_mode 0: none, 1: over the
-// whole q (k) projection, 2: per head with one shared weight of `dim` elements. cache null: q only.
+// whole q (k) projection, 2: per head with one shared weight of `dim` elements, 3: per head after the rotation,
+// without a weight. cache null: q only.
 template <typename T>
 __global__ __launch_bounds__(256) void attn_prepare_kernel(
     T* __restrict__ proj, long ld, T* __restrict__ cache, const long* __restrict__ positions,
     const long* __restrict__ slots, const float* __restrict__ inv_freq, int nfreq, int heads, int kv_heads, int vheads,
     int dim, int vdim, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int norm_mode, bool v_norm,
-    float eps) {
-  extern __shared__ float hinv[];  // norm_mode 2: [heads + kv_heads] inverse rms per head
+    float eps, float amp) {
+  extern __shared__ float hinv[];  // norm_mode 2, 3: [heads + kv_heads] inverse rms per head
   __shared__ float scratch[16];
   const long t = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -85,27 +89,31 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
     b = block_sum(b, scratch);
     iq = 1.f / sqrtf(a / (float)nq + eps);
     ik = 1.f / sqrtf(b / (float)max(nk, 1) + eps);
-  } else if (norm_mode == 2) {
+  } else if (norm_mode >= 2) {
+    const float grow = norm_mode == 3 ? amp : 1.f;     // mode 3: the rotated pairs count as they will be
     const int nh = heads + (own_kv ? kv_heads : 0);   // the key heads follow the query heads in the row
     for (int h = wave; h < nh; h += 4) {
       float a = 0.f;
-      for (int e = lane; e < dim; e += 64) { const float v = ldf<T>(row, (long)h * dim + e); a += v * v; }
+      for (int e = lane; e < dim; e += 64) {
+        const float v = ldf<T>(row, (long)h * dim + e) * (e < 2 * nfreq ? grow : 1.f);
+        a += v * v;
+      }
       a = wave_sum(a);
       if (lane == 0) hinv[h] = 1.f / sqrtf(a / (float)dim + eps);
     }
     __syncthreads();
   }
-  const float* hq = norm_mode == 2 ? hinv : nullptr;
+  const float* hq = norm_mode >= 2 ? hinv : nullptr;
   const int wmod = norm_mode == 2 ? dim : 0;
   const float pos = (float)positions[t];
-  rotate_heads<T>(row, heads, dim, nfreq, pos, inv_freq, iq, hq, q_norm, wmod, tid,
+  rotate_heads<T>(row, heads, dim, nfreq, pos, inv_freq, iq, hq, q_norm, wmod, amp, tid,
                   [&](int e, float v) { stf<T>(row, e, v); });
   if (!own_kv) return;
   const long slot = slots[t];
   if (slot < 0) return;
   T* dst = cache + slot * (long)(nk + nv);
   rotate_heads<T>(row + nq, kv_heads, dim, nfreq, pos, inv_freq, ik, hq != nullptr ? hq + heads : nullptr, k_norm,
-                  wmod, tid, [&](int e, float v) { stf<T>(dst, e, v); });
+                  wmod, amp, tid, [&](int e, float v) { stf<T>(dst, e, v); });
   const T* vr = row + nq + nk;
   for (int g = wave; g < vheads; g += 4) {  // one wave per value head
     float inv = 1.f;
@@ -148,7 +156,7 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
     int block_size, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx, const int* __restrict__ seq_bt,
     int bt_width, int seq0, int seq1, int tq, int hc, int hchunks, int heads, int kv_heads, int dim, int vdim,
     int gate_off, float scale, int window, bool sink, float out_scale, float lam, float post, float eps, int keep,
-    float softcap, const float* __restrict__ sink_w) {
+    float softcap, const float* __restrict__ sink_w, bool channel_gate) {
   extern __shared__ float sm[];
   const int nrows = blockDim.x >> 6;
   const int qd = MAPS * dim;                       // a row's query elements
@@ -258,7 +266,8 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
   }
   if (!active) return;
   float f = out_scale;
-  if (gate_off >= 0) f *= sigmoid_f(ldf<T>(proj, (long)trow * proj_ld + gate_off + head));
+  if (gate_off >= 0 && !channel_gate) f *= sigmoid_f(ldf<T>(proj, (long)trow * proj_ld + gate_off + head));
+  const T* cg = proj + (long)trow * proj_ld + gate_off + (long)head * vdim;   // channel_gate: this head's gates
   T* dst = out + (long)trow * out_ld + (long)head * vdim;
   if constexpr (MAPS == 2) {
     const float i0 = l[0] > 0.f ? 1.f / l[0] : 0.f, i1 = l[1] > 0.f ? lam / l[1] : 0.f;
@@ -279,7 +288,7 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
 #pragma unroll
     for (int c = 0; c < kMaxCh; ++c) {
       const int e = c * kDC + lane;
-      if (c < nvc && e < vdim) stf<T>(dst, e, acc[0][c] * inv);
+      if (c < nvc && e < vdim) stf<T>(dst, e, acc[0][c] * inv * (channel_gate ? sigmoid_f(ldf<T>(cg, e)) : 1.f));
     }
   }
 }
@@ -288,18 +297,18 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
 
 void launch_attn_prepare(void* proj, long ld, void* cache, const long* positions, const long* slots,
                          const float* inv_freq, int nfreq, int T, int heads, int kv_heads, int maps, int dim, int vdim,
-                         const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, bool f32,
-                         hipStream_t s) {
+                         const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, float amp,
+                         bool f32, hipStream_t s) {
   if (T <= 0) return;
   const int qh = heads * maps, kh = kv_heads * maps;
   const size_t smem = (size_t)(qh + kh) * sizeof(float);
   if (f32)
     attn_prepare_kernel<float><<<T, 256, smem, s>>>((float*)proj, ld, (float*)cache, positions, slots, inv_freq, nfreq,
-                                                    qh, kh, kv_heads, dim, vdim, q_norm, k_norm, norm_mode, v_norm, eps);
+                                                    qh, kh, kv_heads, dim, vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp);
   else
     attn_prepare_kernel<unsigned short><<<T, 256, smem, s>>>((unsigned short*)proj, ld, (unsigned short*)cache,
                                                              positions, slots, inv_freq, nfreq, qh, kh, kv_heads, dim,
-                                                             vdim, q_norm, k_norm, norm_mode, v_norm, eps);
+                                                             vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp);
 }
 
 int window_attention_max_vdim() { return kMaxCh * kDC; }
@@ -310,7 +319,7 @@ void launch_generic(void* out, long out_ld, const void* proj, long proj_ld, cons
                     const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                     int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale,
                     int window, bool sink, float out_scale, float lam, float post, float eps, int keep, float softcap,
-                    const float* sink_w, hipStream_t s) {
+                    const float* sink_w, bool channel_gate, hipStream_t s) {
   const int group = heads / kv_heads;
   auto lds = [&](int rows) {
     return ((size_t)rows * MAPS * dim + kKT * (kDC + 1) + (size_t)rows * MAPS * kKT) * sizeof(float) +
@@ -326,7 +335,7 @@ void launch_generic(void* out, long out_ld, const void* proj, long proj_ld, cons
   window_attention_kernel<T, MAPS><<<grid, block, lds(nrows), s>>>(
       (T*)out, out_ld, (const T*)proj, proj_ld, (const T*)cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0,
       seq1, tq, hc, hchunks, heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, lam, post, eps, keep,
-      softcap, sink_w);
+      softcap, sink_w, channel_gate);
 }
 }  // namespace
 
@@ -334,12 +343,13 @@ void launch_window_attention(void* out, long out_ld, const void* proj, long proj
                              const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                              int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off,
                              float scale, int window, bool sink, float out_scale, int maps, float lam, float post,
-                             float eps, int keep, float softcap, const float* sink_w, bool f32, hipStream_t s) {
+                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, bool f32,
+                             hipStream_t s) {
   if (seq1 <= seq0 || rows_bound <= 0) return;
 #define HS_GA(T, M)                                                                                                  \
   launch_generic<T, M>(out, out_ld, proj, proj_ld, cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0, seq1,  \
                        rows_bound, tq, heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, lam, post, \
-                       eps, keep, softcap, sink_w, s)
+                       eps, keep, softcap, sink_w, channel_gate, s)
   if (f32) { if (maps == 2) HS_GA(float, 2); else HS_GA(float, 1); }
   else { if (maps == 2) HS_GA(unsigned short, 2); else HS_GA(unsigned short, 1); }
 #undef HS_GA

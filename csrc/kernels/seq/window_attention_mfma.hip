@@ -1,6 +1,6 @@
 // Window attention on the matrix cores (bf16 activations and cache), same interface as the generic
 // kernel of window_attention.hip: paged cache rows [all key heads | all value heads], sliding
-// window, optional softmax sink, optional per-head sigmoid output gate, output scale.
+// window, optional softmax sink, optional sigmoid output gate (per head or per channel), output scale.
 //
 // A workgroup (4 waves) owns 64 or 128 (token, query head) rows of ONE key/value head: consecutive
 // tokens of one sequence x the query heads of the group, so all rows share one run of keys and a
@@ -68,7 +68,7 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
     int hchunks, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, int window, bool sink,
     float out_scale, int part_keys, float* __restrict__ ws_acc, float* __restrict__ ws_ml, int row_base, int ws_rows,
     float lam, float post, float eps, bool one_row_seqs, bool qvec, int keep, float softcap,
-    const float* __restrict__ sink_w) {
+    const float* __restrict__ sink_w, bool channel_gate) {
   static_assert(!DIFF || MT % 2 == 0, "a wave's row tiles come in pairs: the two maps of the same 16 rows");
   constexpr int RT = DIFF ? MT / 2 : MT;   // distinct 16-row tiles per wave; tile mt is rows mt / kMaps, map mt % kMaps
   constexpr int kLd = KLd<KS>::v;
@@ -325,8 +325,9 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
       continue;
     }
     float f = out_scale;
-    if (gate_off >= 0) f *= sigmoid_f(bf16_to_f32(proj[trow[mt] * proj_ld + gate_off + head[mt]]));
+    if (gate_off >= 0 && !channel_gate) f *= sigmoid_f(bf16_to_f32(proj[trow[mt] * proj_ld + gate_off + head[mt]]));
     f = l_run[mt] > 0.f ? f / l_run[mt] : 0.f;
+    const unsigned short* cg = proj + trow[mt] * proj_ld + gate_off + (long)head[mt] * vdim;   // channel_gate
     unsigned short* dst = out + trow[mt] * out_ld + (long)head[mt] * vdim;
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
@@ -334,7 +335,8 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
       if (d >= vdim) continue;  // vdim % 8 == 0: the four dims are inside together
       u16x4 o;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = f32_to_bf16(acc[mt][j][e] * f);
+      for (int e = 0; e < 4; ++e)
+        o[e] = f32_to_bf16(acc[mt][j][e] * f * (channel_gate ? sigmoid_f(bf16_to_f32(cg[d + e])) : 1.f));
       *reinterpret_cast<u16x4*>(dst + d) = o;
     }
   }
@@ -345,7 +347,7 @@ constexpr int kMaxRuns = 64;
 __global__ __launch_bounds__(128) void window_attention_reduce_kernel(
     unsigned short* __restrict__ out, long out_ld, const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
     const unsigned short* __restrict__ proj, long proj_ld, int gate_off, int nparts, int heads, int ws_rows,
-    int row_base, int vdim, float out_scale) {
+    int row_base, int vdim, float out_scale, bool channel_gate) {
   __shared__ float sc[kMaxRuns];  // each run's weight e^(m_p - M) / L * gate * scale, 0 for empty runs
   const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   if (tid < 64) {  // one wave: run p on lane p
@@ -356,7 +358,7 @@ __global__ __launch_bounds__(128) void window_attention_reduce_kernel(
     const float e = m > -INFINITY ? __builtin_amdgcn_exp2f(m - M) : 0.f;  // the runs' maxima are in the log2 domain
     const float L = wave_sum(l * e);
     float f = out_scale;
-    if (gate_off >= 0) f *= sigmoid_f(bf16_to_f32(proj[(long)(row_base + r) * proj_ld + gate_off + h]));
+    if (gate_off >= 0 && !channel_gate) f *= sigmoid_f(bf16_to_f32(proj[(long)(row_base + r) * proj_ld + gate_off + h]));
     sc[tid] = L > 0.f ? e * f / L : 0.f;
   }
   __syncthreads();
@@ -364,6 +366,7 @@ __global__ __launch_bounds__(128) void window_attention_reduce_kernel(
   for (int d = tid; d < vdim; d += 128) {
     float o = 0.f;
     for (int p = 0; p < nparts; ++p) o += ws_acc[(((long)p * heads + h) * ws_rows + r) * vdim + d] * sc[p];
+    if (channel_gate) o *= sigmoid_f(bf16_to_f32(proj[trow * proj_ld + gate_off + (long)h * vdim + d]));
     out[trow * out_ld + (long)h * vdim + d] = f32_to_bf16(o);
   }
 }
@@ -417,7 +420,7 @@ void launch_mfma(unsigned short* out, long out_ld, const unsigned short* proj, l
                  int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale,
                  int window, bool sink, float out_scale, int nparts, int part_keys, float* ws_acc, float* ws_ml,
                  int row_base, float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                 hipStream_t s) {
+                 bool channel_gate, hipStream_t s) {
   const int group = heads / kv_heads;
   const int rows = kRows * (DIFF ? MT / 2 : MT);
   const int hc = min(group, rows);
@@ -431,7 +434,7 @@ void launch_mfma(unsigned short* out, long out_ld, const unsigned short* proj, l
   window_attention_mfma_kernel<KS, NV, MT, DIFF><<<grid, kThreads, 0, s>>>(
       out, out_ld, proj, proj_ld, cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0, seq1, tq, hc, hchunks,
       heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, part_keys, ws_acc, ws_ml, row_base,
-      rows_bound, lam, post, eps, one_row_seqs, qvec, keep, softcap, sink_w);
+      rows_bound, lam, post, eps, one_row_seqs, qvec, keep, softcap, sink_w, channel_gate);
   if (nparts > 1 && DIFF)
     window_attention_diff_reduce_kernel<<<dim3(rows_bound, heads), 128, 0, s>>>(
         out, out_ld, ws_acc, ws_ml, proj, proj_ld, gate_off, nparts, heads, rows_bound, row_base, vdim, out_scale, lam,
@@ -439,7 +442,7 @@ void launch_mfma(unsigned short* out, long out_ld, const unsigned short* proj, l
   else if (nparts > 1)
     window_attention_reduce_kernel<<<dim3(rows_bound, heads), 128, 0, s>>>(out, out_ld, ws_acc, ws_ml, proj, proj_ld,
                                                                          gate_off, nparts, heads, rows_bound, row_base,
-                                                                         vdim, out_scale);
+                                                                         vdim, out_scale, channel_gate);
 }
 
 }  // namespace
@@ -456,14 +459,14 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
                                   int vdim, int gate_off, float scale, int window, bool sink, float out_scale,
                                   int nparts, int part_keys, float* ws_acc, float* ws_ml, int row_base, int maps,
                                   float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                                  hipStream_t s) {
+                                  bool channel_gate, hipStream_t s) {
   if (seq1 <= seq0 || rows_bound <= 0) return;
 #define HS_WA(KS, NV, MT, DIFF)                                                                                     \
   launch_mfma<KS, NV, MT, DIFF>((unsigned short*)out, out_ld, (const unsigned short*)proj, proj_ld,                  \
                                 (const unsigned short*)cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0,    \
                                 seq1, rows_bound, heads, kv_heads, dim, vdim, gate_off, scale, window, sink,          \
                                 out_scale, nparts, part_keys, ws_acc, ws_ml, row_base, lam, post, eps, keep, softcap,  \
-                                sink_w, s)
+                                sink_w, channel_gate, s)
   // two row tiles per wave where a prompt portion brings enough rows and the accumulators fit the registers
   const int ks = (dim + 31) / 32, nv = (vdim + 15) / 16;
   const bool wide = nparts == 1 && (long)rows_bound * (heads / kv_heads) >= 128 * (long)(seq1 - seq0);

@@ -65,6 +65,7 @@ void mingru_scan(at::Tensor& y, at::Tensor& state, const at::Tensor& proj, const
 }  // namespace
 
 TORCH_LIBRARY(hipserve_seq, m) {
+  hipserve_shared::def_moe_ops(m);
   m.def("scaled_add_group_rmsnorm(Tensor(a!) out, Tensor(b!) residual, Tensor w, int groups, float eps, Tensor? mix, "
         "Tensor? ls1, Tensor? y, Tensor? pair_slot, int top, Tensor? ls2, Tensor? extra) -> ()");
   m.def("latent_prepare(Tensor(a!) cq, Tensor(b!) cache, Tensor proj, Tensor positions, Tensor slots, Tensor q_norm, "
@@ -79,17 +80,13 @@ TORCH_LIBRARY(hipserve_seq, m) {
   m.def("latent_attention_mfma_ok(int kv_rank, int rot_dim) -> bool", &latent_attention_mfma_ok);
   m.def("mingru_scan(Tensor(a!) y, Tensor(b!) state, Tensor proj, Tensor b_z, Tensor b_x, Tensor seq_cu, "
         "Tensor seq_ctx, Tensor seq_state, int max_q) -> ()");
-  m.def("moe_align(Tensor ids, int E, int tile, Tensor(a!) slots, Tensor(b!) tile_expert, Tensor(c!) pair_slot) -> ()");
-  m.def("expert_gemm(Tensor(a!) out, Tensor x, Tensor w, Tensor slots, Tensor tile_expert, int tile, int gather_k, "
-        "int act) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(hipserve_seq, CUDA, m) {
+  hipserve_shared::impl_moe_ops(m);
   m.impl("scaled_add_group_rmsnorm", &scaled_add_group_rmsnorm);
   m.impl("latent_prepare", &latent_prepare);
   m.impl("latent_attention", &latent_attention);
   m.impl("latent_attention_mfma", &latent_attention_mfma);
   m.impl("mingru_scan", &mingru_scan);
-  m.impl("moe_align", &moe_align);
-  m.impl("expert_gemm", &expert_gemm);
 }

@@ -108,6 +108,7 @@ void mlstm(at::Tensor& out, at::Tensor& S, at::Tensor& N, at::Tensor& M, const a
 }  // namespace
 
 TORCH_LIBRARY(hipserve_cell, m) {
+  def_window_ops(m);
   m.def("gated_add_norms(Tensor(a!) out1, Tensor(b!)? out2, Tensor(c!) residual, Tensor w1, Tensor? w2, float eps, "
         "Tensor? y1, Tensor? g1, Tensor? b1, Tensor? y2, Tensor? g2, Tensor? b2, Tensor? ye, Tensor? pair_slot, "
         "Tensor? wts, Tensor? shared) -> ()");
@@ -116,7 +117,6 @@ TORCH_LIBRARY(hipserve_cell, m) {
         "int vdim, float cap, float eps, bool one_row_seqs) -> ()");
   m.def("polynorm(Tensor(a!) out, Tensor x, Tensor coef, float eps) -> ()");
   m.def("gate_mul(Tensor(a!) out, Tensor x, Tensor gate) -> ()");
-  m.def("activation(Tensor(a!) out, Tensor x, int kind, float c0, float c1) -> ()");
   m.def("latent_prepare(Tensor(a!) cq, Tensor(b!) cache, Tensor proj, Tensor positions, Tensor slots, Tensor q_norm, "
         "Tensor kv_norm, Tensor inv_freq, int q_rank, int kv_rank, int rot_dim, float eps) -> ()");
   m.def("latent_attention(Tensor(a!) o_lat, Tensor q_abs, Tensor q, Tensor proj, Tensor cache, Tensor seq_cu, "
@@ -127,38 +127,15 @@ TORCH_LIBRARY(hipserve_cell, m) {
         "Tensor inv_freq, int heads, int dim, int rot_dim, int kv_rank, int gate_off, float scale, int window, "
         "int nparts, int part_keys, Tensor(c!)? ws_acc, Tensor(d!)? ws_ml, int row_base, bool fill_qc) -> ()");
   m.def("latent_attention_mfma_ok(int kv_rank, int rot_dim) -> bool", &latent_attention_mfma_ok);
-  m.def("attn_prepare(Tensor(a!) proj, Tensor(b!)? cache, Tensor positions, Tensor slots, Tensor inv_freq, int heads, "
-        "int kv_heads, int maps, int dim, int vdim, Tensor? q_norm, Tensor? k_norm, int norm_mode, bool v_norm, "
-        "float eps) -> ()");
-  m.def("window_attention(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
-        "int seq0, int seq1, int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, "
-        "float scale, int window, bool sink, float out_scale, int maps, float lam, float post, float eps, int keep, "
-        "float softcap, Tensor? sink_w) -> ()");
-  m.def("window_attention_mfma(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
-        "int seq0, int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, "
-        "int window, bool sink, float out_scale, int nparts, int part_keys, Tensor(b!)? ws_acc, Tensor(c!)? ws_ml, "
-        "int row_base, int maps, float lam, float post, float eps, int keep, float softcap, Tensor? sink_w) -> ()");
-  m.def("window_attention_mfma_ok(int dim, int vdim, int out_ld, int out_off, int maps) -> bool", &window_attention_mfma_ok);
-  m.def("route_topk(Tensor(a!) ids, Tensor(b!) wts, Tensor logits, Tensor correction, int top, float scale, int E, "
-        "int groups, int keep, bool renorm) -> ()");
-  m.def("moe_align(Tensor ids, int E, int tile, Tensor(a!) slots, Tensor(b!) tile_expert, Tensor(c!) pair_slot) -> ()");
-  m.def("expert_gemm(Tensor(a!) out, Tensor x, Tensor w, Tensor slots, Tensor tile_expert, int tile, int gather_k, "
-        "int act) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(hipserve_cell, CUDA, m) {
+  impl_window_ops(m);
   m.impl("gated_add_norms", &gated_add_norms);
   m.impl("mlstm", &mlstm);
   m.impl("polynorm", &polynorm);
   m.impl("gate_mul", &gate_mul);
-  m.impl("activation", &activation);
   m.impl("latent_prepare", &latent_prepare);
   m.impl("latent_attention", &latent_attention);
   m.impl("latent_attention_mfma", &latent_attention_mfma);
-  m.impl("attn_prepare", &attn_prepare);
-  m.impl("window_attention", &window_attention);
-  m.impl("window_attention_mfma", &window_attention_mfma);
-  m.impl("route_topk", &route_topk);
-  m.impl("moe_align", &moe_align);
-  m.impl("expert_gemm", &expert_gemm);
 }

@@ -194,27 +194,15 @@ void wkv_step(at::Tensor& out, at::Tensor& S, const at::Tensor& proj, const at::
 }  // namespace
 
 TORCH_LIBRARY(hipserve_delta, m) {
+  def_window_ops(m);
   m.def("scaled_add_group_rmsnorm(Tensor(a!) out, Tensor(b!) residual, Tensor w, int groups, float eps, Tensor? mix, "
         "Tensor? ls1, Tensor? y, Tensor? pair_slot, int top, Tensor? ls2, Tensor? extra) -> ()");
-  m.def("attn_prepare(Tensor(a!) proj, Tensor(b!)? cache, Tensor positions, Tensor slots, Tensor inv_freq, int heads, "
-        "int kv_heads, int maps, int dim, int vdim, Tensor? q_norm, Tensor? k_norm, int norm_mode, bool v_norm, "
-        "float eps) -> ()");
-  m.def("window_attention(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
-        "int seq0, int seq1, int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, "
-        "float scale, int window, bool sink, float out_scale, int maps, float lam, float post, float eps, int keep, "
-        "float softcap, Tensor? sink_w) -> ()");
-  m.def("window_attention_mfma(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
-        "int seq0, int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, "
-        "int window, bool sink, float out_scale, int nparts, int part_keys, Tensor(b!)? ws_acc, Tensor(c!)? ws_ml, "
-        "int row_base, int maps, float lam, float post, float eps, int keep, float softcap, Tensor? sink_w) -> ()");
-  m.def("window_attention_mfma_ok(int dim, int vdim, int out_ld, int out_off, int maps) -> bool", &window_attention_mfma_ok);
   m.def("gated_delta(Tensor(a!) y, Tensor(b!) S, Tensor(c!) conv_state, Tensor proj, Tensor conv_w, Tensor a_log, "
         "Tensor dt_bias, Tensor norm_w, Tensor seq_cu, Tensor seq_ctx, Tensor seq_state, Tensor(d!) scratch, "
         "int heads, int kv_heads, int dim, int vdim, int taps, float eps) -> ()");
   m.def("delta_rule(Tensor(a!) out, Tensor(b!) S, Tensor proj, Tensor wl, Tensor a_b, Tensor w0, Tensor norm_w, "
         "Tensor seq_cu, Tensor seq_ctx, Tensor seq_state, Tensor(c!) scratch, int heads, int dim, float eps, "
         "float out_scale) -> ()");
-  m.def("activation(Tensor(a!) out, Tensor x, int kind, float c0, float c1) -> ()");
   m.def("add_normed(Tensor(a!) out, Tensor(b!) residual, Tensor w, float eps, Tensor? y, Tensor? ye, Tensor? pair_slot, "
         "Tensor? ids, Tensor? wts, int E, Tensor? h, Tensor? shared) -> ()");
   m.def("token_shift(Tensor(a!) out, Tensor x, Tensor(b!) state, Tensor mu, Tensor seq_cu, Tensor seq_ctx, "
@@ -223,26 +211,15 @@ TORCH_LIBRARY(hipserve_delta, m) {
         "Tensor seq_ctx, Tensor seq_state, Tensor(c!) scratch, int heads, int dim, float eps) -> ()");
   m.def("wkv_step(Tensor(a!) out, Tensor(b!) S, Tensor proj, Tensor low, Tensor w2, Tensor w0, Tensor u, Tensor norm_w, "
         "Tensor seq_cu, Tensor seq_ctx, Tensor seq_state, int heads, int dim, float eps) -> ()");
-  m.def("route_topk(Tensor(a!) ids, Tensor(b!) wts, Tensor logits, Tensor correction, int top, float scale, int E, "
-        "int groups, int keep, bool renorm) -> ()");
-  m.def("moe_align(Tensor ids, int E, int tile, Tensor(a!) slots, Tensor(b!) tile_expert, Tensor(c!) pair_slot) -> ()");
-  m.def("expert_gemm(Tensor(a!) out, Tensor x, Tensor w, Tensor slots, Tensor tile_expert, int tile, int gather_k, "
-        "int act) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(hipserve_delta, CUDA, m) {
+  impl_window_ops(m);
   m.impl("scaled_add_group_rmsnorm", &scaled_add_group_rmsnorm);
-  m.impl("attn_prepare", &attn_prepare);
-  m.impl("window_attention", &window_attention);
-  m.impl("window_attention_mfma", &window_attention_mfma);
   m.impl("gated_delta", &gated_delta);
   m.impl("delta_rule", &delta_rule);
-  m.impl("activation", &activation);
   m.impl("add_normed", &add_normed);
   m.impl("token_shift", &token_shift);
   m.impl("wkv", &wkv);
   m.impl("wkv_step", &wkv_step);
-  m.impl("route_topk", &route_topk);
-  m.impl("moe_align", &moe_align);
-  m.impl("expert_gemm", &expert_gemm);
 }

@@ -43,7 +43,8 @@ HIP_FLAGS = [
 # differential attention, delta-rule and decayed linear-attention recurrences, softmax router and
 # activations; "cell" the parallel block with gated sublayer results, the mLSTM matrix memory, PolyNorm and
 # the gate multiply, plus the latent and window attention, router and activations that such a model also
-# runs. Kernel files shared by several libraries are compiled once and linked into each, so a model of
+# runs; "stream" the residual streams' update and lightning attention beside the window attention, router and
+# experts. Kernel files shared by several libraries are compiled once and linked into each, so a model of
 # those designs builds only what it runs.
 LIBS = {
     "core": ("_C.so", ["kernels/*.hip"], "torch_bindings.cpp"),
@@ -55,6 +56,9 @@ LIBS = {
     "cell": ("_C_cell.so", ["kernels/seq/gated_block.hip", "kernels/seq/mlstm.hip", "kernels/seq/latent_attention*.hip",
                             "kernels/seq/window_attention*.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",
                             "kernels/seq/elementwise.hip", "kernels/moe.hip"], "seq_cell_bindings.cpp"),
+    "stream": ("_C_stream.so", ["kernels/seq/streams.hip", "kernels/seq/lightning.hip", "kernels/seq/window_attention*.hip",
+                                "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip", "kernels/seq/elementwise.hip",
+                                "kernels/moe.hip"], "seq_stream_bindings.cpp"),
 }
 
 
@@ -107,7 +111,8 @@ def _compile(src, obj, cmd, want):
 
 def build_kernels(force: bool = False, jobs: int = 8, verbose: bool = False, lib: str = "core") -> str:
     """Build one kernel library of ``LIBS`` (gfx950 kernels + torch op registrations):
-    ``core`` = hipserve/_C.so, ``seq`` = hipserve/_C_seq.so, ``delta`` = hipserve/_C_delta.so, ``cell`` = hipserve/_C_cell.so."""
+    ``core`` = hipserve/_C.so, ``seq`` = hipserve/_C_seq.so, ``delta`` = hipserve/_C_delta.so, ``cell`` = hipserve/_C_cell.so,
+    ``stream`` = hipserve/_C_stream.so."""
     if not os.path.exists(HIPCC):
         raise RuntimeError(f"hipcc not found at {HIPCC}")
     so_name, patterns, bindings = LIBS[lib]
@@ -232,6 +237,7 @@ def build_all(force: bool = False, jobs: int | None = None, verbose: bool = True
     build_kernels(force=force, jobs=jobs, verbose=verbose, lib="seq")
     build_kernels(force=force, jobs=jobs, verbose=verbose, lib="delta")
     build_kernels(force=force, jobs=jobs, verbose=verbose, lib="cell")
+    build_kernels(force=force, jobs=jobs, verbose=verbose, lib="stream")
     return so, rt
 
 

@@ -13,6 +13,7 @@ from __future__ import annotations
 
 import dataclasses
 import json
+import math
 import os
 from dataclasses import dataclass, field
 
@@ -612,6 +613,35 @@ class TableMoESpec:
 
 
 @dataclass(frozen=True)
+class YarnScaling:
+    """YaRN stretching of rotary frequencies: pairs that turn fewer than ``slow`` times over the ``original``
+    context length are slowed down by ``factor``, pairs that turn more than ``fast`` times are kept, with a linear
+    ramp over the pair index in between; cos and sin grow by ``0.1 ln(factor) + 1``."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    def frequencies(self, base: float, dims: int) -> list:
+        """Angle per position of every pair i < dims / 2 (computed in double precision)."""
+        def pair_of(turns):
+            return dims * math.log(self.original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+        lo = max(math.floor(pair_of(self.fast)), 0)
+        hi = min(math.ceil(pair_of(self.slow)), dims - 1)
+        out = []
+        for i in range(dims // 2):
+            f = base ** (-2.0 * i / dims)
+            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+            out.append(f / self.factor * ramp + f * (1.0 - ramp))
+        return out
+
+    @property
+    def amplitude(self) -> float:
+        return 0.1 * math.log(self.factor) + 1.0
+
+
+@dataclass(frozen=True)
 class WindowAttentionSpec:
     """Grouped-query attention over a sliding window (``window`` keys: the token itself and
     the ``window - 1`` before it; 0 = plain causal) with rotate-half rotary positions on the
@@ -621,11 +651,14 @@ class WindowAttentionSpec:
     ``softcap`` > 0 passes the scaled scores through ``softcap * tanh(. / softcap)``,
     ``keep_first`` > 0 keeps the sequence's first ``keep_first`` tokens visible behind the window,
     ``gate`` multiplies head h's output by sigmoid of a per-head projection of the mixer input,
+    ``channel_gate`` the concatenated heads element by element by sigmoid of a projection of that size,
     ``bias`` adds biases in the q / k / v projections, ``qk_norm`` applies a weighted RMS norm
     over the WHOLE q (and k) projection before the rotation, ``head_norm`` one over every
-    query / key head with a weight of ``dim`` elements that all heads share, ``v_norm`` divides
+    query / key head with a weight of ``dim`` elements that all heads share, ``unit_qk`` divides
+    every query / key head by its root mean square AFTER the rotation (no weight), ``v_norm`` divides
     every value head by its root mean square (cached so), ``out_bias`` adds a bias in the
-    output projection.
+    output projection. ``interleaved``: the rotation pairs coordinate 2i with 2i + 1 (else i with
+    i + rot_dims / 2); ``yarn`` stretches its frequencies and its cos / sin.
 
     ``maps`` = 2 is differential attention: every query head and every key head carries two
     maps side by side ([map 1 | map 2], ``dim`` each); each map is a softmax attention of its
@@ -653,8 +686,17 @@ class WindowAttentionSpec:
     softcap: float = 0.0
     keep_first: int = 0
     sink_weights: bool = False
+    channel_gate: bool = False
+    unit_qk: bool = False
+    interleaved: bool = False
+    yarn: YarnScaling | None = None
 
     kind = "attention"
+
+    @property
+    def gate_size(self) -> int:
+        """Rows of the output gate's projection."""
+        return self.heads * self.vdim if self.channel_gate else self.heads if self.gate else 0
 
     @property
     def q_size(self) -> int:
@@ -752,6 +794,27 @@ class MLstmSpec:
 
 
 @dataclass(frozen=True)
+class LightningSpec:
+    """Linear attention with one fixed decay per head: a ``dim x vdim`` state S <- decay S + k v^T read by q,
+    with SiLU on all three projections; the concatenated heads are RMS-normed TOGETHER, weighted and gated by
+    a sigmoid of a projection of the input."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+
+    kind = "lightning"
+
+    def __post_init__(self):
+        if len(self.decay) != self.heads:
+            raise ValueError(f"{self.heads} heads but {len(self.decay)} decays")
+
+    @property
+    def out_size(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers on the same input, their outputs summed with fixed weights."""
     left: object
@@ -775,9 +838,14 @@ class DenseFFSpec:
 
 @dataclass(frozen=True)
 class RoutedMoESpec:
-    """Mixture of gated feed-forwards with a learned softmax router: the ``top`` experts with
-    the largest score + correction are chosen, weighted by their (uncorrected, not
-    renormalised) score times ``scale``. The last ``identity`` router outputs are experts
+    """Mixture of gated feed-forwards with a learned router (``score``: ``softmax`` over all router
+    outputs, or the ``sigmoid`` of each): the ``top`` experts with the largest score + correction
+    (without ``correction``: the largest score) are chosen, weighted by their (uncorrected, not
+    renormalised) score times ``scale``. ``weight_input``: the weight multiplies the expert's input
+    instead of its output. ``act``: ``silu`` experts compute silu(gate) * up, ``clamped`` ones
+    g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit) (``shared_limit``
+    for the shared expert). ``shared_gate`` multiplies the shared expert's output by the sigmoid of one
+    number per token. The last ``identity`` router outputs are experts
     without weights that return their input; ``shared_ff`` > 0 adds a gated feed-forward that
     every token runs. ``groups`` > 1: the router outputs form that many equal groups of
     neighbours, a group scores the largest corrected score in it, and only the experts of the
@@ -792,6 +860,13 @@ class RoutedMoESpec:
     groups: int = 1
     keep_groups: int = 1
     renorm: bool = False
+    score: str = "softmax"
+    correction: bool = True
+    weight_input: bool = False
+    act: str = "silu"
+    limit: float = 0.0
+    shared_limit: float = 0.0
+    shared_gate: bool = False
 
     kind = "routed_moe"
 
@@ -801,6 +876,18 @@ class HybridLayerSpec:
     mixer: object               # a mixer spec of this section
     mlp: object | None          # TableMoESpec | DenseFFSpec | None
     weights_of: int | None = None   # the layer whose weights this one uses (its own when None)
+
+
+def loop_runs(n: int, start: int, stop: int, times: int) -> list:
+    """Layer runs of ``n`` layers whose span start .. stop - 1 runs ``times`` times in a row:
+    (layer index, pass index, starts_pass) where ``starts_pass`` marks the first layer of every
+    pass of the span but the first."""
+    if stop <= start:
+        return [(i, 0, False) for i in range(n)]
+    out = [(i, 0, False) for i in range(0, start)]
+    for t in range(times):
+        out += [(i, t, t > 0 and i == start) for i in range(start, stop)]
+    return out + [(i, 0, False) for i in range(stop, n)]
 
 
 @dataclass(frozen=True)
@@ -834,12 +921,7 @@ class HybridConfig:
     def runs(self) -> list:
         """Layer runs in execution order: (layer index, pass index, starts_pass) where
         ``starts_pass`` marks the first layer of every pass of the loop but the first."""
-        a, b, n = self.loop_start, self.loop_stop, self.loop_times
-        out = [(i, 0, False) for i in range(0, a)]
-        for t in range(n if b > a else 0):
-            out += [(i, t, t > 0 and i == a) for i in range(a, b)]
-        out += [(i, 0, False) for i in range(b if b > a else a, len(self.layers))]
-        return out
+        return loop_runs(len(self.layers), self.loop_start, self.loop_stop, self.loop_times)
 
     def num_params(self) -> int:
         H, n = self.hidden_size, 2 * self.vocab_size * self.hidden_size
@@ -1184,6 +1266,106 @@ class TopezenConfig:
             bos_token_id=d.get("bos_token_id"), eos_token_id=eos)
 
 
+@dataclass(frozen=True)
+class ZinavikConfig:
+    """Zinavik: a pre-norm decoder given as a list of layers with ``streams`` residual streams
+    (static hyper-connections). For every sublayer, with its own tensors in [s], out [s], mix [from, to],
+
+        u = sum_s in[s] x_s;  y = sublayer(norm(u));  x_t <- sum_s mix[s, t] x_s + out[t] y
+
+    all streams starting as the scaled embedding; the logits read the sum of the streams through
+    the (unscaled) embedding table. The mixer of every layer runs two halves side by side: windowed
+    attention (interleaved YaRN rotation, unit queries and keys after it, kept first tokens, a gate per
+    channel) and lightning attention. Feed-forwards: routed experts with clamped gates, sigmoid
+    scores that weigh the experts' inputs and a gated shared expert; a layer may have none. A span of
+    the list can run several passes with the same weights, each pass with a cache and state of its own."""
+    name: str = "zinavik"
+    architecture: str = "zinavik"
+    family: str = "zinavik"
+    hidden_size: int = 256
+    vocab_size: int = 512
+    layers: tuple = ()
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 1
+    streams: int = 1
+    norm_eps: float = 1e-6
+    embed_scale: float = 1.0
+    max_position_embeddings: int = 1 << 20   # rotary angles are computed, not tabulated
+    default_model_len: int = 32768
+    bos_token_id: int | None = None
+    eos_token_id: tuple = ()
+    vision: object = None
+    num_experts: int = 0                      # engine start-up tuning of the dense families keys on it
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list:
+        """Layer runs in execution order: (layer index, pass index, starts a later pass)."""
+        return loop_runs(len(self.layers), self.loop_start, self.loop_stop, self.loop_times)
+
+    def num_params(self) -> int:
+        H, n = self.hidden_size, self.vocab_size * self.hidden_size
+        for l in self.layers:
+            a, r, f = l.mixer.left, l.mixer.right, l.mlp
+            n += H * (a.q_size + a.cache_dim + a.gate_size + a.heads * a.vdim + 2 * r.heads * r.dim + 3 * r.out_size)
+            if f is not None:
+                n += 3 * H * (f.experts * f.ff + f.shared_ff) + H * (f.experts + (1 if f.shared_gate else 0))
+        return n
+
+    def replace(self, **kw) -> "ZinavikConfig":
+        return dataclasses.replace(self, **kw)
+
+    @staticmethod
+    def attention_spec(m: dict) -> WindowAttentionSpec:
+        rot, mask = m.get("rot") or {}, m.get("mask") or {}
+        sc = rot.get("scaling")
+        yarn = YarnScaling(float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"])) if sc else None
+        return WindowAttentionSpec(
+            heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+            scale=float(m["scale"]), window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0),
+            rot_dims=int(rot.get("dims") or 0), rot_base=float(rot.get("base", 10000.0)), yarn=yarn, interleaved=True,
+            unit_qk=True, channel_gate=True)
+
+    @staticmethod
+    def from_dict(d: dict, name: str = "model") -> "ZinavikConfig":
+        layers = []
+        for l in d["layers"]:
+            m = l["mixer"]
+            if l["type"] != "parallel":
+                raise NotImplementedError(f"unknown mixer {l['type']!r}")
+            r = m["right"]
+            mixer = ParallelMixerSpec(
+                left=ZinavikConfig.attention_spec(m["left"]),
+                right=LightningSpec(heads=int(r["heads"]), dim=int(r["dim"]), vdim=int(r["vdim"]),
+                                    decay=tuple(float(x) for x in r["decay"])),
+                left_scale=float(m.get("left_scale", 1.0)), right_scale=float(m.get("right_scale", 1.0)))
+            f, mlp = l.get("mlp"), None
+            if f is not None:
+                if f.get("kind") != "moe":
+                    raise NotImplementedError(f"unknown feed-forward {f.get('kind')!r}")
+                sh = f.get("shared") or {}
+                mlp = RoutedMoESpec(experts=int(f["router"]["experts"]), top=int(f["router"]["top"]),
+                                    ff=int(f["expert"]["ff"]), limit=float(f["expert"]["limit"]),
+                                    shared_ff=int(sh.get("ff") or 0), shared_limit=float(sh.get("limit") or 0.0),
+                                    shared_gate=bool(sh), score="sigmoid", correction=False, weight_input=True,
+                                    act="clamped")
+            layers.append(HybridLayerSpec(mixer, mlp))
+        lp, norm = d.get("loop") or {}, d.get("norm") or {}
+        if lp and not 0 <= int(lp["start"]) <= int(lp["stop"]) <= len(layers):
+            raise ValueError("the loop leaves the list of layers")
+        eos = d.get("eos_token_id", ())
+        eos = tuple(eos) if isinstance(eos, (list, tuple)) else (eos,)
+        return ZinavikConfig(
+            name=name, hidden_size=int(d["width"]), vocab_size=int(d["vocab"]), layers=tuple(layers),
+            loop_start=int(lp.get("start", 0)), loop_stop=int(lp.get("stop", 0)), loop_times=int(lp.get("times", 1)),
+            streams=int(d.get("streams", 1)), norm_eps=float(norm.get("eps", 1e-6)),
+            embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)), bos_token_id=d.get("bos_token_id"),
+            eos_token_id=eos)
+
+
 def check_kv_sources(layers):
     """A layer that reads another layer's keys and values must name an earlier attention layer
     with a cache of its own and the same key / value head layout."""
@@ -1210,6 +1392,8 @@ def config_from_dict(d: dict, name: str = "model"):
         return KemavikConfig.from_dict(d, name=name)
     if arch == "topezen":
         return TopezenConfig.from_dict(d, name=name)
+    if arch == "zinavik":
+        return ZinavikConfig.from_dict(d, name=name)
     return ModelConfig.from_hf_dict(d, name=name)
 
 
@@ -1323,4 +1507,33 @@ PRESETS.update({
                                    dict(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.125, window=160, keep_first=16,
                                         softcap=50.0),
                                    1536, dict(experts=8, top=2, ff=256, shared_ff=512, groups=4, keep_groups=2), "lmam"),
+})
+
+
+def _mini_zinavik(name, H, V, attn, lightning, moe, order, loop=(0, 0, 1), streams=2, scales=(0.9, 0.6), embed_scale=4.0):
+    """order: 'p' parallel mixer + routed experts, 'n' parallel mixer without a feed-forward."""
+    a = WindowAttentionSpec(interleaved=True, unit_qk=True, channel_gate=True, **attn)
+    decay = tuple(1.0 - 2.0 ** (-1.0 - 7.0 * (h + 1) / lightning["heads"]) for h in range(lightning["heads"]))
+    m = ParallelMixerSpec(a, LightningSpec(decay=decay, **lightning), *scales)
+    f = RoutedMoESpec(score="sigmoid", correction=False, weight_input=True, act="clamped", shared_gate=True, **moe)
+    spec = {"p": HybridLayerSpec(m, f), "n": HybridLayerSpec(m, None)}
+    return ZinavikConfig(name=name, hidden_size=H, vocab_size=V, layers=tuple(spec[c] for c in order),
+                         loop_start=loop[0], loop_stop=loop[1], loop_times=loop[2], streams=streams,
+                         embed_scale=embed_scale, eos_token_id=(2,), bos_token_id=1)
+
+
+PRESETS.update({
+    # CPU plumbing size
+    "tiny-zinavik": _mini_zinavik("tiny-zinavik", 64, 320,
+                                  dict(heads=4, kv_heads=2, dim=16, vdim=24, scale=0.3, window=20, keep_first=3, rot_dims=12,
+                                       yarn=YarnScaling(2.0, 64, 16.0, 1.0)),
+                                  dict(heads=2, dim=16, vdim=24),
+                                  dict(experts=6, top=2, ff=24, limit=4.0, shared_ff=40, shared_limit=5.0), "pnp", loop=(1, 3, 2)),
+    # GPU-test size
+    "small-zinavik": _mini_zinavik("small-zinavik", 512, 1024,
+                                   dict(heads=4, kv_heads=2, dim=64, vdim=64, scale=0.125, window=160, keep_first=8, rot_dims=64,
+                                        rot_base=50000.0, yarn=YarnScaling(4.0, 1024, 32.0, 1.0)),
+                                   dict(heads=4, dim=64, vdim=64),
+                                   dict(experts=8, top=2, ff=256, limit=7.0, shared_ff=512, shared_limit=7.0), "ppn",
+                                   loop=(0, 2, 2), streams=4),
 })

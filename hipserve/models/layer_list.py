@@ -171,6 +171,8 @@ class LayerListModel:
 def _proj_width(mixer) -> int:
     """Columns of a mixer's input projections (all of them together)."""
     if hasattr(mixer, "left"):
+        if mixer.w_in is not None:   # one projection for both halves
+            return mixer.w_in.shape[0]
         return _proj_width(mixer.left) + _proj_width(mixer.right)
     if hasattr(mixer, "w_in_t"):   # batched projections [n, hidden, out] of n blended copies of the input
         return mixer.w_in_t.shape[0] * mixer.w_in_t.shape[2] + (mixer.w_in_t.shape[0] + 1) * mixer.hidden

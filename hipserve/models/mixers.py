@@ -39,8 +39,12 @@ them is one op of the op set:
 * generalized delta rule: merged [r | k | v | a | g | decay bottleneck] projection -> tanh ->
   decay up-projection (32-bit result) -> ``delta_rule`` (decay, removal rate, unit key, the
   recurrence, per-head output norm and sigmoid gate) -> output projection.
+* linear attention with fixed decays (``Lightning``): merged [q | k | v | gate] projection ->
+  ``lightning`` (SiLU, the recurrence from the sequence's state slot, one norm over the
+  concatenated heads, sigmoid gate) -> output projection.
 * parallel mixer: both halves write their scaled head outputs side by side into one
-  buffer, and ONE output projection over the concatenated weights sums them.
+  buffer, and ONE output projection over the concatenated weights sums them; where both
+  halves can take their input projection from outside, ONE input projection serves both.
 * dense feed-forward: up projection -> ``activation`` -> down projection.
 
 * matrix memory (``MLstm``): merged [q | k | v | gate] projection and a 32-bit [input gate | forget
@@ -60,7 +64,7 @@ from __future__ import annotations
 import torch
 import torch.nn.functional as F
 
-from ..config import (DeltaRuleSpec, DenseFFSpec, GatedDeltaSpec, LatentAttentionSpec, MinGRUSpec, MLstmSpec,
+from ..config import (DeltaRuleSpec, DenseFFSpec, GatedDeltaSpec, LatentAttentionSpec, LightningSpec, MinGRUSpec, MLstmSpec,
                       ParallelMixerSpec, RoutedMoESpec, TableMoESpec, WindowAttentionSpec, WkvSpec)
 
 MOE_TILE = 32        # slots per expert tile of the expert GEMMs ...
@@ -340,8 +344,11 @@ class WindowAttention:
         # f_i = base^(-2i / dims), 32-bit
         self.inv_freq = torch.pow(torch.tensor(spec.rot_base, dtype=torch.float32),
                                   -2.0 * i / max(spec.rot_dims, 1)).to(device)
-        self.gate_off = spec.q_size + spec.cache_dim if spec.gate else -1
-        assert spec.maps in (1, 2) and not (spec.gate and spec.kv_from is not None)
+        if spec.yarn is not None:
+            self.inv_freq = torch.tensor(spec.yarn.frequencies(spec.rot_base, spec.rot_dims), dtype=torch.float32).to(device)
+        self.gate_off = spec.q_size + spec.cache_dim if spec.gate_size else -1
+        assert spec.maps in (1, 2) and not (spec.gate_size and spec.kv_from is not None)
+        assert not (spec.channel_gate and spec.maps == 2) and not (spec.unit_qk and (spec.qk_norm or spec.head_norm))
 
     @property
     def out_size(self) -> int:
@@ -353,9 +360,19 @@ class WindowAttention:
     def load(self, get, prefix: str):
         s, dt, dev = self.spec, self.dtype, self.device
         names = self._in_names()
-        self.w_in = torch.cat([get(prefix + n) for n in names + (["g"] if s.gate else [])], 0).to(dev, dt).contiguous()
+
+        def rows(n):
+            w = get(prefix + n)
+            if not s.interleaved or n not in ("q", "k"):
+                return w
+            # the same permutation of every query and key head leaves scores and root mean squares unchanged and
+            # turns the pairs (2i, 2i + 1) into the pairs (i, i + dims / 2) of the kernels
+            return _deinterleave(w.view(-1, s.dim, w.shape[-1]), s.rot_dims).reshape(w.shape)
+
+        assert not s.interleaved or not (s.bias or s.qk_norm or s.head_norm)   # those would be permuted alike
+        self.w_in = torch.cat([rows(n) for n in names + (["g"] if s.gate_size else [])], 0).to(dev, dt).contiguous()
         if s.bias:
-            b = [get(prefix + n + ".b") for n in names] + ([torch.zeros(s.heads)] if s.gate else [])
+            b = [get(prefix + n + ".b") for n in names] + ([torch.zeros(s.gate_size)] if s.gate_size else [])
             self.b_in = torch.cat([x.float() for x in b]).to(dev, dt).contiguous()
         if s.qk_norm or s.head_norm:
             self.q_norm = get(prefix + "q.norm").to(dev, torch.float32)
@@ -376,8 +393,8 @@ class WindowAttention:
         t = {"q": _rand(gen, s.q_size, H, std=std * 4), "o": _rand(gen, H, self.out_size, std=std)}
         if s.kv_from is None:
             t.update({"k": _rand(gen, s.k_size, H, std=std * 4), "v": _rand(gen, s.v_size, H, std=std * 4)})
-        if s.gate:
-            t["g"] = _rand(gen, s.heads, H, std=std * 4)
+        if s.gate_size:
+            t["g"] = _rand(gen, s.gate_size, H, std=std * 4)
         if s.bias:
             t.update({n + ".b": _rand(gen, t[n].shape[0], std=0.3) for n in self._in_names()})
         if s.out_bias:
@@ -394,12 +411,16 @@ class WindowAttention:
             t["sink"] = _rand(gen, s.heads)
         return t
 
-    def mix(self, h, meta, cache, state, out, out_scale: float = 1.0):
+    takes_proj = property(lambda self: self.b_in is None and not self.side_rows)   # ``mix`` takes ``proj`` from outside
+
+    def mix(self, h, meta, cache, state, out, out_scale: float = 1.0, proj=None):
         """Head outputs (before the output projection), times ``out_scale``, into ``out`` [T, heads * vdim]
-        (a column slice of a wider buffer is fine)."""
+        (a column slice of a wider buffer is fine). ``proj``: the input projection's rows, when it is part of
+        a wider one (a column slice, overwritten)."""
         s, ops = self.spec, self.ops
-        proj = F.linear(h, self.w_in, self.b_in)
-        _side(self, proj)
+        if proj is None:
+            proj = F.linear(h, self.w_in, self.b_in)
+            _side(self, proj)
         ops.attn_prepare(proj, cache, meta, self.inv_freq, s, self.q_norm, self.k_norm, self.eps)
         ops.window_attention(out, proj, cache, meta, s, self.gate_off, out_scale, self.lam, self.eps, self.sink_w)
         return out
@@ -619,6 +640,51 @@ class MLstm:
         return F.linear(out, self.w_o)
 
 
+class Lightning:
+    cache_dim = 0
+    takes_proj = True
+
+    def __init__(self, spec: LightningSpec, hidden: int, eps: float, device, dtype, ops):
+        self.spec, self.hidden, self.eps, self.device, self.dtype, self.ops = spec, hidden, eps, device, dtype, ops
+        self.w_in = None     # [q | k | v | gate, hidden]
+        self.norm = None     # fp32 [heads * vdim]
+        self.w_o = None
+        # decay^0 .. decay^64 per head, computed in double precision (column 1 is the decay itself)
+        d = torch.tensor(spec.decay, dtype=torch.float64)
+        self.powers = torch.stack([d ** n for n in range(65)], 1).to(torch.float32).to(device).contiguous()
+
+    @property
+    def out_size(self) -> int:
+        return self.spec.out_size
+
+    def state_shapes(self, slots: int):
+        s = self.spec
+        return [(slots, s.heads, s.dim, s.vdim)]
+
+    def load(self, get, prefix: str):
+        dt, dev = self.dtype, self.device
+        self.w_in = torch.cat([get(prefix + n) for n in ("q", "k", "v", "g")], 0).to(dev, dt).contiguous()
+        self.norm = get(prefix + "norm").to(dev, torch.float32).contiguous()
+        self.w_o = get(prefix + "o").to(dev, dt).contiguous()
+
+    def init_random(self, gen, std: float):
+        s, H = self.spec, self.hidden
+        qk = s.heads * s.dim
+        return {"q": _rand(gen, qk, H, std=std * 4), "k": _rand(gen, qk, H, std=std * 4),
+                "v": _rand(gen, s.out_size, H, std=std * 4), "g": _rand(gen, s.out_size, H, std=std * 4),
+                "norm": 1.0 + 0.2 * _rand(gen, s.out_size), "o": _rand(gen, H, s.out_size, std=std)}
+
+    def mix(self, h, meta, cache, state, out, out_scale: float = 1.0, proj=None):
+        if proj is None:
+            proj = F.linear(h, self.w_in)
+        self.ops.lightning(out, state[0], proj, self.powers, self.norm, self.spec, self.eps, meta, out_scale)
+        return out
+
+    def forward(self, h, meta, cache, state):
+        out = torch.empty(h.shape[0], self.out_size, device=h.device, dtype=h.dtype)
+        return F.linear(self.mix(h, meta, cache, state, out), self.w_o)
+
+
 class ParallelMixer:
     """left_scale * left(h) + right_scale * right(h): both halves write their scaled head outputs
     into one [T, left | right] buffer; one GEMM with the concatenated output weights sums them."""
@@ -628,6 +694,8 @@ class ParallelMixer:
         self.left = make_mixer(spec.left, hidden, eps, device, dtype, ops)
         self.right = make_mixer(spec.right, hidden, eps, device, dtype, ops)
         self.w_o = None      # [hidden, left out | right out]
+        self.w_in = None     # [left inputs | zero rows up to a multiple of 8 | right inputs, hidden], when one GEMM serves both
+        self.split = 0       # rows of w_in before the right half's
 
     @property
     def cache_dim(self) -> int:
@@ -644,6 +712,11 @@ class ParallelMixer:
         self.right.load(get, prefix + "right.")
         self.w_o = torch.cat([self.left.w_o, self.right.w_o], 1).contiguous()
         self.left.w_o = self.right.w_o = None
+        if getattr(self.left, "takes_proj", False) and getattr(self.right, "takes_proj", False):
+            wl, wr = self.left.w_in, self.right.w_in
+            self.split = -(-wl.shape[0] // 8) * 8   # 16-byte aligned rows in bf16
+            self.w_in = torch.cat([F.pad(wl, (0, 0, 0, self.split - wl.shape[0])), wr], 0).contiguous()
+            self.left.w_in = self.right.w_in = None
 
     def init_random(self, gen, std: float):
         t = {"left." + k: v for k, v in self.left.init_random(gen, std).items()}
@@ -653,6 +726,11 @@ class ParallelMixer:
     def forward(self, h, meta, cache, state):
         a, b = self.left.out_size, self.right.out_size
         buf = torch.empty(h.shape[0], a + b, device=h.device, dtype=h.dtype)
+        if self.w_in is not None:
+            proj = F.linear(h, self.w_in)
+            self.left.mix(h, meta, cache, state, buf[:, :a], self.spec.left_scale, proj[:, :self.split])
+            self.right.mix(h, meta, cache, state, buf[:, a:], self.spec.right_scale, proj[:, self.split:])
+            return F.linear(buf, self.w_o)
         self.left.mix(h, meta, cache, state, buf[:, :a], self.spec.left_scale)
         self.right.mix(h, meta, cache, state, buf[:, a:], self.spec.right_scale)
         return F.linear(buf, self.w_o)
@@ -705,7 +783,10 @@ class RoutedMoE:
     """``forward`` returns the parts of the mixture's output, (ye, pair_slot, ids, wts, experts, h, shared),
     which the residual update (``add_normed``) combines: row ``pair_slot[t * top + j]`` of ``ye`` is the
     output of token t's j-th choice ``ids[t, j]`` (a value >= experts is an identity expert: the token's
-    own input), weighted ``wts[t, j]``; ``shared`` is the shared expert's output or None."""
+    own input), weighted ``wts[t, j]`` (already applied to the experts' inputs with ``spec.weight_input``:
+    their gate | up products, being linear, are scaled in the GEMM's epilogue); ``shared`` is the shared
+    expert's output or None, to be multiplied by the sigmoid of ``shared_gate`` [T, 1] where that is not None
+    (one more row of the router, so it is 32-bit)."""
 
     side_weight, side_rows, side_out = "ws_gu", 0, None
 
@@ -717,11 +798,19 @@ class RoutedMoE:
         self.w_down = None        # [E, hidden, ff]
         self.ws_gu = self.ws_down = None   # the shared expert's [2 * shared_ff, hidden], [hidden, shared_ff]
         self.packed = None        # (gate | up, down) in the packed grouped-GEMM layout, made at the first large batch
+        self.shared_gate = None   # [T, 1] fp32 after forward, before its sigmoid
+        assert spec.act in ("silu", "clamped") and spec.score in ("softmax", "sigmoid")
+        assert not (spec.weight_input and spec.identity)
+        self.epilogue = 2 if spec.act == "silu" else 3
 
     def load(self, get, prefix: str):
         s, dt, dev = self.spec, self.dtype, self.device
-        self.w_router = get(prefix + "router").to(dev, dt).contiguous()
-        self.correction = get(prefix + "correction").to(dev, torch.float32).contiguous()
+        router = get(prefix + "router")
+        if s.shared_gate:
+            router = torch.cat([router, get(prefix + "shared.sg")], 0)
+        self.w_router = router.to(dev, dt).contiguous()
+        if s.correction:
+            self.correction = get(prefix + "correction").to(dev, torch.float32).contiguous()
         self.w_gu = torch.stack([torch.cat([get(f"{prefix}e{e}.gate"), get(f"{prefix}e{e}.up")], 0)
                                  for e in range(s.experts)]).to(dev, dt).contiguous()
         self.w_down = torch.stack([get(f"{prefix}e{e}.down") for e in range(s.experts)]).to(dev, dt).contiguous()
@@ -733,6 +822,10 @@ class RoutedMoE:
         s, H = self.spec, self.hidden
         n = s.experts + s.identity
         t = {"router": _rand(gen, n, H, std=std * 8), "correction": _rand(gen, n, std=0.1)}
+        if not s.correction:
+            del t["correction"]
+        if s.shared_gate:
+            t["shared.sg"] = _rand(gen, 1, H, std=std * 8)
         for e in range(s.experts):
             t.update({f"e{e}.gate": _rand(gen, s.ff, H, std=std * 4), f"e{e}.up": _rand(gen, s.ff, H, std=std * 4),
                       f"e{e}.down": _rand(gen, H, s.ff, std=std * 4)})
@@ -746,12 +839,17 @@ class RoutedMoE:
         T, dev = h.shape[0], h.device
         ids = torch.empty(T, s.top, dtype=torch.int32, device=dev)
         wts = torch.empty(T, s.top, dtype=torch.float32, device=dev)
-        ops.route_topk(ids, wts, _linear32(h, self.w_router), self.correction, s.top, s.scale, s.experts,
-                       s.groups, s.keep_groups, s.renorm)
+        logits = _linear32(h, self.w_router)
+        if s.shared_gate:
+            n = s.experts + s.identity
+            logits, self.shared_gate = logits[:, :n], logits[:, n:]
+        ops.route_topk(ids, wts, logits, self.correction, s.top, s.scale, s.experts, s.groups, s.keep_groups, s.renorm,
+                       s.score)
+        scale = wts if s.weight_input else None
         # the identity experts share one bucket (s.experts) that no GEMM tile serves
         P, nb = T * s.top, s.experts + (1 if s.identity else 0)
         if self._packed_ok(h, P, nb):
-            ye, pair_slot = self._experts_packed(h, ids, P, nb)
+            ye, pair_slot = self._experts_packed(h, ids, P, nb, scale)
             return ye, pair_slot, ids, wts, s.experts, h, self._shared(h)
         tile = MOE_TILE_LARGE if P >= 4 * MOE_TILE_LARGE * nb else MOE_TILE
         cap = -(-(P + nb * (tile - 1)) // tile) * tile
@@ -760,7 +858,8 @@ class RoutedMoE:
         pair_slot = torch.empty(P, dtype=torch.int32, device=dev)
         ops.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
         act = torch.empty(cap, s.ff, device=dev, dtype=h.dtype)
-        ops.expert_gemm(act, h, self.w_gu, slots, tile_expert, tile, s.top, 2)      # silu(gate) * up in the epilogue
+        # the gate and the pair's input weight in the epilogue
+        ops.expert_gemm(act, h, self.w_gu, slots, tile_expert, tile, s.top, self.epilogue, scale, s.limit)
         ye = torch.empty(cap, self.hidden, device=dev, dtype=h.dtype)
         ops.expert_gemm(ye, act, self.w_down, slots, tile_expert, tile, 0, 0)
         return ye, pair_slot, ids, wts, s.experts, h, self._shared(h)
@@ -775,7 +874,7 @@ class RoutedMoE:
         if not n:
             return None
         a = torch.empty(h.shape[0], n, device=h.device, dtype=h.dtype)
-        self.ops.activation(a, g[:, :2 * n], "silu_mul")
+        self.ops.activation(a, g[:, :2 * n], "silu_mul" if self.spec.act == "silu" else "clamped_glu", self.spec.shared_limit)
         return F.linear(a, self.ws_down)
 
     def _packed_ok(self, h: torch.Tensor, P: int, nb: int) -> bool:
@@ -786,10 +885,10 @@ class RoutedMoE:
                 and self.hidden % 256 == 0 and s.ff % 256 == 0
                 and P >= MOE_PACKED_MIN_PAIRS_PER_EXPERT * nb and not torch.cuda.is_current_stream_capturing())
 
-    def _experts_packed(self, h: torch.Tensor, ids: torch.Tensor, P: int, nb: int):
+    def _experts_packed(self, h: torch.Tensor, ids: torch.Tensor, P: int, nb: int, scale=None):
         """Large bf16 batches: the experts as two launches of the packed-layout grouped GEMM of the dense
-        families' MoE prefill (token rows gathered through the slot table inside the first one, the SiLU gate
-        in its epilogue). The identity bucket sorts last, so the GEMMs simply stop before its tiles."""
+        families' MoE prefill (token rows gathered through the slot table inside the first one, the gate and
+        the pairs' input weights in its epilogue). The identity bucket sorts last, so the GEMMs simply stop before its tiles."""
         from ..ops import gemm
 
         s, dev = self.spec, h.device
@@ -812,7 +911,8 @@ class RoutedMoE:
             ntiles = ((tile_expert >= 0) & (tile_expert < E)).sum(dtype=torch.int32).view(1)
         pgu, pd = self.packed
         act = torch.empty(cap, ff, dtype=h.dtype, device=dev)
-        op.prefill_gemm_packed_grouped(act, h, pgu, 2 * ff, 2, tile_expert, ntiles, gemm.PW_WM, gemm.PW_RW, slots, s.top)
+        op.prefill_gemm_packed_grouped(act, h, pgu, 2 * ff, 2 if s.act == "silu" else 5, tile_expert, ntiles, gemm.PW_WM,
+                                       gemm.PW_RW, slots, s.top, scale, s.limit)
         ye = torch.empty(cap, H, dtype=h.dtype, device=dev)
         op.prefill_gemm_packed_grouped(ye, act, pd, H, 0, tile_expert, ntiles, gemm.PW_WM, gemm.PW_RW)
         return ye, pair_slot
@@ -839,6 +939,8 @@ def make_mixer(spec, hidden: int, eps: float, device, dtype, ops):
         return DeltaRule(spec, hidden, eps, device, dtype, ops)
     if isinstance(spec, MLstmSpec):
         return MLstm(spec, hidden, eps, device, dtype, ops)
+    if isinstance(spec, LightningSpec):
+        return Lightning(spec, hidden, eps, device, dtype, ops)
     if isinstance(spec, ParallelMixerSpec):
         return ParallelMixer(spec, hidden, eps, device, dtype, ops)
     if isinstance(spec, LatentAttentionSpec):

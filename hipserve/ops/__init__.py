@@ -1,8 +1,9 @@
 """hipserve op library.
 
 ``KernelOps`` calls the hand-written gfx950 kernels in ``hipserve/_C.so``
-(``torch.ops.hipserve.*``) and, for the layer-list decoders, ``hipserve/_C_seq.so`` and
-``hipserve/_C_delta.so`` and ``hipserve/_C_cell.so`` (``torch.ops.hipserve_seq.*``, ``torch.ops.hipserve_delta.*``, ``torch.ops.hipserve_cell.*``); each library is loaded at the first use of one of its kernels. ``ReferenceOps`` is the plain-PyTorch oracle used by
+(``torch.ops.hipserve.*``) and, for the layer-list decoders, ``hipserve/_C_seq.so``, ``_C_delta.so``,
+``_C_cell.so`` and ``_C_stream.so`` (``torch.ops.hipserve_seq.*`` and so on); each library is loaded at the
+first use of one of its kernels. ``ReferenceOps`` is the plain-PyTorch oracle used by
 the CPU plumbing engine and by the numerics tests. The choice is made ONCE, when
 an engine is built for a device — never per call. On a GPU device the native
 library is mandatory: a missing/unloadable ``_C.so`` raises instead of silently
@@ -19,14 +20,13 @@ from . import reference as ref
 
 _PKG = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 _LIB = os.path.join(_PKG, "_C.so")
-_LIB_SEQ = os.path.join(_PKG, "_C_seq.so")  # the layer-list decoders' kernels (torch.ops.hipserve_seq)
-_LIB_DELTA = os.path.join(_PKG, "_C_delta.so")  # ... window attention / delta rules (torch.ops.hipserve_delta)
-_LIB_CELL = os.path.join(_PKG, "_C_cell.so")  # ... gated parallel blocks, mLSTM, PolyNorm (torch.ops.hipserve_cell)
+# the layer-list decoders' kernels, a library (and a torch.ops namespace hipserve_<name>) per set of designs:
+# seq: latent attention, minGRU, table experts; delta: window attention, delta rules, decayed linear attention;
+# cell: gated parallel blocks, mLSTM, PolyNorm; stream: residual streams, lightning attention
+_SEQ_LIBS = {n: os.path.join(_PKG, f"_C_{n}.so") for n in ("seq", "delta", "cell", "stream")}
 _lock = threading.Lock()
 _loaded = False
-_loaded_seq = False
-_loaded_delta = False
-_loaded_cell = False
+_loaded_seq: set = set()
 
 
 def library_path() -> str:
@@ -51,50 +51,36 @@ def load_library(build_if_missing: bool = False) -> str:
         return _LIB
 
 
-def load_seq_library() -> str:
-    """Load hipserve/_C_seq.so into torch.ops (idempotent); built first when it is missing
-    (a few hipcc seconds: four kernel files)."""
-    global _loaded_seq
+def load_kernel_library(name: str) -> str:
+    """Load hipserve/_C_<name>.so (a key of ``_SEQ_LIBS``) into torch.ops (idempotent); built first when it is
+    missing (a few hipcc seconds)."""
+    path = _SEQ_LIBS[name]
     with _lock:
-        if _loaded_seq:
-            return _LIB_SEQ
-        if not os.path.exists(_LIB_SEQ):
+        if name in _loaded_seq:
+            return path
+        if not os.path.exists(path):
             from .._build import build_kernels
 
-            build_kernels(lib="seq")
-        torch.ops.load_library(_LIB_SEQ)
-        _loaded_seq = True
-        return _LIB_SEQ
+            build_kernels(lib=name)
+        torch.ops.load_library(path)
+        _loaded_seq.add(name)
+        return path
+
+
+def load_seq_library() -> str:
+    return load_kernel_library("seq")
 
 
 def load_delta_library() -> str:
-    """Load hipserve/_C_delta.so into torch.ops (idempotent); built first when it is missing."""
-    global _loaded_delta
-    with _lock:
-        if _loaded_delta:
-            return _LIB_DELTA
-        if not os.path.exists(_LIB_DELTA):
-            from .._build import build_kernels
-
-            build_kernels(lib="delta")
-        torch.ops.load_library(_LIB_DELTA)
-        _loaded_delta = True
-        return _LIB_DELTA
+    return load_kernel_library("delta")
 
 
 def load_cell_library() -> str:
-    """Load hipserve/_C_cell.so into torch.ops (idempotent); built first when it is missing."""
-    global _loaded_cell
-    with _lock:
-        if _loaded_cell:
-            return _LIB_CELL
-        if not os.path.exists(_LIB_CELL):
-            from .._build import build_kernels
+    return load_kernel_library("cell")
 
-            build_kernels(lib="cell")
-        torch.ops.load_library(_LIB_CELL)
-        _loaded_cell = True
-        return _LIB_CELL
+
+def load_stream_library() -> str:
+    return load_kernel_library("stream")
 
 
 def core_built() -> bool:
@@ -118,11 +104,9 @@ class KernelOps:
 
     def __init__(self):
         self._core = None
-        self._seq_ops = None
-        self._delta_ops = None
-        self._cell_ops = None
-        # the library whose copy of the shared kernels runs ("seq" / "delta" / "cell"): a model sets it to the one
-        # its mixers load anyway, so it never builds or loads another
+        self._lib_ops = {}
+        # the library whose copy of the shared kernels runs ("seq" / "delta" / "cell" / "stream"): a model sets it to
+        # the one its mixers load anyway, so it never builds or loads another
         self.norm_library = "seq"
 
     @property
@@ -133,36 +117,27 @@ class KernelOps:
             self._core = torch.ops.hipserve
         return self._core
 
-    @property
-    def _seq(self):
-        if self._seq_ops is None:
-            load_seq_library()
-            self._seq_ops = torch.ops.hipserve_seq
-        return self._seq_ops
+    def _lib(self, name: str):
+        """torch.ops.hipserve_<name>, its library loaded at the first use."""
+        if name not in self._lib_ops:
+            load_kernel_library(name)
+            self._lib_ops[name] = getattr(torch.ops, "hipserve_" + name)
+        return self._lib_ops[name]
 
-    @property
-    def _delta(self):
-        if self._delta_ops is None:
-            load_delta_library()
-            self._delta_ops = torch.ops.hipserve_delta
-        return self._delta_ops
-
-    @property
-    def _cell(self):
-        if self._cell_ops is None:
-            load_cell_library()
-            self._cell_ops = torch.ops.hipserve_cell
-        return self._cell_ops
+    _seq = property(lambda self: self._lib("seq"))
+    _delta = property(lambda self: self._lib("delta"))
+    _cell = property(lambda self: self._lib("cell"))
+    _stream = property(lambda self: self._lib("stream"))
 
     @property
     def _latent_lib(self):
         """The library whose copy of the latent-attention kernels runs."""
-        return self._cell if self.norm_library == "cell" else self._seq
+        return self._lib("cell" if self.norm_library == "cell" else "seq")
 
     @property
     def _window_lib(self):
         """The library whose copy of the window attention, router and activation kernels runs."""
-        return self._cell if self.norm_library == "cell" else self._delta
+        return self._lib(self.norm_library if self.norm_library in ("cell", "stream") else "delta")
 
     def rmsnorm(self, out, x, w, eps, out8=None):
         """out8: (e4m3 [rows, hidden] uint8, scales fp32 [rows]) per-token FP8 copy of out."""
@@ -312,11 +287,12 @@ class KernelOps:
         self._seq.mingru_scan(y, state, proj, b_z, b_x, meta.seq_cu, meta.seq_ctx, meta.seq_state, meta.max_q)
 
     def attn_prepare(self, proj, cache, meta, inv_freq, sp, q_norm, k_norm, eps):
-        mode = 1 if sp.qk_norm else 2 if sp.head_norm else 0
+        mode = 1 if sp.qk_norm else 2 if sp.head_norm else 3 if sp.unit_qk else 0
         own_kv = sp.kv_from is None   # else the layer reads another layer's cache: only q is prepared
         self._window_lib.attn_prepare(proj, cache if own_kv else None, meta.positions, meta.slot_mapping, inv_freq, sp.heads,
-                                 sp.kv_heads, sp.maps, sp.dim, sp.vdim, q_norm if mode else None,
-                                 k_norm if mode and own_kv else None, mode, sp.v_norm, eps)
+                                 sp.kv_heads, sp.maps, sp.dim, sp.vdim, q_norm if mode in (1, 2) else None,
+                                 k_norm if mode in (1, 2) and own_kv else None, mode, sp.v_norm, eps,
+                                 sp.yarn.amplitude if sp.yarn is not None else 1.0)
 
     WINDOW_PREFILL_TQ = 4  # tokens per workgroup of a prompt portion (x the query heads of one key/value head)
     # bf16 runs the MFMA kernel (HIPSERVE_WINDOW_MFMA=0: the generic kernel, as fp32 does)
@@ -331,7 +307,7 @@ class KernelOps:
         nseq = meta.seq_ctx.shape[0]
         nd = meta.num_decode
         npf, Tp = nseq - nd, meta.num_prefill_tokens
-        diff = (sp.maps, lam, 1.0 - sp.diff, eps, sp.keep_first, sp.softcap, sink_w)
+        diff = (sp.maps, lam, 1.0 - sp.diff, eps, sp.keep_first, sp.softcap, sink_w, sp.channel_gate)
         if (proj.dtype == torch.bfloat16 and self.WINDOW_MFMA
                 and self._window_lib.window_attention_mfma_ok(sp.dim, sp.vdim, out.stride(0), out.storage_offset(), sp.maps)):
             # bf16: the matrix-core kernel; decode rows split their keys into runs merged by a reduce kernel
@@ -374,7 +350,7 @@ class KernelOps:
         self._delta.delta_rule(out, state[0], proj, wl, a_b, w0, norm_w, meta.seq_cu, meta.seq_ctx, meta.seq_state,
                              scratch, sp.heads, sp.dim, eps, out_scale)
 
-    ACTIVATIONS = {"tanh": 0, "xielu": 1, "relu2": 2, "silu_mul": 3}
+    ACTIVATIONS = {"tanh": 0, "xielu": 1, "relu2": 2, "silu_mul": 3, "clamped_glu": 4}
 
     def activation(self, out, x, kind, c0=0.0, c1=0.0):
         self._window_lib.activation(out, x, self.ACTIVATIONS[kind], c0, c1)
@@ -404,12 +380,14 @@ class KernelOps:
 
     ROUTER_MAX_OUTPUTS = 256
 
-    def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False):
+    def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False,
+                   score="softmax"):
         if logits.shape[1] > self.ROUTER_MAX_OUTPUTS or groups > 64:
             # more router outputs than a wave holds: device-side torch ops
-            ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm)
+            ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
             return
-        self._window_lib.route_topk(ids, wts, logits.contiguous(), correction, top, scale, E, groups, keep_groups, renorm)
+        self._window_lib.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm,
+                                    score == "sigmoid")
 
     # ---- parallel blocks with gated sublayer results, mLSTM, PolyNorm (csrc/kernels/seq/gated_block.hip, mlstm.hip,
     # elementwise.hip)
@@ -440,9 +418,7 @@ class KernelOps:
     @property
     def _moe_lib(self):
         """The library whose copy of the expert alignment and expert GEMMs runs (the one the model loads anyway)."""
-        if self.norm_library == "cell":
-            return self._cell
-        return self._delta if self.norm_library == "delta" else self._seq
+        return self._lib(self.norm_library)
 
     def moe_align(self, experts, E, tile, slots, tile_expert, pair_slot):
         if E <= 128:
@@ -466,9 +442,38 @@ class KernelOps:
         te = torch.searchsorted(ends, t, right=True)
         tile_expert.copy_(torch.where(te < E, te, torch.full_like(te, -1)).to(torch.int32))
 
-    def expert_gemm(self, out, x, w, slots, tile_expert, tile, gather_k, act):
-        """act: False / 0 none, True / 1 squared ReLU, 2: w = [gate rows; up rows], out = silu(gate) * up."""
-        self._moe_lib.expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, int(act))
+    def expert_gemm(self, out, x, w, slots, tile_expert, tile, gather_k, act, row_scale=None, limit=0.0):
+        """act: False / 0 none, True / 1 squared ReLU, 2: w = [gate rows; up rows], out = silu(gate) * up, 3: the same
+        with the gate clamped at ``limit``; ``row_scale`` fp32 [pairs] multiplies each pair's product before it."""
+        self._moe_lib.expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, int(act), row_scale, limit)
+
+    # ---- residual streams, lightning attention (csrc/kernels/seq/streams.hip, lightning.hip)
+    def stream_update(self, out, dst, src, coef, w, eps, y1=None, y2=None):
+        """``y2``: a sublayer's result rows or, for a mixture of experts, (ye, pair_slot, wts or top, shared, gate)."""
+        ye = pair_slot = wts = shared = gate = None
+        top = 0
+        if isinstance(y2, tuple):
+            ye, pair_slot, wts, shared, gate = y2
+            top, wts = (wts, None) if isinstance(wts, int) else (wts.shape[1], wts)
+            y2 = None
+        self._stream.stream_update(out, dst, src, coef, w, eps, y1, y2, ye, pair_slot, wts, top, shared, gate)
+        return out
+
+    # bf16 prompt portions run the chunked matrix-core kernel (HIPSERVE_LIGHTNING_MFMA=0: the scan, as fp32 does)
+    LIGHTNING_MFMA = os.environ.get("HIPSERVE_LIGHTNING_MFMA", "1") != "0"
+
+    def lightning(self, out, S, proj, powers, norm_w, sp, eps, meta, out_scale=1.0):
+        """Prompt portions (the step's first sequences) run the chunked kernel or the scan, decode rows the
+        one-row kernel; one launch norms and gates the concatenated heads of all rows."""
+        nd, nseq = meta.num_decode, meta.seq_ctx.shape[0]
+        npf = nseq - nd
+        T = proj.shape[0]
+        mfma = (npf > 0 and self.LIGHTNING_MFMA and proj.dtype == torch.bfloat16
+                and self._stream.lightning_mfma_ok(sp.dim, sp.vdim, proj.stride(0), proj.storage_offset()))
+        rows = meta.num_prefill_tokens if npf and not mfma else 0   # the scan reads them as dense fp32 rows
+        scratch = torch.empty(T * sp.out_size + rows * sp.heads * (2 * sp.dim + sp.vdim), device=proj.device, dtype=torch.float32)
+        self._stream.lightning(out, S, proj, powers, norm_w, meta.seq_cu, meta.seq_ctx, meta.seq_state, scratch, npf,
+                               meta.num_prefill_tokens, sp.heads, sp.dim, sp.vdim, eps, out_scale, mfma)
 
 
 class ReferenceOps:
@@ -576,8 +581,15 @@ class ReferenceOps:
     def moe_align(self, experts, E, tile, slots, tile_expert, pair_slot):
         ref.moe_align(experts, E, tile, slots, tile_expert, pair_slot)
 
-    def expert_gemm(self, out, x, w, slots, tile_expert, tile, gather_k, act):
-        ref.expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, int(act))
+    def expert_gemm(self, out, x, w, slots, tile_expert, tile, gather_k, act, row_scale=None, limit=0.0):
+        ref.expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, int(act), row_scale, limit)
+
+    def stream_update(self, out, dst, src, coef, w, eps, y1=None, y2=None):
+        ref.stream_update(out, dst, src, coef, w, eps, y1, y2)
+        return out
+
+    def lightning(self, out, S, proj, powers, norm_w, sp, eps, meta, out_scale=1.0):
+        ref.lightning(out, S, proj, powers[:, 1], norm_w, sp, eps, meta.seq_cu, meta.seq_ctx, meta.seq_state, out_scale)
 
     def attn_prepare(self, proj, cache, meta, inv_freq, sp, q_norm, k_norm, eps):
         ref.attn_prepare(proj, cache, meta.positions, meta.slot_mapping, inv_freq, sp, q_norm, k_norm, eps)
@@ -616,8 +628,9 @@ class ReferenceOps:
         wl = torch.nn.functional.linear(t.float(), w2.float())
         ref.wkv(out, state, proj, wl, w0, u, norm_w, sp, eps, meta.seq_cu, meta.seq_ctx, meta.seq_state)
 
-    def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False):
-        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm)
+    def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False,
+                   score="softmax"):
+        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
 
     def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta):
         ref.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta.seq_cu,

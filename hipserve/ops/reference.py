@@ -416,14 +416,14 @@ def scaled_add_group_rmsnorm(out, residual, w, groups, eps, mix=None, ls1=None, 
     out.copy_((g.reshape(T, H) * w.float()).to(out.dtype))
 
 
-def partial_rope(x: torch.Tensor, pos: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+def partial_rope(x: torch.Tensor, pos: torch.Tensor, inv_freq: torch.Tensor, amp: float = 1.0) -> torch.Tensor:
     """Rotate-half RoPE of the first 2 * len(inv_freq) elements of the last dim (fp32);
-    pair (i, i + n): (u cos a - v sin a, v cos a + u sin a), a = pos * inv_freq[i]."""
+    pair (i, i + n): (u cos a - v sin a, v cos a + u sin a) * amp, a = pos * inv_freq[i]."""
     n = inv_freq.shape[0]
     a = pos.float().unsqueeze(-1) * inv_freq.float()
     while a.dim() < x.dim():
         a = a.unsqueeze(-2)
-    c, s = a.cos(), a.sin()
+    c, s = a.cos() * amp, a.sin() * amp
     u, v = x[..., :n].float(), x[..., n:2 * n].float()
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * n:].float()], -1)
 
@@ -516,10 +516,17 @@ def moe_align(experts, E, tile, slots, tile_expert, pair_slot):
         pos += nt * tile
 
 
-def expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, act):
+def clamped_glu(g, u, limit):
+    """g sigmoid(1.702 g) (u + 1) of g = min(gate, limit), u = clamp(up, -limit, limit)."""
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+
+
+def expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, act, row_scale=None, limit=0.0):
     """out[slot] = act(W[e(slot)] . x[row(slot)]); row = slots[slot] // gather_k (gather_k > 0)
     or the slot itself; act 0: none, 1: squared ReLU, 2: W = [gate rows; up rows] and
-    out = silu(gate) * up (half as wide). Padding slots are left untouched."""
+    out = silu(gate) * up (half as wide), 3: the same with ``clamped_glu``. ``row_scale`` [pairs]: the pair's
+    input times row_scale[pair]. Padding slots are left untouched."""
     sl = slots.tolist()
     te = tile_expert.tolist()
     for s, p in enumerate(sl):
@@ -530,6 +537,11 @@ def expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, act):
             continue
         row = p // gather_k if gather_k > 0 else s
         v = w[e].float() @ x[row].float()
+        if row_scale is not None:
+            v = v * row_scale.view(-1)[p].float()
+        if act == 3:
+            n = v.shape[0] // 2
+            v = clamped_glu(v[:n], v[n:], limit)
         if act == 1:
             v = torch.relu(v) ** 2
         elif act == 2:
@@ -552,7 +564,8 @@ def attn_prepare(proj, cache, positions, slots, inv_freq, sp, q_norm, k_norm, ep
     over the whole projection, a weight per element; ``sp.head_norm``: over every head - and map -
     of ``dim`` elements, one weight of ``dim`` elements for all) and the rotation; the cache row of
     slots >= 0 gets [keys | values], keys normed and rotated alike, values divided by their per-head
-    root mean square when ``sp.v_norm``."""
+    root mean square when ``sp.v_norm``. ``sp.yarn``: cos and sin times its amplitude; ``sp.unit_qk``:
+    every rotated query / key head divided by its root mean square."""
     T = proj.shape[0]
     nq, nk, nv = sp.q_size, sp.k_size, sp.v_size
     own_kv = sp.kv_from is None
@@ -566,13 +579,20 @@ def attn_prepare(proj, cache, positions, slots, inv_freq, sp, q_norm, k_norm, ep
     q = q.reshape(T, sp.heads * sp.maps, sp.dim)
     if sp.head_norm:
         q = _rows_rms(q, eps) * q_norm.float()
-    proj[:, :nq] = partial_rope(q, positions, inv_freq).reshape(T, nq).to(proj.dtype)
+    amp = sp.yarn.amplitude if sp.yarn is not None else 1.0
+    q = partial_rope(q, positions, inv_freq, amp)
+    if sp.unit_qk:
+        q = _rows_rms(q, eps)
+    proj[:, :nq] = q.reshape(T, nq).to(proj.dtype)
     if not own_kv:
         return
     k = k.reshape(T, sp.kv_heads * sp.maps, sp.dim)
     if sp.head_norm:
         k = _rows_rms(k, eps) * k_norm.float()
-    k = partial_rope(k, positions, inv_freq).reshape(T, nk)
+    k = partial_rope(k, positions, inv_freq, amp)
+    if sp.unit_qk:
+        k = _rows_rms(k, eps)
+    k = k.reshape(T, nk)
     if sp.v_norm:
         v = _rows_rms(v.reshape(T, sp.kv_heads, sp.vdim), eps).reshape(T, nv)
     ok = slots >= 0
@@ -585,7 +605,8 @@ def window_attention(out, proj, cache, seq_cu, seq_ctx, seq_bt, sp, gate_off, ou
     0 <= pos - j < window or j < sp.keep_first; scores s_j = q . k * scale, then
     softcap * tanh(s_j / softcap) (softcap > 0); weights exp(s_j) / (sink + sum exp(s_j)) with
     sink = exp(sink_w[h]) (1 without weights); out[t, h * vdim ..] =
-    weighted values * sigmoid(proj[t, gate_off + h]) (gate_off >= 0) * out_scale.
+    weighted values * sigmoid(proj[t, gate_off + h]) (gate_off >= 0; ``sp.channel_gate``: element e of the
+    concatenated heads times sigmoid(proj[t, gate_off + e])) * out_scale.
     ``sp.maps`` = 2: query and key heads hold [map 1 | map 2]; the head output is
     o = a1 - lam * a2 of the two maps' weighted values, o / sqrt(mean(o^2) + eps) * (1 - sp.diff)."""
     bs = cache.shape[1]
@@ -624,7 +645,9 @@ def window_attention(out, proj, cache, seq_cu, seq_ctx, seq_bt, sp, gate_off, ou
             o = o.view(b - a, H, 2, dv)
             o = o[:, :, 0] - lam * o[:, :, 1]
             o = _rows_rms(o, eps) * (1.0 - sp.diff)
-        if gate_off >= 0:
+        if gate_off >= 0 and sp.channel_gate:
+            o = o * torch.sigmoid(proj[a:b, gate_off:gate_off + H * dv].float()).view(b - a, H, dv)
+        elif gate_off >= 0:
             o = o * torch.sigmoid(proj[a:b, gate_off:gate_off + H].float()).unsqueeze(-1)
         out[a:b] = (o * out_scale).reshape(b - a, H * dv).to(out.dtype)
 
@@ -712,7 +735,8 @@ def delta_rule(out, S, proj, wl, a_b, w0, norm_w, sp, eps, seq_cu, seq_ctx, seq_
 def activation(out, x, kind, c0=0.0, c1=0.0):
     """Elementwise: ``tanh``; ``relu2`` = max(z, 0)^2; ``xielu`` with c0 = softplus(p),
     c1 = 1/2 + softplus(q): c0 z^2 + z/2 for z > 0, c1 (exp(z) - 1 - z) + z/2 otherwise;
-    ``silu_mul``: x rows = [gate | up], out = silu(gate) * up (half as wide)."""
+    ``silu_mul``: x rows = [gate | up], out = silu(gate) * up (half as wide); ``clamped_glu``: the same with
+    g sigmoid(1.702 g) (u + 1), g = min(gate, c0), u = clamp(up, -c0, c0)."""
     z = x.float()
     if kind == "tanh":
         r = torch.tanh(z)
@@ -721,6 +745,9 @@ def activation(out, x, kind, c0=0.0, c1=0.0):
     elif kind == "silu_mul":
         n = z.shape[-1] // 2
         r = z[..., :n] * torch.sigmoid(z[..., :n]) * z[..., n:]
+    elif kind == "clamped_glu":
+        n = z.shape[-1] // 2
+        r = clamped_glu(z[..., :n], z[..., n:], c0)
     elif kind == "xielu":
         zn = z.clamp(max=0.0)
         r = torch.where(z > 0, c0 * z * z + 0.5 * z, c1 * (torch.expm1(zn) - zn) + 0.5 * z)
@@ -792,15 +819,16 @@ def wkv(out, S, proj, wl, w0, u, norm_w, sp, eps, seq_cu, seq_ctx, seq_state):
         out[a0:b0] = (_rows_rms(o, eps).reshape(n, N) * norm_w.float() * (g * torch.sigmoid(g))).to(out.dtype)
 
 
-def route_topk(ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False):
-    """s = softmax(logits) (fp32, over all router outputs); the ``top`` outputs with the largest
+def route_topk(ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False, score="softmax"):
+    """s = softmax(logits) (fp32, over all router outputs) or, ``score`` = ``sigmoid``, the sigmoid of each; the ``top`` outputs with the largest
     s + correction are chosen (ties: the lower index); wts = s * scale of the chosen, ids = their
     index, outputs >= E (experts without weights) all written as E. ``groups`` > 1: the outputs
     form equal groups of neighbours, a group scores its largest s + correction, and outputs
     outside the ``keep_groups`` best groups cannot be chosen. ``renorm``: the chosen s are divided
-    by their sum (+ 1e-20) before the scaling."""
-    s = torch.softmax(logits.float(), -1)
-    c = s + correction.float()
+    by their sum (+ 1e-20) before the scaling. ``correction`` None: chosen by the logits themselves, whose
+    order is that of s (a saturated s would tie)."""
+    s = torch.sigmoid(logits.float()) if score == "sigmoid" else torch.softmax(logits.float(), -1)
+    c = s + correction.float() if correction is not None else logits.float()
     if groups > 1:
         T, n = c.shape
         best = c.view(T, groups, n // groups).max(-1).values
@@ -895,3 +923,66 @@ def mlstm(out, S, N, M, proj, gates, b_if, norm_w, sp, eps, seq_cu, seq_ctx, seq
             o[t] = torch.einsum("hkv,hk->hv", st, q[t]) / den[:, None]
         S[slot], N[slot], M[slot] = st, nn, mm
         out[a0:b0] = (_rows_rms(o, eps).reshape(n, H * dv) * norm_w.float() * torch.sigmoid(gate)).to(out.dtype)
+
+
+# ---------------------------------------------------------------------------------
+# several residual streams mixed between sublayers (static hyper-connections), linear
+# attention with one fixed decay per head over state slots
+
+def stream_update(out, dst, src, coef, w, eps, y1=None, y2=None):
+    """src [T, S, H] are the residual streams (fp32), or [T, H]: all S streams equal to it. coef (fp32) holds
+    M [S, S] (from, to), p1 [S], p2 [S], c [S] one after the other:
+      x_t = sum_s M[s, t] src_s + p1[t] y1 + p2[t] y2;   u = sum_t c[t] x_t;   out = u / rms(u) * w
+    dst (may be src, or None) gets x. y1 [T, H]; y2 [T, H] or a mixture's parts (ye, pair_slot, wts, shared, gate):
+    sum_j wts[t, j] ye[pair_slot[t * top + j]] (wts an int = top: all ones) + sigmoid(gate[t]) shared[t] (gate None: one)."""
+    n = coef.numel()
+    S = int(round((9 + 4 * n) ** 0.5 - 3) // 2)
+    assert S * S + 3 * S == n
+    M, p1, p2, c = coef[:S * S].view(S, S), coef[S * S:S * S + S], coef[S * S + S:S * S + 2 * S], coef[S * S + 2 * S:]
+    x = src.float() if src.dim() == 3 else src.float().unsqueeze(1).expand(-1, S, -1)
+    x = torch.einsum("st,nsh->nth", M, x)
+    if y1 is not None:
+        x = x + p1[:, None] * y1.float()[:, None]
+    if isinstance(y2, tuple):
+        ye, pair_slot, wts, shared, gate = y2
+        T = src.shape[0]
+        top = wts if isinstance(wts, int) else wts.shape[1]
+        y = ye.float().index_select(0, pair_slot.long()).view(T, top, -1)
+        y = y.sum(1) if isinstance(wts, int) else (y * wts.float().unsqueeze(-1)).sum(1)
+        if shared is not None:
+            y = y + (shared.float() if gate is None else shared.float() * torch.sigmoid(gate.float().view(T, 1)))
+        y2 = y
+    if y2 is not None:
+        x = x + p2[:, None] * y2.float()[:, None]
+    out.copy_((_rows_rms(torch.einsum("t,nth->nh", c, x), eps) * w.float()).to(out.dtype))
+    if dst is not None:
+        dst.copy_(x)
+
+
+def lightning(out, S, proj, decay, norm_w, sp, eps, seq_cu, seq_ctx, seq_state, out_scale=1.0):
+    """proj rows = [q | k | v | gate] pre-activations. Per head, from the sequence's slot (zeros when the step starts
+    at position 0): q, k, v through SiLU; S = decay S + k v^T; o = S^T q. The concatenated heads:
+    out = o / rms(o) * norm_w * sigmoid(gate) * out_scale. S [slots, heads, dim, vdim], decay fp32 [heads]."""
+    H, d, dv = sp.heads, sp.dim, sp.vdim
+    cu = [int(x) for x in seq_cu]
+    lam = decay.float()[:, None, None]
+    for s in range(len(cu) - 1):
+        a, b = cu[s], cu[s + 1]
+        n = b - a
+        if n == 0:
+            continue
+        slot, start = int(seq_state[s]), int(seq_ctx[s]) - n
+        p = proj[a:b].float()
+        qkv = p[:, :2 * H * d + H * dv]
+        qkv = qkv * torch.sigmoid(qkv)
+        q, k = qkv[:, :H * d].view(n, H, d), qkv[:, H * d:2 * H * d].view(n, H, d)
+        v = qkv[:, 2 * H * d:].view(n, H, dv)
+        gate = p[:, 2 * H * d + H * dv:2 * H * d + 2 * H * dv]
+        st = S[slot].clone() if start > 0 else torch.zeros_like(S[slot])
+        o = torch.empty(n, H, dv, device=proj.device)
+        for t in range(n):
+            st = lam * st + k[t, :, :, None] * v[t, :, None, :]
+            o[t] = torch.einsum("hkv,hk->hv", st, q[t])
+        S[slot] = st
+        o = _rows_rms(o.reshape(n, H * dv), eps) * norm_w.float() * torch.sigmoid(gate) * out_scale
+        out[a:b] = o.to(out.dtype)
