@@ -182,7 +182,9 @@ void launch_stream_update(void* out, float* dst, const float* src, bool one_row,
 
 // Lightning attention over state slots S [slots, heads, dim, vdim] (lightning.hip): proj rows = [q | k | v | gate | ..];
 // powers [heads, 65] = decay^0 .. decay^64; sequences 0 .. npf-1 are prompt portions (pf_rows rows in all, first in
-// the batch), the others bring one row each. scratch: T * heads * vdim floats, and without `mfma` another
+// the batch), the others bring one row each. mfma: bf16 on the matrix cores, portions cut into nseg segments of seg_len
+// tokens (a multiple of 64; nseg * seg_len covers the longest) that run side by side when nseg > 1. scratch:
+// T * heads * vdim floats, with segments another npf * nseg * heads * dim * vdim, without `mfma` another
 // pf_rows * heads * (2 dim + vdim).
 int lightning_max_dim();
 int lightning_powers();
@@ -190,6 +192,6 @@ bool lightning_mfma_ok(int dim, int vdim, long ld, long offset);
 void launch_lightning(void* out, long out_ld, float* S, const void* proj, long ld, const float* powers,
                       const float* norm_w, const int* seq_cu, const int* seq_ctx, const int* seq_state, int nseq,
                       int npf, int T, int pf_rows, float* scratch, int heads, int dim, int vdim, float eps,
-                      float out_scale, bool mfma, bool f32, hipStream_t s);
+                      float out_scale, bool mfma, int nseg, int seg_len, bool f32, hipStream_t s);
 
 }  // namespace hipserve

@@ -7,6 +7,9 @@
 // Prompt portions, bf16: lightning_chunk, 64 tokens at a time on the matrix cores. For query i and key j of a chunk
 //   o_i = lam^(i+1) S^T q_i + sum_{j <= i} lam^(i-j) (q_i . k_j) v_j
 //   S' = lam^m S + sum_j lam^(m-1-j) k_j v_j^T                          (m tokens in the chunk)
+// Few long sequences would leave most of the chip idle, so they are cut into segments that run side by side:
+// lightning_chunk<.., true> sums every segment's own keys and values, lightning_carry turns those sums into the
+// state before each segment (one pass over them in order), and the segments then run as sequences of their own.
 // The state stays in fp32 accumulator registers from the first chunk to the last. Whatever carries a decay or the
 // state enters an MFMA as the sum of two bf16 numbers (the rounding and what it left), so the products see it
 // to 16 bits; q, k and v are bf16 like every activation.
@@ -142,37 +145,51 @@ constexpr int kTLd = kC + 8;   // row stride of the token-minor tiles (elements;
 // they are; the state update sums over tokens and takes any order that both its operands share.
 HS_DEVICE int tok_col(int tt) { return (tt & 32) + 8 * ((tt >> 2) & 3) + 4 * ((tt >> 4) & 1) + (tt & 3); }
 
-template <int KS, int NT>
+template <int KS, int NT, bool SUM>
 constexpr size_t chunk_lds() {
-  return ((size_t)kC * (32 * KS + 8) + 2 * 32 * KS * kTLd + 16 * NT * kTLd + 2 * 16 * NT * (32 * KS + 8)) * 2 +
-         (kPowers + 3) * sizeof(float);
+  const size_t both = (2 * 32 * KS + 16 * NT) * kTLd * 2 + (kPowers + 3) * sizeof(float);
+  return SUM ? both : both + ((size_t)kC * (32 * KS + 8) + 2 * 16 * NT * (32 * KS + 8)) * 2;
 }
 
-// grid (heads, ceil(vdim / (16 NT)), sequences), 4 waves. dim <= 32 KS; dim % 8 == 0, vdim % 8 == 0. Wave w owns the
-// chunk's query rows 16 w .. 16 w + 15 (scores and outputs never leave its registers) and the state rows
-// 16 DT w .. (the rest of the update).
-template <int KS, int NT>
+// grid (heads, ceil(vdim / (16 NT)), sequences x nseg), 4 waves. dim <= 32 KS; dim % 8 == 0, vdim % 8 == 0. Wave w owns
+// the chunk's query rows 16 w .. 16 w + 15 (scores and outputs never leave its registers) and the state rows
+// 16 DT w .. (the rest of the update). nseg > 1: segment z % nseg of sequence z / nseg, seg_len tokens (a multiple
+// of 64) from the state ws[z, head]; the last segment's last state goes into the slot. SUM: only the state update,
+// from zero, for every segment but a sequence's last; the sum goes to ws[z, head].
+template <int KS, int NT, bool SUM>
 __global__ __launch_bounds__(256) void lightning_chunk_kernel(
     float* __restrict__ o, float* __restrict__ S, const unsigned short* __restrict__ proj, long ld,
     const float* __restrict__ powers, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx,
-    const int* __restrict__ seq_state, int heads, int dim, int vdim) {
+    const int* __restrict__ seq_state, int heads, int dim, int vdim, float* __restrict__ ws, int nseg, int seg_len) {
   constexpr int DP = 32 * KS, KLd = DP + 8, VB = 16 * NT;
   constexpr int DT = KS >= 2 ? KS / 2 : 1;   // 16-row state tiles per wave
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-  unsigned short* kr = reinterpret_cast<unsigned short*>(smem);   // [token][dim] k
-  unsigned short* kth = kr + kC * KLd;    // [dim][token] lam^(m-1-j) k_j, rounded ...
+  unsigned short* kth = reinterpret_cast<unsigned short*>(smem);   // [dim][token] lam^(m-1-j) k_j, rounded ...
   unsigned short* ktl = kth + DP * kTLd;  // ... and the rest
   unsigned short* vt = ktl + DP * kTLd;   // [vdim][token]
-  unsigned short* sh = vt + VB * kTLd;    // [vdim][dim] the state, rounded ...
+  float* pw = reinterpret_cast<float*>(vt + VB * kTLd);
+  unsigned short* kr = reinterpret_cast<unsigned short*>(pw + kPowers + 3);   // [token][dim] k
+  unsigned short* sh = kr + kC * KLd;     // [vdim][dim] the state, rounded ...
   unsigned short* sl = sh + VB * KLd;     // ... and the rest
-  float* pw = reinterpret_cast<float*>(sl + VB * KLd);
-  const int s = blockIdx.z, h = blockIdx.x, vb0 = blockIdx.y * VB;
+  const int z = blockIdx.z, s = z / nseg, seg = z - s * nseg, h = blockIdx.x, vb0 = blockIdx.y * VB;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, g = lane >> 4;
-  const int r0 = seq_cu[s], n = seq_cu[s + 1] - r0;
-  if (n <= 0) return;
-  const bool carried = seq_ctx[s] - n > 0;
+  int r0 = seq_cu[s], n = seq_cu[s + 1] - r0;
+  bool carried = seq_ctx[s] - n > 0;
   float* Sp = S + (((long)seq_state[s] * heads + h) * dim) * vdim;
+  const float* S0 = Sp;
+  bool last = true;
+  if (nseg > 1) {
+    const int at = seg * seg_len;
+    last = at + seg_len >= n;
+    if (SUM && last) return;
+    n = min(seg_len, n - at);
+    r0 += at;
+    float* wp = ws + ((long)z * heads + h) * dim * vdim;
+    if (SUM) { Sp = wp; carried = false; }
+    else { S0 = wp; carried = true; }
+  }
+  if (n <= 0) return;
   const unsigned short* pq = proj + (long)r0 * ld + (long)h * dim;
   const unsigned short* pk = pq + (long)heads * dim;
   const unsigned short* pv = proj + (long)r0 * ld + 2L * heads * dim + (long)h * vdim + vb0;
@@ -187,36 +204,44 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int d = 16 * (DT * wave + a) + 4 * g + i, v = vb0 + 16 * b + c;
-        st[a][b][i] = (carried && d < dim && v < vdim) ? Sp[(long)d * vdim + v] : 0.f;
+        st[a][b][i] = (carried && d < dim && v < vdim) ? S0[(long)d * vdim + v] : 0.f;
       }
-  constexpr int kKC = DP / 8, kVC = VB / 8;          // 16-byte pieces per token row
-  constexpr int kKF = kC * kKC / 256, kVF = (kC * kVC + 255) / 256;
-  u16x8 kf[kKF], vf[kVF], qf[KS];
+  // staging items: four neighbouring tokens x 8 channels, so the token-minor tiles take 8-byte stores
+  constexpr int kKC = DP / 8, kVC = VB / 8;                         // 16-byte pieces per token row
+  constexpr int kKI = 16 * kKC / 256 > 0 ? 16 * kKC / 256 : 1;
+  static_assert(16 * kVC <= 256, "one value item per thread");
+  u16x8 kf[kKI][4], vf[4], qf[KS];
   const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  const int vq = tid / kVC, vch = tid % kVC;
   auto fetch = [&](int t0) {
     const int m = n - t0;
 #pragma unroll
-    for (int i = 0; i < kKF; ++i) {
-      const int tt = (tid + 256 * i) / kKC, ch = (tid + 256 * i) % kKC;
-      kf[i] = (tt < m && 8 * ch < dim) ? *reinterpret_cast<const u16x8*>(pk + (long)(t0 + tt) * ld + 8 * ch) : zero;
+    for (int i = 0; i < kKI; ++i) {
+      const int kq = (tid + 256 * i) / kKC, ch = (tid + 256 * i) % kKC;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        kf[i][j] = (kq < 16 && 4 * kq + j < m && 8 * ch < dim)
+                       ? *reinterpret_cast<const u16x8*>(pk + (long)(t0 + 4 * kq + j) * ld + 8 * ch)
+                       : zero;
     }
 #pragma unroll
-    for (int i = 0; i < kVF; ++i) {
-      const int tt = (tid + 256 * i) / kVC, ch = (tid + 256 * i) % kVC;
-      vf[i] = (tt < m && tt < kC && vb0 + 8 * ch < vdim) ? *reinterpret_cast<const u16x8*>(pv + (long)(t0 + tt) * ld + 8 * ch)
-                                                        : zero;
-    }
+    for (int j = 0; j < 4; ++j)
+      vf[j] = (vq < 16 && 4 * vq + j < m && vb0 + 8 * vch < vdim)
+                  ? *reinterpret_cast<const u16x8*>(pv + (long)(t0 + 4 * vq + j) * ld + 8 * vch)
+                  : zero;
+    if constexpr (!SUM) {
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-      qf[ks] = (16 * wave + c < m && 32 * ks + 8 * g < dim)
-                   ? *reinterpret_cast<const u16x8*>(pq + (long)(t0 + 16 * wave + c) * ld + 32 * ks + 8 * g)
-                   : zero;
+      for (int ks = 0; ks < KS; ++ks)
+        qf[ks] = (16 * wave + c < m && 32 * ks + 8 * g < dim)
+                     ? *reinterpret_cast<const u16x8*>(pq + (long)(t0 + 16 * wave + c) * ld + 32 * ks + 8 * g)
+                     : zero;
+    }
   };
   fetch(0);
   for (int t0 = 0; t0 < n; t0 += kC) {
     const int m = min(kC, n - t0);
     __syncthreads();   // the previous chunk's reads are done (and pw is there, the first time)
-    if (owner) {
+    if (!SUM && owner) {
 #pragma unroll
       for (int a = 0; a < DT; ++a)
 #pragma unroll
@@ -233,41 +258,56 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(
         }
     }
 #pragma unroll
-    for (int i = 0; i < kKF; ++i) {
-      const int tt = (tid + 256 * i) / kKC, ch = (tid + 256 * i) % kKC;
-      const float f = pw[max(m - 1 - tt, 0)];
-      const int col = tok_col(tt) ^ (((ch >> 1) & 7) << 3);
-      u16x8 kb;
+    for (int i = 0; i < kKI; ++i) {
+      const int kq = (tid + 256 * i) / kKC, ch = (tid + 256 * i) % kKC;
+      if (kq < 16) {
+        const int col = tok_col(4 * kq) ^ (((ch >> 1) & 7) << 3);
+        float f[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          f[j] = pw[max(m - 1 - (4 * kq + j), 0)];   // rows past the end are zero
+#pragma unroll
+          for (int e = 0; e < 8; ++e) kf[i][j][e] = f32_to_bf16(silu_fast(bf16_to_f32(kf[i][j][e])));
+          if (!SUM) *reinterpret_cast<u16x8*>(kr + (4 * kq + j) * KLd + 8 * ch) = kf[i][j];
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          u16x4 hi, lo;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const float x = f[j] * bf16_to_f32(kf[i][j][e]);
+            hi[j] = f32_to_bf16(x);
+            lo[j] = f32_to_bf16(x - bf16_to_f32(hi[j]));
+          }
+          *reinterpret_cast<u16x4*>(kth + (8 * ch + e) * kTLd + col) = hi;
+          *reinterpret_cast<u16x4*>(ktl + (8 * ch + e) * kTLd + col) = lo;
+        }
+      }
+    }
+    if (vq < 16) {
+      const int col = tok_col(4 * vq) ^ (((vch >> 1) & 7) << 3);
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        kb[e] = f32_to_bf16(silu_fast(bf16_to_f32(kf[i][e])));
-        const float x = f * bf16_to_f32(kb[e]);
-        const unsigned short hi = f32_to_bf16(x);
-        kth[(8 * ch + e) * kTLd + col] = hi;
-        ktl[(8 * ch + e) * kTLd + col] = f32_to_bf16(x - bf16_to_f32(hi));
-      }
-      *reinterpret_cast<u16x8*>(kr + tt * KLd + 8 * ch) = kb;
-    }
+        u16x4 x;
 #pragma unroll
-    for (int i = 0; i < kVF; ++i) {
-      const int tt = (tid + 256 * i) / kVC, ch = (tid + 256 * i) % kVC;
-      if (tt < kC) {
-        const int col = tok_col(tt) ^ (((ch >> 1) & 7) << 3);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) vt[(8 * ch + e) * kTLd + col] = f32_to_bf16(silu_fast(bf16_to_f32(vf[i][e])));
+        for (int j = 0; j < 4; ++j) x[j] = f32_to_bf16(silu_fast(bf16_to_f32(vf[j][e])));
+        *reinterpret_cast<u16x4*>(vt + (8 * vch + e) * kTLd + col) = x;
       }
     }
     bf16x8 q[KS];
+    if constexpr (!SUM) {
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      u16x8 x;
+      for (int ks = 0; ks < KS; ++ks) {
+        u16x8 x;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] = f32_to_bf16(silu_fast(bf16_to_f32(qf[ks][e])));
-      q[ks] = __builtin_bit_cast(bf16x8, x);
+        for (int e = 0; e < 8; ++e) x[e] = f32_to_bf16(silu_fast(bf16_to_f32(qf[ks][e])));
+        q[ks] = __builtin_bit_cast(bf16x8, x);
+      }
     }
     __syncthreads();
     if (t0 + kC < n) fetch(t0 + kC);   // the next chunk's loads fly during this chunk's math
     auto frag = [&](const unsigned short* p) { return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u16x8*>(p)); };
+    if constexpr (!SUM) {
     // what the state before the chunk gives: O^T tiles, lane (c, g) holds columns 16 b + 4 g + i of row 16 wave + c
     f32x4 acc[NT];
 #pragma unroll
@@ -327,6 +367,7 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(
       for (int b = 0; b < NT; ++b)
         if (vb0 + 16 * b + 4 * g < vdim) *reinterpret_cast<f32x4*>(dst + 16 * b + 4 * g) = acc[b];
     }
+    }
     if (owner) {
       const float f = pw[m];
 #pragma unroll
@@ -348,6 +389,7 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(
       }
     }
   }
+  if (!SUM && !last) return;
 #pragma unroll
   for (int a = 0; a < DT; ++a)
 #pragma unroll
@@ -359,16 +401,57 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(
       }
 }
 
-template <int KS, int NT>
-void launch_chunk(float* o, float* S, const unsigned short* proj, long ld, const float* powers, const int* seq_cu,
-                  const int* seq_ctx, const int* seq_state, int nseq, int heads, int dim, int vdim, hipStream_t s) {
-  constexpr size_t smem = chunk_lds<KS, NT>();
+// ws[s, seg, head]: a segment's own sum on entry (all but the last segment's), the state before the segment on exit.
+// grid (ceil(dim * vdim / 256), heads, sequences)
+__global__ __launch_bounds__(256) void lightning_carry_kernel(float* __restrict__ ws, const float* __restrict__ S,
+                                                             const float* __restrict__ powers,
+                                                             const int* __restrict__ seq_cu,
+                                                             const int* __restrict__ seq_ctx,
+                                                             const int* __restrict__ seq_state, int heads, int dv,
+                                                             int nseg, int seg_len) {
+  const int s = blockIdx.z, h = blockIdx.y, e = blockIdx.x * 256 + threadIdx.x;
+  if (e >= dv) return;
+  const int n = seq_cu[s + 1] - seq_cu[s];
+  float f = 1.f;   // decay^seg_len
+  for (int i = 0; i < seg_len; i += 64) f *= powers[h * kPowers + 64];
+  float cur = seq_ctx[s] - n > 0 ? S[((long)seq_state[s] * heads + h) * dv + e] : 0.f;
+  float* p = ws + ((long)s * nseg * heads + h) * dv + e;
+  const long step = (long)heads * dv;
+  for (int at = 0; at < n; at += seg_len, p += step) {
+    const float own = at + seg_len < n ? *p : 0.f;
+    *p = cur;
+    cur = __builtin_fmaf(f, cur, own);
+  }
+}
+
+template <int KS, int NT, bool SUM>
+void launch_chunk1(float* o, float* S, const unsigned short* proj, long ld, const float* powers, const int* seq_cu,
+                   const int* seq_ctx, const int* seq_state, int nseq, int heads, int dim, int vdim, float* ws, int nseg,
+                   int seg_len, hipStream_t s) {
+  constexpr size_t smem = chunk_lds<KS, NT, SUM>();
   static_assert(smem <= 160 * 1024, "LDS");
-  static const bool ok = hipFuncSetAttribute(reinterpret_cast<const void*>(&lightning_chunk_kernel<KS, NT>),
+  static const bool ok = hipFuncSetAttribute(reinterpret_cast<const void*>(&lightning_chunk_kernel<KS, NT, SUM>),
                                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess;
   (void)ok;
-  lightning_chunk_kernel<KS, NT><<<dim3(heads, (vdim + 16 * NT - 1) / (16 * NT), nseq), 256, smem, s>>>(
-      o, S, proj, ld, powers, seq_cu, seq_ctx, seq_state, heads, dim, vdim);
+  lightning_chunk_kernel<KS, NT, SUM><<<dim3(heads, (vdim + 16 * NT - 1) / (16 * NT), nseq * nseg), 256, smem, s>>>(
+      o, S, proj, ld, powers, seq_cu, seq_ctx, seq_state, heads, dim, vdim, ws, nseg, seg_len);
+}
+
+template <int KS>
+void launch_chunk(float* o, float* S, const unsigned short* proj, long ld, const float* powers, const int* seq_cu,
+                  const int* seq_ctx, const int* seq_state, int nseq, int heads, int dim, int vdim, float* ws, int nseg,
+                  int seg_len, hipStream_t s) {
+  // narrow column blocks (two workgroups per CU) while wide ones leave compute units idle
+  const bool narrow = vdim <= 32 || (long)nseq * nseg * heads * ((vdim + 63) / 64) < 512;
+  if (nseg > 1) {
+    launch_chunk1<KS, 4, true>(o, S, proj, ld, powers, seq_cu, seq_ctx, seq_state, nseq, heads, dim, vdim, ws, nseg, seg_len, s);
+    lightning_carry_kernel<<<dim3((dim * vdim + 255) / 256, heads, nseq), 256, 0, s>>>(
+        ws, S, powers, seq_cu, seq_ctx, seq_state, heads, dim * vdim, nseg, seg_len);
+  }
+  if (narrow)
+    launch_chunk1<KS, 2, false>(o, S, proj, ld, powers, seq_cu, seq_ctx, seq_state, nseq, heads, dim, vdim, ws, nseg, seg_len, s);
+  else
+    launch_chunk1<KS, 4, false>(o, S, proj, ld, powers, seq_cu, seq_ctx, seq_state, nseq, heads, dim, vdim, ws, nseg, seg_len, s);
 }
 
 // ---------------------------------------------------------------- one row per sequence
@@ -490,19 +573,19 @@ __global__ __launch_bounds__(256) void lightning_out_kernel(T* __restrict__ out,
 template <typename T>
 void run(void* out, long out_ld, float* S, const void* proj_, long ld, const float* powers, const float* norm_w,
          const int* seq_cu, const int* seq_ctx, const int* seq_state, int nseq, int npf, int T_rows, int pf_rows,
-         float* scratch, int heads, int dim, int vdim, float eps, float out_scale, bool mfma, hipStream_t s) {
+         float* scratch, int heads, int dim, int vdim, float eps, float out_scale, bool mfma, int nseg, int seg_len,
+         hipStream_t s) {
   const T* proj = static_cast<const T*>(proj_);
   const int N = heads * vdim;
   float* o = scratch;                              // [T_rows, heads * vdim]
   if (npf > 0 && mfma) {
     if constexpr (sizeof(T) == 2) {
       auto p = reinterpret_cast<const unsigned short*>(proj);
-#define HS_LC(KS, NT) launch_chunk<KS, NT>(o, S, p, ld, powers, seq_cu, seq_ctx, seq_state, npf, heads, dim, vdim, s)
-      // narrower column blocks while the wide ones leave compute units idle
-      const bool narrow = vdim <= 32 || (long)npf * heads * ((vdim + 63) / 64) < 256;
-      if (dim <= 32) { if (narrow) HS_LC(1, 2); else HS_LC(1, 4); }
-      else if (dim <= 64) { if (narrow) HS_LC(2, 2); else HS_LC(2, 4); }
-      else { if (narrow) HS_LC(4, 2); else HS_LC(4, 4); }
+      float* ws = o + (long)T_rows * N;              // nseg > 1: [npf, nseg, heads, dim, vdim]
+#define HS_LC(KS) launch_chunk<KS>(o, S, p, ld, powers, seq_cu, seq_ctx, seq_state, npf, heads, dim, vdim, ws, nseg, seg_len, s)
+      if (dim <= 32) HS_LC(1);
+      else if (dim <= 64) HS_LC(2);
+      else HS_LC(4);
 #undef HS_LC
     }
   } else if (npf > 0) {
@@ -556,14 +639,14 @@ bool lightning_mfma_ok(int dim, int vdim, long ld, long offset) {
 void launch_lightning(void* out, long out_ld, float* S, const void* proj, long ld, const float* powers,
                       const float* norm_w, const int* seq_cu, const int* seq_ctx, const int* seq_state, int nseq,
                       int npf, int T, int pf_rows, float* scratch, int heads, int dim, int vdim, float eps,
-                      float out_scale, bool mfma, bool f32, hipStream_t s) {
+                      float out_scale, bool mfma, int nseg, int seg_len, bool f32, hipStream_t s) {
   if (nseq <= 0 || T <= 0) return;
   if (f32)
     run<float>(out, out_ld, S, proj, ld, powers, norm_w, seq_cu, seq_ctx, seq_state, nseq, npf, T, pf_rows, scratch,
-               heads, dim, vdim, eps, out_scale, false, s);
+               heads, dim, vdim, eps, out_scale, false, 1, 0, s);
   else
     run<unsigned short>(out, out_ld, S, proj, ld, powers, norm_w, seq_cu, seq_ctx, seq_state, nseq, npf, T, pf_rows,
-                        scratch, heads, dim, vdim, eps, out_scale, mfma, s);
+                        scratch, heads, dim, vdim, eps, out_scale, mfma, nseg, seg_len, s);
 }
 
 }  // namespace hipserve

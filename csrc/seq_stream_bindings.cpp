@@ -67,7 +67,8 @@ bool lightning_mfma_ok(int64_t dim, int64_t vdim, int64_t ld, int64_t offset) {
 void lightning(at::Tensor& out, at::Tensor& S, const at::Tensor& proj, const at::Tensor& powers,
                const at::Tensor& norm_w, const at::Tensor& seq_cu, const at::Tensor& seq_ctx,
                const at::Tensor& seq_state, at::Tensor& scratch, int64_t npf, int64_t pf_rows, int64_t heads, int64_t dim,
-               int64_t vdim, double eps, double out_scale, bool mfma) {
+               int64_t vdim, double eps, double out_scale, bool mfma, int64_t nseg, int64_t seg_len,
+               int64_t max_q) {
   CHECK_DEV(proj); CHECK_F32(S); CHECK_F32(powers); CHECK_F32(norm_w); CHECK_F32(scratch);
   CHECK_I32(seq_cu); CHECK_I32(seq_ctx); CHECK_I32(seq_state);
   const bool f32 = is_f32(proj, "lightning");
@@ -82,12 +83,16 @@ void lightning(at::Tensor& out, at::Tensor& S, const at::Tensor& proj, const at:
               "lightning: prompt portions first, then one row per sequence");
   TORCH_CHECK(!mfma || (!f32 && hipserve::lightning_mfma_ok(dim, vdim, proj.stride(0), proj.storage_offset())),
               "lightning: the chunk kernel takes bf16 and heads of multiples of 8 elements, keys up to 128");
-  TORCH_CHECK(scratch.numel() >= T * N + ((npf > 0 && !mfma) ? pf_rows * heads * (2 * dim + vdim) : 0));
+  TORCH_CHECK(nseg >= 1 && (nseg == 1 || (seg_len > 0 && seg_len % 64 == 0 && nseg * seg_len >= max_q)) && npf * nseg <= 65535,
+              "lightning: segments of a multiple of 64 tokens that cover the longest portion");
+  TORCH_CHECK(npf == 0 || scratch.numel() >= T * N + (!mfma ? pf_rows * heads * (2 * dim + vdim)
+                                                          : nseg > 1 ? npf * nseg * heads * dim * vdim : 0));
+  TORCH_CHECK(scratch.numel() >= T * N);
   c10::hip::HIPGuardMasqueradingAsCUDA g(proj.device());
   hipserve::launch_lightning(out.data_ptr(), out.stride(0), S.data_ptr<float>(), proj.data_ptr(), proj.stride(0),
                              powers.data_ptr<float>(), norm_w.data_ptr<float>(), seq_cu.data_ptr<int>(),
                              seq_ctx.data_ptr<int>(), seq_state.data_ptr<int>(), nseq, npf, T, pf_rows,
-                             scratch.data_ptr<float>(), heads, dim, vdim, (float)eps, (float)out_scale, mfma, f32,
+                             scratch.data_ptr<float>(), heads, dim, vdim, (float)eps, (float)out_scale, mfma, nseg, seg_len, f32,
                              cur_stream());
 }
 
@@ -99,7 +104,7 @@ TORCH_LIBRARY(hipserve_stream, m) {
         "Tensor? y2, Tensor? ye, Tensor? pair_slot, Tensor? wts, int top, Tensor? shared, Tensor? gate) -> ()");
   m.def("lightning(Tensor(a!) out, Tensor(b!) S, Tensor proj, Tensor powers, Tensor norm_w, Tensor seq_cu, "
         "Tensor seq_ctx, Tensor seq_state, Tensor(c!) scratch, int npf, int pf_rows, int heads, int dim, int vdim, "
-        "float eps, float out_scale, bool mfma) -> ()");
+        "float eps, float out_scale, bool mfma, int nseg, int seg_len, int max_q) -> ()");
   m.def("lightning_mfma_ok(int dim, int vdim, int ld, int offset) -> bool", &lightning_mfma_ok);
 }
 

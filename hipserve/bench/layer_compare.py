@@ -5,7 +5,9 @@ Fikizen beside a dense sliding-window model (grouped-query attention + gated den
 feed-forward), Kemavik beside Fikizen (the other design that mixes attention layers with
 linear recurrences; its attention has no window), Topezen beside Kemavik (attention layers, a
 matrix-valued recurrence and routed experts with a shared expert in both) and beside Kesirax (the
-other design with latent attention). Random-init weights, synthetic prompts, a few layers of each (the per-layer
+other design with latent attention), Zinavik beside Topezen (window attention with kept first
+tokens, a matrix-valued recurrence and routed experts in both) and beside Fikizen (the other
+design with parallel mixers). Random-init weights, synthetic prompts, a few layers of each (the per-layer
 cost is what is compared). ``--layer-models`` picks the models; the ratios are given per pair.
 
 Per size and model, through the engine's own scheduler and step function:
@@ -118,10 +120,30 @@ def topezen_config(name, s):
                          bos_token_id=1)
 
 
+def zinavik_config(name, s):
+    """Four layers, each window attention (64 kept first tokens) and lightning attention side by side + routed experts.
+    Each half has half of the heads, so a layer's mixer holds about as many weights as one full-width mixer of the
+    designs beside it. Four residual streams."""
+    from ..config import (HybridLayerSpec, LightningSpec, ParallelMixerSpec, RoutedMoESpec, WindowAttentionSpec,
+                          YarnScaling, ZinavikConfig)
+
+    H = s["heads"] // 2
+    attn = WindowAttentionSpec(heads=H, kv_heads=max(1, H // 4), dim=128, vdim=128, scale=128 ** -0.5, window=s["window"],
+                               keep_first=64, rot_dims=128, rot_base=1e6, yarn=YarnScaling(4.0, 4096, 32.0, 1.0),
+                               interleaved=True, unit_qk=True, channel_gate=True)
+    lightning = LightningSpec(heads=H, dim=128, vdim=128, decay=tuple(1.0 - 2.0 ** (-1 - 8 * (h + 1) / H) for h in range(H)))
+    moe = RoutedMoESpec(experts=s["experts"], top=s["top"], ff=s["ff"], limit=7.0, shared_ff=s["ff"], shared_limit=7.0,
+                        shared_gate=True, score="sigmoid", correction=False, weight_input=True, act="clamped")
+    layer = HybridLayerSpec(ParallelMixerSpec(attn, lightning, 0.75, 1.25), moe)
+    return ZinavikConfig(name=f"zinavik-{name}", hidden_size=s["width"], vocab_size=s["vocab"], layers=(layer,) * 4,
+                         streams=4, embed_scale=float(s["width"]) ** 0.5, max_position_embeddings=16384,
+                         eos_token_id=(2,), bos_token_id=1)
+
+
 MODELS = {"kesirax": kesirax_config, "mixtral": mixtral_config, "fikizen": fikizen_config, "dense": dense_config,
-          "kemavik": kemavik_config, "topezen": topezen_config}
+          "kemavik": kemavik_config, "topezen": topezen_config, "zinavik": zinavik_config}
 PAIRS = (("kesirax", "mixtral"), ("fikizen", "dense"), ("kemavik", "fikizen"), ("kemavik", "mixtral"),
-         ("topezen", "kemavik"), ("topezen", "kesirax"))
+         ("topezen", "kemavik"), ("topezen", "kesirax"), ("zinavik", "topezen"), ("zinavik", "fikizen"))
 
 
 def measure(mcfg, batch, prompt_len, new_tokens, device="cuda", repeats=2):

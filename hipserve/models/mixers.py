@@ -363,7 +363,7 @@ class WindowAttention:
 
         def rows(n):
             w = get(prefix + n)
-            if not s.interleaved or n not in ("q", "k"):
+            if not s.interleaved or not s.rot_dims or n not in ("q", "k"):
                 return w
             # the same permutation of every query and key head leaves scores and root mean squares unchanged and
             # turns the pairs (2i, 2i + 1) into the pairs (i, i + dims / 2) of the kernels

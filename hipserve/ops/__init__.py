@@ -461,6 +461,8 @@ class KernelOps:
 
     # bf16 prompt portions run the chunked matrix-core kernel (HIPSERVE_LIGHTNING_MFMA=0: the scan, as fp32 does)
     LIGHTNING_MFMA = os.environ.get("HIPSERVE_LIGHTNING_MFMA", "1") != "0"
+    LIGHTNING_SEGMENT = 256    # tokens per segment of long portions (a multiple of 64) ...
+    LIGHTNING_FILL = 1024      # ... while fewer (sequence, head, 32-column block) workgroups than this would run
 
     def lightning(self, out, S, proj, powers, norm_w, sp, eps, meta, out_scale=1.0):
         """Prompt portions (the step's first sequences) run the chunked kernel or the scan, decode rows the
@@ -471,9 +473,17 @@ class KernelOps:
         mfma = (npf > 0 and self.LIGHTNING_MFMA and proj.dtype == torch.bfloat16
                 and self._stream.lightning_mfma_ok(sp.dim, sp.vdim, proj.stride(0), proj.storage_offset()))
         rows = meta.num_prefill_tokens if npf and not mfma else 0   # the scan reads them as dense fp32 rows
-        scratch = torch.empty(T * sp.out_size + rows * sp.heads * (2 * sp.dim + sp.vdim), device=proj.device, dtype=torch.float32)
+        nseg, seg = 1, self.LIGHTNING_SEGMENT
+        blocks = npf * sp.heads * -(-sp.vdim // 32)
+        if mfma and meta.max_q >= 2 * seg and blocks < self.LIGHTNING_FILL:
+            while blocks * -(-meta.max_q // seg) > 4 * self.LIGHTNING_FILL:
+                seg *= 2
+            nseg = -(-meta.max_q // seg)
+        extra = npf * nseg * sp.heads * sp.dim * sp.vdim if nseg > 1 else rows * sp.heads * (2 * sp.dim + sp.vdim)
+        scratch = torch.empty(T * sp.out_size + extra, device=proj.device, dtype=torch.float32)
         self._stream.lightning(out, S, proj, powers, norm_w, meta.seq_cu, meta.seq_ctx, meta.seq_state, scratch, npf,
-                               meta.num_prefill_tokens, sp.heads, sp.dim, sp.vdim, eps, out_scale, mfma)
+                               meta.num_prefill_tokens, sp.heads, sp.dim, sp.vdim, eps, out_scale, mfma,
+                               nseg, seg, meta.max_q)
 
 
 class ReferenceOps:
