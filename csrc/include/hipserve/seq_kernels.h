@@ -71,6 +71,15 @@ int route_topk_max_outputs();
 void launch_route_topk(int* ids, float* wts, const float* logits, long ld, const float* correction, int T, int n,
                        int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s);
 
+// Router and expert alignment (moe_align's tables) of a small batch in one launch: T * top <= route_align_max_pairs(),
+// n <= route_topk_max_outputs() router outputs, nb <= 128 buckets (experts, and one more for the identity experts).
+// slots has `cap` entries (a multiple of tile, at least T * top + nb * (tile - 1) up to that multiple).
+int route_align_max_pairs();
+int route_align_max_slots();
+void launch_route_align(int* ids, float* wts, int* slots, int cap, int* tile_expert, int tile, int* pair_slot,
+                        const float* logits, long ld, const float* correction, int T, int n, int top, float scale, int E,
+                        int nb, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s);
+
 // Window attention on a paged cache [blocks, block_size, kv_heads * dim | kv_heads * vdim] (window_attention.hip).
 // attn_prepare: per row of proj = [q | k | v | ...]: optional RMS norm of q and k (norm_mode 0: none; 1: over the
 // whole projection, weights per element; 2: per head - and map - of `dim` elements, one weight of `dim` elements),
@@ -169,13 +178,15 @@ void launch_mlstm(void* out, float* S, float* N, float* M, const void* proj, lon
                   int nseq, int T, float* scratch, int heads, int dim, int vdim, float cap, float eps,
                   bool one_row_seqs, bool f32, hipStream_t s);
 
-// Residual streams (streams.hip): src fp32 [T, S, H] (one_row: [T, H], all streams equal to it), coef =
+// Residual streams (streams.hip): src fp32 [T, S, H] (one_row: all streams equal [T, H], or with `table` the embedding
+// table_scale * table[ids[t]] in the activation type), coef =
 // [M (S x S, from x to) | p1 | p2 | c]: x_t = sum_s M[s, t] src_s + p1[t] y1 + p2[t] y2; out = norm(sum_t c[t] x_t) * w;
 // dst (may be src or null) = x. y2: a row, or (y2 null, ye not) sum_j wts[t, j] ye[pair_slot[t top + j]] (wts null:
 // ones) + sigmoid(gate[t * gate_ld]) * shared (gate null: one).
 int stream_update_max_streams();
 int stream_update_max_width();
-void launch_stream_update(void* out, float* dst, const float* src, bool one_row, const float* coef, int S,
+void launch_stream_update(void* out, float* dst, const float* src, bool one_row, const void* table, const long* ids,
+                          long vocab, float table_scale, const float* coef, int S,
                           const float* w, int T, int H, float eps, const void* y1, const void* y2, const void* ye,
                           const int* pair_slot, const float* wts, int top, const void* shared, const float* gate,
                           long gate_ld, bool f32, hipStream_t s);

@@ -157,6 +157,32 @@ inline void route_topk(at::Tensor& ids, at::Tensor& wts, const at::Tensor& logit
                               sigmoid, cur_stream());
 }
 
+inline void route_align(at::Tensor& ids, at::Tensor& wts, at::Tensor& slots, at::Tensor& tile_expert,
+                        at::Tensor& pair_slot, const at::Tensor& logits, const c10::optional<at::Tensor>& correction,
+                        int64_t top, double scale, int64_t E, int64_t nb, int64_t tile, int64_t groups, int64_t keep,
+                        bool renorm, bool sigmoid) {
+  CHECK_DEV(logits); CHECK_F32(wts); CHECK_I32(ids); CHECK_I32(slots); CHECK_I32(tile_expert); CHECK_I32(pair_slot);
+  TORCH_CHECK(logits.scalar_type() == at::kFloat && rows2d(logits), "route_align: fp32 logits");
+  const long T = logits.size(0), n = logits.size(1), P = T * top, cap = slots.numel();
+  TORCH_CHECK(n >= 1 && n <= hipserve::route_topk_max_outputs() && top >= 1 && top <= n &&
+              P <= hipserve::route_align_max_pairs(), "route_align: a small batch");
+  if (correction.has_value()) {
+    CHECK_F32(*correction);
+    TORCH_CHECK(correction->numel() == n, "route_align: a correction per output");
+  }
+  TORCH_CHECK(ids.numel() == P && wts.numel() == P && pair_slot.numel() >= P && E >= 0 && E <= n);
+  TORCH_CHECK(nb >= 1 && nb <= 128 && nb >= std::min(E + (E < n ? 1 : 0), n), "route_align: a bucket per expert");
+  TORCH_CHECK(tile >= 1 && cap % tile == 0 && cap >= P + nb * (tile - 1) && cap <= hipserve::route_align_max_slots() &&
+              tile_expert.numel() == cap / tile, "route_align: slots cover the padding");
+  TORCH_CHECK(groups >= 1 && groups <= 64 && n % groups == 0 && keep >= 1 && keep <= groups &&
+              (groups == 1 || keep * (n / groups) >= top), "route_align: groups of equal size that can hold the choice");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(logits.device());
+  hipserve::launch_route_align(ids.data_ptr<int>(), wts.data_ptr<float>(), slots.data_ptr<int>(), cap,
+                               tile_expert.data_ptr<int>(), tile, pair_slot.data_ptr<int>(), logits.data_ptr<float>(),
+                               logits.stride(0), (const float*)opt_ptr(correction), T, n, top, (float)scale, E, nb,
+                               groups, keep, renorm, sigmoid, cur_stream());
+}
+
 inline void polynorm(at::Tensor& out, const at::Tensor& x, const at::Tensor& coef, double eps) {
   CHECK_DEV(x); CHECK_F32(coef);
   const bool f32 = is_f32(x, "polynorm");
@@ -196,6 +222,9 @@ inline void def_window_ops(torch::Library& m) {
   m.def("activation(Tensor(a!) out, Tensor x, int kind, float c0, float c1) -> ()");
   m.def("route_topk(Tensor(a!) ids, Tensor(b!) wts, Tensor logits, Tensor? correction, int top, float scale, int E, "
         "int groups, int keep, bool renorm, bool sigmoid=False) -> ()");
+  m.def("route_align(Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) slots, Tensor(d!) tile_expert, Tensor(e!) pair_slot, "
+        "Tensor logits, Tensor? correction, int top, float scale, int E, int nb, int tile, int groups, int keep, "
+        "bool renorm, bool sigmoid) -> ()");
   def_moe_ops(m);
 }
 
@@ -205,6 +234,7 @@ inline void impl_window_ops(torch::Library& m) {
   m.impl("window_attention_mfma", &window_attention_mfma);
   m.impl("activation", &activation);
   m.impl("route_topk", &route_topk);
+  m.impl("route_align", &route_align);
   impl_moe_ops(m);
 }
 

@@ -15,21 +15,18 @@ namespace {
 
 constexpr int kSlots = 4;
 
-__global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, float* __restrict__ wts,
-                                                         const float* __restrict__ logits, long ld,
-                                                         const float* __restrict__ correction, int T, int n, int top,
-                                                         float scale, int E, int groups, int keep, bool renorm,
-                                                         bool sigmoid) {
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+// One wave routes token t; ids_row / wts_row take its `top` choices, lds_ids (may be null) the ids once more.
+HS_DEVICE void route_token(int* __restrict__ ids_row, float* __restrict__ wts_row, int* lds_ids,
+                           const float* __restrict__ row, const float* __restrict__ correction, int n, int top,
+                           float scale, int E, int groups, int keep, bool renorm, bool sigmoid) {
   const int lane = threadIdx.x & 63;
-  if (t >= T) return;
   float p[kSlots], c[kSlots];
   float z[kSlots];
   float mx = -INFINITY;
 #pragma unroll
   for (int s = 0; s < kSlots; ++s) {
     const int e = lane + 64 * s;
-    z[s] = e < n ? logits[(long)t * ld + e] : -INFINITY;
+    z[s] = e < n ? row[e] : -INFINITY;
     mx = fmaxf(mx, z[s]);
   }
   mx = wave_max(mx);
@@ -91,7 +88,8 @@ __global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, 
 #pragma unroll
     for (int s = 0; s < kSlots; ++s) {
       if (who == lane + 64 * s) {
-        ids[(long)t * top + j] = min(who, E);
+        ids_row[j] = min(who, E);
+        if (lds_ids != nullptr) lds_ids[j] = min(who, E);
         mine[s] = j;
         chosen += p[s];
         c[s] = -INFINITY;
@@ -101,10 +99,78 @@ __global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, 
   const float f = renorm ? scale / (wave_sum(chosen) + 1e-20f) : scale;
 #pragma unroll
   for (int s = 0; s < kSlots; ++s)
-    if (mine[s] >= 0) wts[(long)t * top + mine[s]] = p[s] * f;
+    if (mine[s] >= 0) wts_row[mine[s]] = p[s] * f;
+}
+
+__global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, float* __restrict__ wts,
+                                                         const float* __restrict__ logits, long ld,
+                                                         const float* __restrict__ correction, int T, int n, int top,
+                                                         float scale, int E, int groups, int keep, bool renorm,
+                                                         bool sigmoid) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t >= T) return;
+  route_token(ids + (long)t * top, wts + (long)t * top, nullptr, logits + (long)t * ld, correction, n, top, scale, E,
+              groups, keep, renorm, sigmoid);
+}
+
+// ---- router and alignment of a small batch in one workgroup: the choices go to LDS, pair p's place among the
+// pairs of its bucket is the number of earlier pairs there (as many LDS reads as there are pairs), and the
+// tables are put together in LDS and written once.
+constexpr int kAlignThreads = 1024, kMaxPairs = 256, kMaxBuckets = 128, kMaxSlots = 8192;
+
+__global__ __launch_bounds__(kAlignThreads) void route_align_kernel(
+    int* __restrict__ ids, float* __restrict__ wts, int* __restrict__ slots, int cap, int* __restrict__ tile_expert,
+    int tile, int* __restrict__ pair_slot, const float* __restrict__ logits, long ld,
+    const float* __restrict__ correction, int T, int n, int top, float scale, int E, int nb, int groups, int keep,
+    bool renorm, bool sigmoid) {
+  __shared__ int sid[kMaxPairs], cnt[kMaxBuckets], off[kMaxBuckets];
+  extern __shared__ int tab[];   // [cap] slots, [cap / tile] experts
+  const int tid = threadIdx.x, P = T * top, nt = cap / tile;
+  for (int t = tid >> 6; t < T; t += kAlignThreads / 64)
+    route_token(ids + (long)t * top, wts + (long)t * top, sid + t * top, logits + (long)t * ld, correction, n, top, scale,
+                E, groups, keep, renorm, sigmoid);
+  for (int i = tid; i < cap + nt; i += kAlignThreads) tab[i] = -1;
+  __syncthreads();
+  int rank = 0;
+  if (tid < P) {
+    const int e = sid[tid];
+    for (int p = 0; p < tid; ++p) rank += sid[p] == e;
+  } else if (tid >= 512 && tid < 512 + nb) {
+    int c = 0;
+    for (int p = 0; p < P; ++p) c += sid[p] == tid - 512;
+    cnt[tid - 512] = (c + tile - 1) / tile;   // tiles of the bucket
+  }
+  __syncthreads();
+  if (tid < nb) {
+    int at = 0;
+    for (int e = 0; e < tid; ++e) at += cnt[e];
+    off[tid] = at;
+    for (int k = 0; k < cnt[tid]; ++k) tab[cap + at + k] = tid;
+  }
+  __syncthreads();
+  if (tid < P) {
+    const int slot = off[sid[tid]] * tile + rank;
+    tab[slot] = tid;
+    pair_slot[tid] = slot;
+  }
+  __syncthreads();
+  for (int i = tid; i < cap; i += kAlignThreads) slots[i] = tab[i];
+  for (int i = tid; i < nt; i += kAlignThreads) tile_expert[i] = tab[cap + i];
 }
 
 }  // namespace
+
+int route_align_max_pairs() { return kMaxPairs; }
+int route_align_max_slots() { return kMaxSlots; }
+
+void launch_route_align(int* ids, float* wts, int* slots, int cap, int* tile_expert, int tile, int* pair_slot,
+                        const float* logits, long ld, const float* correction, int T, int n, int top, float scale, int E,
+                        int nb, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s) {
+  if (T <= 0) return;
+  route_align_kernel<<<1, kAlignThreads, (size_t)(cap + cap / tile) * sizeof(int), s>>>(
+      ids, wts, slots, cap, tile_expert, tile, pair_slot, logits, ld, correction, T, n, top, scale, E, nb, groups, keep,
+      renorm, sigmoid);
+}
 
 int route_topk_max_outputs() { return 64 * kSlots; }
 

@@ -1,5 +1,6 @@
 // Update of S residual streams between two sublayers, the next sublayer's input and its norm, one
-// workgroup per token row (fp32 streams [T, S, H], or one row [T, H] that all S streams equal):
+// workgroup per token row (fp32 streams [T, S, H]; or all S streams equal one row, src [T, H] or the embedding
+// scale * table[ids[t]], so the first layer needs no embedding pass of its own):
 //   x_t = sum_s M[s, t] src_s + p1[t] y1 + p2[t] y2
 //   u = sum_t c[t] x_t,   out = u / sqrt(mean(u^2) + eps) * w,   dst_t = x_t (dst null: not written)
 // y2 = a sublayer's row, or a mixture's output
@@ -49,7 +50,8 @@ template <> struct Row<unsigned short, 4> {
 // SS streams (0: n_streams, at most kMaxStreams); V channels per thread and step (H % V == 0).
 template <typename T, int SS, int V>
 __global__ __launch_bounds__(kNT) void stream_update_kernel(
-    T* __restrict__ out, float* dst, const float* src, bool one_row, const float* __restrict__ coef, int n_streams,
+    T* __restrict__ out, float* dst, const float* src, bool one_row, const T* __restrict__ table,
+    const long* __restrict__ ids, long vocab, float table_scale, const float* __restrict__ coef, int n_streams,
     const float* __restrict__ w, int H, float eps, const T* __restrict__ y1, const T* __restrict__ y2,
     const T* __restrict__ ye, const int* __restrict__ pair_slot, const float* __restrict__ wts, int top,
     const T* __restrict__ shared, const float* __restrict__ gate, long gate_ld) {
@@ -65,13 +67,19 @@ __global__ __launch_bounds__(kNT) void stream_update_kernel(
   const float* p2 = p1 + S;
   const float* c = p2 + S;
   const float* xrow = src + t * (one_row ? 1L : (long)S) * H;
+  const T* erow = table != nullptr ? table + min(max(ids[t], 0L), vocab - 1) * H : nullptr;
   const float sg = gate != nullptr ? sigmoid_f(gate[t * gate_ld]) : 1.f;
   float sq = 0.f;
   for (int e = V * tid; e < H; e += V * kNT) {
     float x[N][V];
 #pragma unroll kUn
     for (int s = 0; s < S; ++s) {
-      if (s == 0 || !one_row) Row<float, V>::ld(xrow + (long)s * H + e, x[s]);
+      if (table == nullptr && (s == 0 || !one_row)) Row<float, V>::ld(xrow + (long)s * H + e, x[s]);
+    }
+    if (table != nullptr) {
+      Row<T, V>::ld(erow + e, x[0]);
+#pragma unroll
+      for (int i = 0; i < V; ++i) x[0][i] *= table_scale;
     }
     float a[V], b[V];
 #pragma unroll
@@ -133,7 +141,8 @@ __global__ __launch_bounds__(kNT) void stream_update_kernel(
 int stream_update_max_streams() { return kMaxStreams; }
 int stream_update_max_width() { return 15000; }   // u waits in 60 KB of LDS
 
-void launch_stream_update(void* out, float* dst, const float* src, bool one_row, const float* coef, int S,
+void launch_stream_update(void* out, float* dst, const float* src, bool one_row, const void* table, const long* ids,
+                          long vocab, float table_scale, const float* coef, int S,
                           const float* w, int T, int H, float eps, const void* y1, const void* y2, const void* ye,
                           const int* pair_slot, const float* wts, int top, const void* shared, const float* gate,
                           long gate_ld, bool f32, hipStream_t s) {
@@ -141,8 +150,8 @@ void launch_stream_update(void* out, float* dst, const float* src, bool one_row,
   const size_t smem = (size_t)H * sizeof(float);
   const bool v4 = H % 4 == 0;
 #define HS_SU(TT, SS, V)                                                                                             \
-  stream_update_kernel<TT, SS, V><<<T, kNT, smem, s>>>((TT*)out, dst, src, one_row, coef, S, w, H, eps, (const TT*)y1,  \
-                                                       (const TT*)y2, (const TT*)ye, pair_slot, wts, top,            \
+  stream_update_kernel<TT, SS, V><<<T, kNT, smem, s>>>((TT*)out, dst, src, one_row, (const TT*)table, ids, vocab,       \
+                                                       table_scale, coef, S, w, H, eps, (const TT*)y1, (const TT*)y2, (const TT*)ye, pair_slot, wts, top,            \
                                                        (const TT*)shared, gate, gate_ld)
 #define HS_SS(TT, V)                          \
   switch (S) {                                \

@@ -467,9 +467,13 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
                                 seq1, rows_bound, heads, kv_heads, dim, vdim, gate_off, scale, window, sink,          \
                                 out_scale, nparts, part_keys, ws_acc, ws_ml, row_base, lam, post, eps, keep, softcap,  \
                                 sink_w, channel_gate, s)
-  // two row tiles per wave where a prompt portion brings enough rows and the accumulators fit the registers
+  // two row tiles per wave where a prompt portion brings enough rows and the accumulators fit the registers, except
+  // where 128-row workgroups would all be resident at once (two per CU): the rows with few visible keys then leave their
+  // CU idle, and twice as many smaller workgroups even that out (8192 rows x 8 heads: 183 -> 143 us)
+  const long wide_wgs = (long)rows_bound * heads / 128;
   const int ks = (dim + 31) / 32, nv = (vdim + 15) / 16;
-  const bool wide = nparts == 1 && (long)rows_bound * (heads / kv_heads) >= 128 * (long)(seq1 - seq0);
+  const bool wide = nparts == 1 && (long)rows_bound * (heads / kv_heads) >= 128 * (long)(seq1 - seq0) &&
+                    (wide_wgs < 64 || wide_wgs >= 1024);
   if (maps == 2) {
     // row tiles come in pairs (the two maps): 64 rows per workgroup. Four tiles per wave (128 rows) measured
     // slower on 4 x 2048-row prompts (532 against 396 us with 64-dim maps and 128-dim values): too many registers.

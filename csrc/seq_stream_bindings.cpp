@@ -16,22 +16,33 @@ namespace {
 
 using namespace hipserve_shared;
 
-void stream_update(at::Tensor& out, const c10::optional<at::Tensor>& dst, const at::Tensor& src, const at::Tensor& coef,
+void stream_update(at::Tensor& out, const c10::optional<at::Tensor>& dst, const c10::optional<at::Tensor>& src,
+                   const c10::optional<at::Tensor>& table, const c10::optional<at::Tensor>& ids, double table_scale,
+                   const at::Tensor& coef,
                    const at::Tensor& w, double eps, const c10::optional<at::Tensor>& y1,
                    const c10::optional<at::Tensor>& y2, const c10::optional<at::Tensor>& ye,
                    const c10::optional<at::Tensor>& pair_slot, const c10::optional<at::Tensor>& wts, int64_t top,
                    const c10::optional<at::Tensor>& shared, const c10::optional<at::Tensor>& gate) {
-  CHECK_DEV(out); CHECK_CONTIG(out); CHECK_F32(src); CHECK_F32(coef); CHECK_F32(w);
+  CHECK_DEV(out); CHECK_CONTIG(out); CHECK_F32(coef); CHECK_F32(w);
   const bool f32 = is_f32(out, "stream_update");
-  TORCH_CHECK(out.dim() == 2 && (src.dim() == 2 || src.dim() == 3), "stream_update: out [T, H], src [T, S, H] or [T, H]");
+  TORCH_CHECK(out.dim() == 2 && src.has_value() != table.has_value(), "stream_update: streams or an embedding table");
   const long T = out.size(0), H = out.size(1);
-  const bool one_row = src.dim() == 2;
+  const bool one_row = !src.has_value() || src->dim() == 2;
   long S = 1;
   while (S * S + 3 * S < coef.numel()) ++S;
   TORCH_CHECK(S * S + 3 * S == coef.numel() && S <= hipserve::stream_update_max_streams(),
               "stream_update: coefficients of at most ", hipserve::stream_update_max_streams(), " streams");
   TORCH_CHECK(H <= hipserve::stream_update_max_width(), "stream_update: width");
-  TORCH_CHECK(src.size(0) == T && src.size(-1) == H && (one_row || src.size(1) == S) && w.numel() == H);
+  TORCH_CHECK(w.numel() == H);
+  if (src.has_value()) {
+    CHECK_F32(*src);
+    TORCH_CHECK((src->dim() == 2 || src->dim() == 3) && src->size(0) == T && src->size(-1) == H &&
+                (one_row || src->size(1) == S), "stream_update: src [T, S, H] or [T, H]");
+  } else {
+    TORCH_CHECK(table->scalar_type() == out.scalar_type() && table->is_contiguous() && table->dim() == 2 &&
+                table->size(1) == H && table->size(0) >= 1 && ids.has_value() && ids->scalar_type() == at::kLong &&
+                ids->is_contiguous() && ids->numel() >= T, "stream_update: table [vocab, H] and one id per row");
+  }
   if (dst.has_value()) {
     CHECK_F32(*dst);
     TORCH_CHECK(dst->dim() == 3 && dst->size(0) == T && dst->size(1) == S && dst->size(2) == H);
@@ -54,8 +65,9 @@ void stream_update(at::Tensor& out, const c10::optional<at::Tensor>& dst, const 
   }
   c10::hip::HIPGuardMasqueradingAsCUDA g(out.device());
   hipserve::launch_stream_update(
-      out.data_ptr(), dst.has_value() ? dst->data_ptr<float>() : nullptr, src.data_ptr<float>(), one_row,
-      coef.data_ptr<float>(), S, w.data_ptr<float>(), T, H, (float)eps, opt_ptr(y1), opt_ptr(y2), opt_ptr(ye),
+      out.data_ptr(), dst.has_value() ? dst->data_ptr<float>() : nullptr, (const float*)opt_ptr(src), one_row,
+      opt_ptr(table), table.has_value() ? ids->data_ptr<long>() : nullptr, table.has_value() ? table->size(0) : 0,
+      (float)table_scale, coef.data_ptr<float>(), S, w.data_ptr<float>(), T, H, (float)eps, opt_ptr(y1), opt_ptr(y2), opt_ptr(ye),
       (const int*)opt_ptr(pair_slot), (const float*)opt_ptr(wts), top, ye.has_value() ? opt_ptr(shared) : nullptr,
       ye.has_value() ? (const float*)opt_ptr(gate) : nullptr, gate.has_value() ? gate->stride(0) : 0, f32, cur_stream());
 }
@@ -100,7 +112,7 @@ void lightning(at::Tensor& out, at::Tensor& S, const at::Tensor& proj, const at:
 
 TORCH_LIBRARY(hipserve_stream, m) {
   def_window_ops(m);
-  m.def("stream_update(Tensor(a!) out, Tensor(b!)? dst, Tensor src, Tensor coef, Tensor w, float eps, Tensor? y1, "
+  m.def("stream_update(Tensor(a!) out, Tensor(b!)? dst, Tensor? src, Tensor? table, Tensor? ids, float table_scale, Tensor coef, Tensor w, float eps, Tensor? y1, "
         "Tensor? y2, Tensor? ye, Tensor? pair_slot, Tensor? wts, int top, Tensor? shared, Tensor? gate) -> ()");
   m.def("lightning(Tensor(a!) out, Tensor(b!) S, Tensor proj, Tensor powers, Tensor norm_w, Tensor seq_cu, "
         "Tensor seq_ctx, Tensor seq_state, Tensor(c!) scratch, int npf, int pf_rows, int heads, int dim, int vdim, "

@@ -150,7 +150,8 @@ def build_kernels(force: bool = False, jobs: int = 8, verbose: bool = False, lib
                     if out.strip():
                         print(out, flush=True)
     so = os.path.join(PKG, so_name)
-    if tasks or not os.path.exists(so):
+    # an object shared with another library may have been compiled by that library's build
+    if tasks or not os.path.exists(so) or any(os.path.getmtime(o) > os.path.getmtime(so) for o in objs):
         # Link with the host toolchain and WITHOUT -lamdhip64: the HIP runtime
         # symbols resolve through libtorch_hip's own libamdhip64, so the process
         # never maps a second (system) HIP runtime next to torch's.

@@ -29,8 +29,8 @@ them is one op of the op set:
   decay bottleneck -> tanh -> decay up-projection (32-bit result) -> ``wkv`` (decay, bonus, the
   recurrence from the sequence's state slot, per-head output norm and SiLU gate) -> output
   projection.
-* routed experts (``RoutedMoE``): 32-bit router logits -> ``route_topk`` (softmax, corrected
-  selection, weights) -> ``moe_align`` tiles -> ``expert_gemm`` (gate | up, SiLU gate in its epilogue)
+* routed experts (``RoutedMoE``): 32-bit router logits -> ``route_align`` (scores, corrected
+  selection, weights, tiles; one launch for small batches) -> ``expert_gemm`` (gate | up, the gate in its epilogue)
   -> ``expert_gemm`` (down); the weighted combine, the identity experts and the shared
   expert are folded into the residual update (``add_normed``).
 * gated delta rule: merged [q | k | v | beta | decay | gate] projection -> ``gated_delta``
@@ -843,12 +843,13 @@ class RoutedMoE:
         if s.shared_gate:
             n = s.experts + s.identity
             logits, self.shared_gate = logits[:, :n], logits[:, n:]
-        ops.route_topk(ids, wts, logits, self.correction, s.top, s.scale, s.experts, s.groups, s.keep_groups, s.renorm,
-                       s.score)
+        router = (logits, self.correction, s.top, s.scale, s.experts)
+        options = (s.groups, s.keep_groups, s.renorm, s.score)
         scale = wts if s.weight_input else None
         # the identity experts share one bucket (s.experts) that no GEMM tile serves
         P, nb = T * s.top, s.experts + (1 if s.identity else 0)
         if self._packed_ok(h, P, nb):
+            ops.route_topk(ids, wts, *router, *options)
             ye, pair_slot = self._experts_packed(h, ids, P, nb, scale)
             return ye, pair_slot, ids, wts, s.experts, h, self._shared(h)
         tile = MOE_TILE_LARGE if P >= 4 * MOE_TILE_LARGE * nb else MOE_TILE
@@ -856,7 +857,7 @@ class RoutedMoE:
         slots = torch.empty(cap, dtype=torch.int32, device=dev)
         tile_expert = torch.empty(cap // tile, dtype=torch.int32, device=dev)
         pair_slot = torch.empty(P, dtype=torch.int32, device=dev)
-        ops.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
+        ops.route_align(ids, wts, slots, tile_expert, pair_slot, *router, nb, tile, *options)
         act = torch.empty(cap, s.ff, device=dev, dtype=h.dtype)
         # the gate and the pair's input weight in the epilogue
         ops.expert_gemm(act, h, self.w_gu, slots, tile_expert, tile, s.top, self.epilogue, scale, s.limit)

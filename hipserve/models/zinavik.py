@@ -23,7 +23,6 @@ once per layer, instead of read and written twice.
 from __future__ import annotations
 
 import torch
-import torch.nn.functional as F
 
 from .layer_list import LayerListModel
 from .mixers import RoutedMoE
@@ -103,16 +102,14 @@ class ZinavikModel(LayerListModel):
         if meta.id_src is not None:  # decode lookahead: row i's id is the previous step's sample tok[src[i]]
             src, tok = meta.id_src
             ids = torch.where(src >= 0, tok.index_select(0, src.clamp(min=0)), ids)
-        x = F.embedding(ids, self.embed).to(torch.float32, copy=True)
-        if cfg.embed_scale != 1.0:
-            x *= cfg.embed_scale
-        streams = torch.empty(T, cfg.streams, H, device=x.device, dtype=torch.float32)
+        streams = torch.empty(T, cfg.streams, H, device=ids.device, dtype=torch.float32)
+        # the streams' current value: all of them are the scaled embedding until the first layer's updates
+        x = (self.embed, ids, cfg.embed_scale)
 
         def norm_of(r):
             return self.final_norm if r == len(self.runs) else self.layers[self.runs[r][0]].norm1
 
-        # x: the streams' current value, [T, H] as long as all of them are the embedding
-        h = ops.stream_update(torch.empty(T, H, device=x.device, dtype=self.dtype), None, x, self.coef0, norm_of(0),
+        h = ops.stream_update(torch.empty(T, H, device=ids.device, dtype=self.dtype), None, x, self.coef0, norm_of(0),
                               cfg.norm_eps)
         for r, (i, _, _) in enumerate(self.runs):
             lw = self.layers[i]

@@ -389,6 +389,19 @@ class KernelOps:
         self._window_lib.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm,
                                     score == "sigmoid")
 
+    ROUTE_ALIGN_PAIRS, ROUTE_ALIGN_SLOTS = 256, 8192   # batches whose router and alignment run in one launch
+
+    def route_align(self, ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile, groups=1,
+                    keep_groups=1, renorm=False, score="softmax"):
+        """``route_topk`` and ``moe_align`` (``nb`` buckets) of the choices."""
+        if (ids.numel() <= self.ROUTE_ALIGN_PAIRS and slots.numel() <= self.ROUTE_ALIGN_SLOTS and nb <= 128 and groups <= 64
+                and logits.shape[1] <= self.ROUTER_MAX_OUTPUTS and self._window_lib is self._moe_lib):
+            self._window_lib.route_align(ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile,
+                                         groups, keep_groups, renorm, score == "sigmoid")
+            return
+        self.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+        self.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
+
     # ---- parallel blocks with gated sublayer results, mLSTM, PolyNorm (csrc/kernels/seq/gated_block.hip, mlstm.hip,
     # elementwise.hip)
     def gated_add_norms(self, out1, out2, residual, w1, w2, eps, first=None, second=None):
@@ -449,14 +462,20 @@ class KernelOps:
 
     # ---- residual streams, lightning attention (csrc/kernels/seq/streams.hip, lightning.hip)
     def stream_update(self, out, dst, src, coef, w, eps, y1=None, y2=None):
-        """``y2``: a sublayer's result rows or, for a mixture of experts, (ye, pair_slot, wts or top, shared, gate)."""
+        """``src``: the streams, or (table, ids, scale): all of them equal the embedding ``scale * table[ids]``. ``y2``: a
+        sublayer's result rows or, for a mixture of experts, (ye, pair_slot, wts or top, shared, gate)."""
+        table = ids = None
+        scale = 1.0
+        if isinstance(src, tuple):
+            table, ids, scale = src
+            src = None
         ye = pair_slot = wts = shared = gate = None
         top = 0
         if isinstance(y2, tuple):
             ye, pair_slot, wts, shared, gate = y2
             top, wts = (wts, None) if isinstance(wts, int) else (wts.shape[1], wts)
             y2 = None
-        self._stream.stream_update(out, dst, src, coef, w, eps, y1, y2, ye, pair_slot, wts, top, shared, gate)
+        self._stream.stream_update(out, dst, src, table, ids, scale, coef, w, eps, y1, y2, ye, pair_slot, wts, top, shared, gate)
         return out
 
     # bf16 prompt portions run the chunked matrix-core kernel (HIPSERVE_LIGHTNING_MFMA=0: the scan, as fp32 does)
@@ -641,6 +660,11 @@ class ReferenceOps:
     def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False,
                    score="softmax"):
         ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+
+    def route_align(self, ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile, groups=1,
+                    keep_groups=1, renorm=False, score="softmax"):
+        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+        ref.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
 
     def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta):
         ref.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta.seq_cu,

@@ -930,7 +930,8 @@ def mlstm(out, S, N, M, proj, gates, b_if, norm_w, sp, eps, seq_cu, seq_ctx, seq
 # attention with one fixed decay per head over state slots
 
 def stream_update(out, dst, src, coef, w, eps, y1=None, y2=None):
-    """src [T, S, H] are the residual streams (fp32), or [T, H]: all S streams equal to it. coef (fp32) holds
+    """src [T, S, H] are the residual streams (fp32), or [T, H]: all S streams equal to it, or (table, ids, scale): all
+    of them equal scale * table[ids]. coef (fp32) holds
     M [S, S] (from, to), p1 [S], p2 [S], c [S] one after the other:
       x_t = sum_s M[s, t] src_s + p1[t] y1 + p2[t] y2;   u = sum_t c[t] x_t;   out = u / rms(u) * w
     dst (may be src, or None) gets x. y1 [T, H]; y2 [T, H] or a mixture's parts (ye, pair_slot, wts, shared, gate):
@@ -939,6 +940,9 @@ def stream_update(out, dst, src, coef, w, eps, y1=None, y2=None):
     S = int(round((9 + 4 * n) ** 0.5 - 3) // 2)
     assert S * S + 3 * S == n
     M, p1, p2, c = coef[:S * S].view(S, S), coef[S * S:S * S + S], coef[S * S + S:S * S + 2 * S], coef[S * S + 2 * S:]
+    if isinstance(src, tuple):
+        table, ids, scale = src
+        src = table[ids].float() * scale
     x = src.float() if src.dim() == 3 else src.float().unsqueeze(1).expand(-1, S, -1)
     x = torch.einsum("st,nsh->nth", M, x)
     if y1 is not None:

@@ -293,6 +293,34 @@ def test_routed_experts_alone(target, shape):
     assert rel_err(x, want) < TOL[target[1]] and rel_err(out, O.rms_unit(want, EPS)) < TOL[target[1]]
 
 
+@pytest.mark.parametrize("target", TARGETS)
+@pytest.mark.parametrize("T,experts,identity,top,tile", [(1, 1, 0, 1, 32), (16, 16, 0, 2, 32), (128, 100, 3, 2, 32), (51, 7, 2, 5, 64),
+                                                         (3, 9, 0, 9, 32), (256, 128, 0, 1, 32), (129, 20, 0, 2, 32)])
+def test_router_and_alignment_in_one_launch(target, T, experts, identity, top, tile):
+    """Same choices and weights as the router alone; every pair sits in one slot of a tile of its expert."""
+    dev = torch.device(target[0])
+    ops = stream_ops(dev)
+    g = torch.Generator().manual_seed(T)
+    n, nb = experts + identity, experts + (1 if identity else 0)
+    logits = torch.randn(T, n + 3, generator=g).to(dev)[:, :n]
+    corr = torch.randn(n, generator=g).to(dev) if T % 2 else None
+    P = T * top
+    cap = -(-(P + nb * (tile - 1)) // tile) * tile
+    ids, wts = torch.empty(T, top, dtype=torch.int32, device=dev), torch.empty(T, top, device=dev)
+    slots, te, ps = (torch.full((k,), 77, dtype=torch.int32, device=dev) for k in (cap, cap // tile, P))
+    args = (logits, corr, top, 1.5, experts)
+    ops.route_align(ids, wts, slots, te, ps, *args, nb, tile, 1, 1, True, "sigmoid")
+    ids2, wts2 = torch.empty_like(ids), torch.empty_like(wts)
+    ops.route_topk(ids2, wts2, *args, 1, 1, True, "sigmoid")
+    assert torch.equal(ids, ids2) and torch.allclose(wts, wts2)
+    slots, te, ps, flat = slots.tolist(), te.tolist(), ps.tolist(), ids.view(-1).tolist()
+    assert sorted(p for p in slots if p >= 0) == list(range(P)) and all(p >= -1 for p in slots)
+    for p in range(P):
+        assert slots[ps[p]] == p and te[ps[p] // tile] == flat[p]
+    used = sum(-(-flat.count(e) // tile) for e in range(nb))
+    assert te[used:] == [-1] * (len(te) - used) and all(0 <= e < nb for e in te[:used])
+
+
 def test_experts_what_matters():
     """The weight on an expert's input is not a weight on its output; both limits, the one-sided clamp of the gate, the
     missing renormalisation and the shared expert's gate show."""
@@ -391,6 +419,11 @@ def test_stream_update_alone(target, S, width):
         assert torch.equal(src.cpu(), x) and rel_err(out, o) < tol          # not written back
         out = run(src, src, a.to(dev, dt) if a is not None else None, arg)  # in place
         assert torch.allclose(src.cpu().double(), xs, atol=2e-4, rtol=1e-4) and rel_err(out, o) < tol
+    table, ids = rnd(11, width).to(dt).float(), torch.tensor([3, 0, 10, 3, 7])
+    dst = torch.full((T, S, width), 9.0, device=dev)
+    xs, o = want(2.5 * table[ids][:, None].expand(T, S, width), y1.double(), None)
+    out = run((table.to(dev, dt), ids.to(dev), 2.5), dst, y1.to(dev, dt))
+    assert torch.allclose(dst.cpu().double(), xs, atol=2e-4, rtol=1e-4) and rel_err(out, o) < tol
     one = rnd(T, width)
     dst = torch.full((T, S, width), 9.0, device=dev)
     xs, o = want(one[:, None].expand(T, S, width), y1.double(), None)
