@@ -1,5 +1,5 @@
-// Prefill GEMM over the decode kernels' packed weight layout (VERDICT r3, next round item
-// 1: one weight layout for prefill and decode, hand-written MFMA on the prefill hot path):
+// Prefill GEMM over the decode kernels' packed weight layout (one weight layout for prefill and
+// decode, hand-written MFMA on the prefill hot path):
 //
 //   C[M, N] = X[M, K] . W[N, K]^T      bf16 in, fp32 accumulate, epilogue fused
 //
@@ -68,7 +68,7 @@ HS_DEVICE void pw_barrier() {
 }
 
 // MFMA on an AGPR accumulator as inline asm: with the builtin, hipcc moved the 256
-// accumulators between AGPRs inside the loop (tools/asm_stats.py: ~200 v_accvgpr moves
+// accumulators between AGPRs inside the loop (about 200 v_accvgpr moves
 // per 128 MFMAs). asm MFMAs are invisible to the hazard recognizer: the epilogue covers the
 // MFMA -> VALU read of the accumulators by hand.
 HS_DEVICE void pw_mfma(f32x4& acc, const u32x4& w, const u32x4& x) {
@@ -94,7 +94,7 @@ HS_DEVICE PwTile pw_make(int L, int tiles_m, int tiles_n, int wn, const unsigned
   const int tl = min(T.t, ntiles - 1);  // waves past the last weight tile compute a copy, store nothing
   // this m-tile's expert. readfirstlane: a load through a generic pointer counts as
   // divergent, which put the weight descriptor in VGPRs and wrapped every weight load of
-  // the main loop in a waterfall loop (tools/asm_stats.py: 197 VALU per loop body vs 0)
+  // the main loop in a waterfall loop (197 VALU instructions per loop body vs 0)
   if constexpr (kGroup) Wp += (long)__builtin_amdgcn_readfirstlane(grp.tile_expert[tm]) * grp.estride;
   T.w = __builtin_amdgcn_make_buffer_rsrc((void*)(Wp + (long)tl * KS * 32768), 0, KS * 65536, 0x00020000);
   if constexpr (kGather) {  // token rows through the slot table; padding slots read past the end = zero
@@ -207,7 +207,6 @@ __global__ __launch_bounds__(PW_T) __attribute__((amdgpu_waves_per_eu(1, 1))) vo
   // weight loads of one loop body all stream the same tile (nq % RW == 0): their buffer
   // resource and K offset are chosen once per body (wrs, wk), so a load costs one scalar
   // add — per-load selects cost ~6 SALU each and delayed the next MFMA group
-  // (tools/asm_stats.py)
   auto slot = [&](auto jc, int s0, const __amdgpu_buffer_rsrc_t& wrs, int wk) {
     constexpr int J = decltype(jc)::value, H = J & 1;
     const int s = s0 + J / 2, buf = s & 1;
