@@ -56,6 +56,22 @@ void launch_expert_gemm(void* out, const void* x, long x_ld, const void* w, cons
                         int ntiles_cap, int tile, int gather_k, int N, int K, int act, int E, const float* row_scale,
                         float limit, bool f32, hipStream_t s);
 
+// Norms before and after a sublayer (sandwich.hip): residual[T, H] (fp32, in place; `table` [vocab, H] in the activation
+// type: it starts as table_scale * table[ids[t]]) += mult * y / rms(y) * w_post; out = residual / rms(residual) * w_next.
+// y: rows `a` (b null); a_scale a / rms(a) * a_w + b_scale b / rms(b) * b_w; or (a null, ye not) a mixture's output
+// sum_j wts[t, j] ye[pair_slot[t top + j]] + sigmoid(gate[t * gate_ld]) * shared (gate null: one). a and ye null: no y.
+struct SandwichUpdate {
+  void* out; float* residual;
+  const float *w_next, *w_post;
+  int T, H; float eps, mult;
+  const void* table; const long* ids; long vocab; float table_scale;
+  const void *a, *b; const float *a_w, *b_w; float a_scale, b_scale;
+  const void* ye; const int* pair_slot; const float* wts; int top;
+  const void* shared; const float* gate; long gate_ld;
+};
+int sandwich_update_max_width();
+void launch_sandwich_update(const SandwichUpdate& p, bool f32, hipStream_t s);
+
 // Residual update with the norm on the sublayer's output (group_norm.hip): residual[T, H] (fp32, in place) +=
 // y / sqrt(mean(y^2) + eps) * w; out = residual in the activation type. y null: the addend is a mixture's output,
 // shared (or 0) + sum_j wts[t, j] * (ids[t, j] < E ? ye[pair_slot[t * top + j]] : h[t]).
@@ -65,11 +81,12 @@ void launch_add_normed(void* out, float* residual, const float* w, int T, int H,
 
 // Router (router.hip): s = softmax(logits[T, n]) or the sigmoid of each (rows of stride ld); the `top` largest
 // s + correction are chosen (ties: the lower index; correction null: the largest logits); ids[T, top] = min(index, E), wts[T, top] = s * scale. groups > 1: only outputs of the `keep`
-// groups (of n / groups neighbours) with the largest s + correction can be chosen; renorm: the chosen s are
+// groups (of n / groups neighbours) with the largest s + correction (top2: the largest sum of two) can be chosen; renorm: the chosen s are
 // divided by their sum + 1e-20 first.
 int route_topk_max_outputs();
 void launch_route_topk(int* ids, float* wts, const float* logits, long ld, const float* correction, int T, int n,
-                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s);
+                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, bool top2,
+                       hipStream_t s);
 
 // Router and expert alignment (moe_align's tables) of a small batch in one launch: T * top <= route_align_max_pairs(),
 // n <= route_topk_max_outputs() router outputs, nb <= 128 buckets (experts, and one more for the identity experts).
@@ -78,21 +95,22 @@ int route_align_max_pairs();
 int route_align_max_slots();
 void launch_route_align(int* ids, float* wts, int* slots, int cap, int* tile_expert, int tile, int* pair_slot,
                         const float* logits, long ld, const float* correction, int T, int n, int top, float scale, int E,
-                        int nb, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s);
+                        int nb, int groups, int keep, bool renorm, bool sigmoid, bool top2, hipStream_t s);
 
 // Window attention on a paged cache [blocks, block_size, kv_heads * dim | kv_heads * vdim] (window_attention.hip).
 // attn_prepare: per row of proj = [q | k | v | ...]: optional RMS norm of q and k (norm_mode 0: none; 1: over the
 // whole projection, weights per element; 2: per head - and map - of `dim` elements, one weight of `dim` elements),
 // rotate-half rotation of the first 2 * nfreq dims per head (cos and sin times amp; norm_mode 3: every rotated head
-// divided by its root mean square), optional per-head unit-rms values; q in place, k / v
+// divided by its root mean square), the query at position p times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
+// (temp_every > 0), optional per-head unit-rms values; q in place, k / v
 // into cache row slots[t] (>= 0). `maps` query / key maps per head (rows hold heads * maps * dim query and
 // kv_heads * maps * dim key elements). cache null: the rows are [q | ...] and only q is prepared.
 void launch_attn_prepare(void* proj, long ld, void* cache, const long* positions, const long* slots,
                          const float* inv_freq, int nfreq, int T, int heads, int kv_heads, int maps, int dim, int vdim,
                          const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, float amp,
-                         bool f32, hipStream_t s);
+                         float temp_coef, int temp_every, bool f32, hipStream_t s);
 // Sequences seq0 .. seq1-1 of the step, `tq` tokens per workgroup: keys 0 <= pos - j < window (0: all) or
-// j < keep, scores q . k * scale, through softcap * tanh(. / softcap) when softcap > 0,
+// j < keep (chunk > 0, with window = keep = 0: j <= pos in pos's chunk of `chunk` positions), scores q . k * scale, through softcap * tanh(. / softcap) when softcap > 0,
 // weights exp(s_j) / (sink + sum exp) with sink = exp(sink_w[h]) (1 when sink_w is null),
 // head output times sigmoid(proj[t, gate_off + h]) (gate_off >= 0; channel_gate: element e of the concatenated
 // heads times sigmoid(proj[t, gate_off + e])) and
@@ -103,8 +121,8 @@ void launch_window_attention(void* out, long out_ld, const void* proj, long proj
                              const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                              int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off,
                              float scale, int window, bool sink, float out_scale, int maps, float lam, float post,
-                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, bool f32,
-                             hipStream_t s);
+                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, int chunk,
+                             bool f32, hipStream_t s);
 
 // bf16 on the matrix cores (window_attention_mfma.hip): 64 (token, head) rows of one key/value head per
 // workgroup, 32-key tiles. nparts > 1 (rows of one token each, rows_bound of them from batch row row_base on):
@@ -118,16 +136,33 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
                                   int vdim, int gate_off, float scale, int window, bool sink, float out_scale,
                                   int nparts, int part_keys, float* ws_acc, float* ws_ml, int row_base, int maps,
                                   float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                                  bool channel_gate, hipStream_t s);
+                                  bool channel_gate, int chunk, hipStream_t s);
 
-// Delta-rule recurrences over state slots (delta_scan.hip). scratch: fp32, T * (2 * kv_heads * dim +
-// 2 * heads * vdim + 2 * heads) floats for the gated rule, T * 7 * heads * dim for the generalized one.
+// Delta-rule recurrences over state slots (delta_scan.hip). Gated rule: proj rows = [q | k | v | ...] with beta's
+// columns from off_b on and the decay's / the gate's pre-activations from off_a / off_g on, or from `decay` (fp32
+// [T, heads * dim]: a decay per key channel) and `gate` ([T, heads * vdim], activation type); dt_bias has as many
+// elements as a token has decays. scratch: fp32, T * (2 * kv_heads * dim + 2 * heads * vdim + heads * (1 + decays per
+// head)) floats; the generalized rule's: T * 7 * heads * dim.
 int delta_max_dim();
 int delta_max_taps();
-void launch_gated_delta(void* y, float* S, float* conv_state, const void* proj, long ld, const float* conv_w,
-                        const float* a_log, const float* dt_bias, const float* norm_w, const int* seq_cu,
-                        const int* seq_ctx, const int* seq_state, int nseq, int T, float* scratch, int heads,
-                        int kv_heads, int dim, int vdim, int taps, float eps, bool f32, hipStream_t s);
+struct GatedDelta {
+  void* y; long y_ld;
+  float *S, *conv_state;
+  const void* proj; long ld;
+  const float *conv_w, *a_log, *dt_bias, *norm_w;
+  const int *seq_cu, *seq_ctx, *seq_state;
+  int nseq, T, heads, kv_heads, dim, vdim, taps, off_a, off_g, off_b;
+  float eps;
+  bool channel, silu;                   // a decay per key channel; the gate through SiLU (else sigmoid)
+  const float* decay; const void* gate; // launch_gated_delta, channel
+  const void *a2, *g2; int ra, rg;      // launch_gated_delta_step, channel: up-projections [heads * dim, ra], [heads * vdim, rg]
+};
+void launch_gated_delta(const GatedDelta& p, float* scratch, bool f32, hipStream_t s);
+// The same for steps in which every sequence has ONE row: everything in one launch (two where heads share queries and
+// keys); the decay's and the gate's bottleneck outputs are columns off_a / off_g of proj. dim, vdim <= 256,
+// ra + rg <= gated_delta_step_max_rank().
+int gated_delta_step_max_rank();
+void launch_gated_delta_step(const GatedDelta& p, bool f32, hipStream_t s);
 void launch_delta_rule(void* out, long out_ld, float* S, const void* proj, long ld, const float* wl, const float* a_b,
                        const float* w0, const float* norm_w, const int* seq_cu, const int* seq_ctx,
                        const int* seq_state, int nseq, int T, float* scratch, int heads, int dim, float eps,

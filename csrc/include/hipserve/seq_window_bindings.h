@@ -8,11 +8,12 @@ namespace hipserve_shared {
 inline void attn_prepare(at::Tensor& proj, const c10::optional<at::Tensor>& cache, const at::Tensor& positions,
                   const at::Tensor& slots, const at::Tensor& inv_freq, int64_t heads, int64_t kv_heads, int64_t maps,
                   int64_t dim, int64_t vdim, const c10::optional<at::Tensor>& q_norm,
-                  const c10::optional<at::Tensor>& k_norm, int64_t norm_mode, bool v_norm, double eps, double amp) {
+                  const c10::optional<at::Tensor>& k_norm, int64_t norm_mode, bool v_norm, double eps, double amp,
+                  double temp_coef, int64_t temp_every) {
   CHECK_DEV(proj); CHECK_F32(inv_freq);
   const bool f32 = is_f32(proj, "attn_prepare");
   TORCH_CHECK(heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 1 && vdim >= 1 && (maps == 1 || maps == 2));
-  TORCH_CHECK(norm_mode >= 0 && norm_mode <= 3 && (heads + kv_heads) * maps <= 8192);
+  TORCH_CHECK(temp_every >= 0 && temp_every < (1LL << 31) && norm_mode >= 0 && norm_mode <= 3 && (heads + kv_heads) * maps <= 8192);
   const long T = proj.size(0), nq = heads * maps * dim, nk = kv_heads * maps * dim, nv = kv_heads * vdim;
   const bool own_kv = cache.has_value();
   TORCH_CHECK(rows2d(proj) && proj.size(1) >= nq + (own_kv ? nk + nv : 0));
@@ -36,7 +37,7 @@ inline void attn_prepare(at::Tensor& proj, const c10::optional<at::Tensor>& cach
   hipserve::launch_attn_prepare(proj.data_ptr(), proj.stride(0), own_kv ? cache->data_ptr() : nullptr,
                                 positions.data_ptr<long>(), slots.data_ptr<long>(), inv_freq.data_ptr<float>(),
                                 inv_freq.numel(), T, heads, kv_heads, maps, dim, vdim, (const float*)opt_ptr(q_norm),
-                                own_kv ? (const float*)opt_ptr(k_norm) : nullptr, norm_mode, v_norm, (float)eps, (float)amp, f32,
+                                own_kv ? (const float*)opt_ptr(k_norm) : nullptr, norm_mode, v_norm, (float)eps, (float)amp, (float)temp_coef, temp_every, f32,
                                 cur_stream());
 }
 
@@ -45,7 +46,8 @@ inline void window_attention(at::Tensor& out, const at::Tensor& proj, const at::
                       int64_t rows_bound, int64_t tq, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
                       int64_t gate_off, double scale, int64_t window, bool sink, double out_scale, int64_t maps,
                       double lam, double post, double eps, int64_t keep, double softcap,
-                      const c10::optional<at::Tensor>& sink_w, bool channel_gate) {
+                      const c10::optional<at::Tensor>& sink_w, bool channel_gate, int64_t chunk) {
+  TORCH_CHECK(chunk >= 0 && (chunk == 0 || (window == 0 && keep == 0)), "window attention: chunks or a window");
   CHECK_DEV(proj); CHECK_CONTIG(cache); CHECK_I32(seq_cu); CHECK_I32(seq_ctx); CHECK_I32(seq_bt);
   const bool f32 = is_f32(proj, "window_attention");
   TORCH_CHECK(maps == 1 || maps == 2);
@@ -72,7 +74,7 @@ inline void window_attention(at::Tensor& out, const at::Tensor& proj, const at::
                                     seq_bt.data_ptr<int>(), seq_bt.size(1), seq0, seq1, rows_bound, tq, heads, kv_heads,
                                     dim, vdim, gate_off, (float)scale, window, sink, (float)out_scale, maps, (float)lam,
                                     (float)post, (float)eps, keep, (float)softcap, (const float*)opt_ptr(sink_w),
-                                    channel_gate, f32, cur_stream());
+                                    channel_gate, chunk, f32, cur_stream());
 }
 
 inline bool window_attention_mfma_ok(int64_t dim, int64_t vdim, int64_t out_ld, int64_t out_off, int64_t maps) {
@@ -86,7 +88,8 @@ inline void window_attention_mfma(at::Tensor& out, const at::Tensor& proj, const
                            int64_t part_keys, const c10::optional<at::Tensor>& ws_acc,
                            const c10::optional<at::Tensor>& ws_ml, int64_t row_base, int64_t maps, double lam,
                            double post, double eps, int64_t keep, double softcap,
-                           const c10::optional<at::Tensor>& sink_w, bool channel_gate) {
+                           const c10::optional<at::Tensor>& sink_w, bool channel_gate, int64_t chunk) {
+  TORCH_CHECK(chunk >= 0 && (chunk == 0 || (window == 0 && keep == 0)), "window attention: chunks or a window");
   CHECK_DEV(proj); CHECK_CONTIG(cache); CHECK_I32(seq_cu); CHECK_I32(seq_ctx); CHECK_I32(seq_bt);
   TORCH_CHECK(proj.scalar_type() == at::kBFloat16 && out.scalar_type() == at::kBFloat16 &&
               cache.scalar_type() == at::kBFloat16, "window_attention_mfma: bf16 only");
@@ -124,7 +127,7 @@ inline void window_attention_mfma(at::Tensor& out, const at::Tensor& proj, const
                                          rows_bound, heads, kv_heads, dim, vdim, gate_off, (float)scale, window, sink,
                                          (float)out_scale, nparts, part_keys, wa, wm, row_base, maps, (float)lam,
                                          (float)post, (float)eps, keep, (float)softcap, (const float*)opt_ptr(sink_w),
-                                         channel_gate, cur_stream());
+                                         channel_gate, chunk, cur_stream());
 }
 
 inline void activation(at::Tensor& out, const at::Tensor& x, int64_t kind, double c0, double c1) {
@@ -139,7 +142,7 @@ inline void activation(at::Tensor& out, const at::Tensor& x, int64_t kind, doubl
 }
 
 inline void route_topk(at::Tensor& ids, at::Tensor& wts, const at::Tensor& logits, const c10::optional<at::Tensor>& correction,
-                int64_t top, double scale, int64_t E, int64_t groups, int64_t keep, bool renorm, bool sigmoid) {
+                int64_t top, double scale, int64_t E, int64_t groups, int64_t keep, bool renorm, bool sigmoid, bool top2) {
   CHECK_DEV(logits); CHECK_F32(wts); CHECK_I32(ids);
   TORCH_CHECK(logits.scalar_type() == at::kFloat && rows2d(logits), "route_topk: fp32 logits");
   const long T = logits.size(0), n = logits.size(1);
@@ -154,13 +157,13 @@ inline void route_topk(at::Tensor& ids, at::Tensor& wts, const at::Tensor& logit
   c10::hip::HIPGuardMasqueradingAsCUDA g(logits.device());
   hipserve::launch_route_topk(ids.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(), logits.stride(0),
                               (const float*)opt_ptr(correction), T, n, top, (float)scale, E, groups, keep, renorm,
-                              sigmoid, cur_stream());
+                              sigmoid, top2, cur_stream());
 }
 
 inline void route_align(at::Tensor& ids, at::Tensor& wts, at::Tensor& slots, at::Tensor& tile_expert,
                         at::Tensor& pair_slot, const at::Tensor& logits, const c10::optional<at::Tensor>& correction,
                         int64_t top, double scale, int64_t E, int64_t nb, int64_t tile, int64_t groups, int64_t keep,
-                        bool renorm, bool sigmoid) {
+                        bool renorm, bool sigmoid, bool top2) {
   CHECK_DEV(logits); CHECK_F32(wts); CHECK_I32(ids); CHECK_I32(slots); CHECK_I32(tile_expert); CHECK_I32(pair_slot);
   TORCH_CHECK(logits.scalar_type() == at::kFloat && rows2d(logits), "route_align: fp32 logits");
   const long T = logits.size(0), n = logits.size(1), P = T * top, cap = slots.numel();
@@ -180,7 +183,7 @@ inline void route_align(at::Tensor& ids, at::Tensor& wts, at::Tensor& slots, at:
   hipserve::launch_route_align(ids.data_ptr<int>(), wts.data_ptr<float>(), slots.data_ptr<int>(), cap,
                                tile_expert.data_ptr<int>(), tile, pair_slot.data_ptr<int>(), logits.data_ptr<float>(),
                                logits.stride(0), (const float*)opt_ptr(correction), T, n, top, (float)scale, E, nb,
-                               groups, keep, renorm, sigmoid, cur_stream());
+                               groups, keep, renorm, sigmoid, top2, cur_stream());
 }
 
 inline void polynorm(at::Tensor& out, const at::Tensor& x, const at::Tensor& coef, double eps) {
@@ -208,23 +211,23 @@ inline void gate_mul(at::Tensor& out, const at::Tensor& x, const at::Tensor& gat
 inline void def_window_ops(torch::Library& m) {
   m.def("attn_prepare(Tensor(a!) proj, Tensor(b!)? cache, Tensor positions, Tensor slots, Tensor inv_freq, int heads, "
         "int kv_heads, int maps, int dim, int vdim, Tensor? q_norm, Tensor? k_norm, int norm_mode, bool v_norm, "
-        "float eps, float amp=1.0) -> ()");
+        "float eps, float amp=1.0, float temp_coef=0.0, int temp_every=0) -> ()");
   m.def("window_attention(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
         "int seq0, int seq1, int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, "
         "float scale, int window, bool sink, float out_scale, int maps, float lam, float post, float eps, int keep, "
-        "float softcap, Tensor? sink_w, bool channel_gate=False) -> ()");
+        "float softcap, Tensor? sink_w, bool channel_gate=False, int chunk=0) -> ()");
   m.def("window_attention_mfma(Tensor(a!) out, Tensor proj, Tensor cache, Tensor seq_cu, Tensor seq_ctx, Tensor seq_bt, "
         "int seq0, int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, "
         "int window, bool sink, float out_scale, int nparts, int part_keys, Tensor(b!)? ws_acc, Tensor(c!)? ws_ml, "
         "int row_base, int maps, float lam, float post, float eps, int keep, float softcap, Tensor? sink_w, "
-        "bool channel_gate=False) -> ()");
+        "bool channel_gate=False, int chunk=0) -> ()");
   m.def("window_attention_mfma_ok(int dim, int vdim, int out_ld, int out_off, int maps) -> bool", &window_attention_mfma_ok);
   m.def("activation(Tensor(a!) out, Tensor x, int kind, float c0, float c1) -> ()");
   m.def("route_topk(Tensor(a!) ids, Tensor(b!) wts, Tensor logits, Tensor? correction, int top, float scale, int E, "
-        "int groups, int keep, bool renorm, bool sigmoid=False) -> ()");
+        "int groups, int keep, bool renorm, bool sigmoid=False, bool top2=False) -> ()");
   m.def("route_align(Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) slots, Tensor(d!) tile_expert, Tensor(e!) pair_slot, "
         "Tensor logits, Tensor? correction, int top, float scale, int E, int nb, int tile, int groups, int keep, "
-        "bool renorm, bool sigmoid) -> ()");
+        "bool renorm, bool sigmoid, bool top2=False) -> ()");
   def_moe_ops(m);
 }
 

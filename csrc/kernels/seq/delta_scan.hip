@@ -2,6 +2,7 @@
 //
 // gated delta rule (per head, one decay g and one write strength beta per token):
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+// the same with a decay g per key channel (the rows of S), from a bottleneck
 // generalized delta rule (per head, decay w and removal rate a per key channel, unit key u):
 //   S <- diag(w) S - (a * u)(u^T S) + k v^T  (both terms read the old S);  o = S^T r
 //
@@ -17,6 +18,9 @@
 // (+ SiLU) from the step's rows and the sequence's last taps - 1 inputs, unit vectors, sigmoid /
 // softplus / exp of the decays and rates. head_norm_gate finishes both: per-head RMS norm of the
 // read-out, weight, SiLU or sigmoid gate, optional scale.
+//
+// Steps in which every sequence brings one row run the whole gated rule of a (sequence, head) in one workgroup
+// (gated_delta_step).
 #include "seq_common.h"
 #include "hipserve/seq_kernels.h"
 
@@ -31,49 +35,124 @@ HS_DEVICE int find_seq(const int* __restrict__ seq_cu, int nseq, int row) {
   return -1;
 }
 
-// proj rows = [q | k | v | beta | decay | gate]; C = conv channels (q, k, v). One workgroup per token.
-//   qk[t] = [unit(silu(conv q)) * dim^-1/2 | unit(silu(conv k))]  per head,  vv[t] = silu(conv v),
-//   bg[t] = [beta (heads) | g (heads)].
-template <typename T>
+// What enters the gated rule, as fp32 rows. One wave per item and run of kPrepTokens rows; the items of a row are
+//   the query heads: unit(silu(conv q)) dim^-1/2,  the key heads: unit(silu(conv k))      -> qk[t] = [q | k]
+//   the value channels in parts of 256: silu(conv v)                                       -> vv[t]
+//   the heads' decays: exp(-exp(a_log) softplus(. + dt_bias)), one per head or (CH) per head and key channel
+//   (dec [T, heads * dim])                                                                 -> gg[t]
+//   beta: sigmoid                                                                          -> bb[t]
+// Lane l owns channels l, l + 64, ... of its item and keeps their last TAPS - 1 inputs in registers while it walks
+// the rows (TAPS 0: any number of taps, inputs read again per row).
+constexpr int kPrepTokens = 16, kPrepCh = 4;   // kPrepCh * 64: most channels of an item
+
+template <typename T, int TAPS, bool CH>
 __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(
-    float* __restrict__ qk, float* __restrict__ vv, float* __restrict__ bg, const T* __restrict__ proj, long ld,
-    const float* __restrict__ conv_state, const float* __restrict__ conv_w, const float* __restrict__ a_log,
-    const float* __restrict__ dt_bias, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx,
-    const int* __restrict__ seq_state, int nseq, int heads, int kv_heads, int dim, int vdim, int taps) {
-  extern __shared__ float xs[];  // [C] convolved + SiLU
-  const int t = blockIdx.x;
-  const int s = find_seq(seq_cu, nseq, t);
-  if (s < 0) return;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int r0 = seq_cu[s], n = seq_cu[s + 1] - r0;
-  const bool carried = seq_ctx[s] - n > 0;
-  const int nqk = kv_heads * dim, C = 2 * nqk + heads * vdim, hist = taps - 1;
-  const float* cs = conv_state + (long)seq_state[s] * max(hist, 1) * C;
-  for (int c = tid; c < C; c += 256) {
-    float a = 0.f;
-    for (int j = 0; j < taps; ++j) {
-      const int r = t - hist + j;  // batch row of the tap's input
-      float x;
-      if (r >= r0) x = ldf<T>(proj, (long)r * ld + c);
-      else x = carried ? cs[(long)(hist + r - r0) * C + c] : 0.f;
-      a = __builtin_fmaf(conv_w[(long)c * taps + j], x, a);
+    float* __restrict__ qk, float* __restrict__ vv, float* __restrict__ gg, float* __restrict__ bb,
+    const T* __restrict__ proj, long ld, const float* __restrict__ dec, const float* __restrict__ conv_state,
+    const float* __restrict__ conv_w, const float* __restrict__ a_log, const float* __restrict__ dt_bias,
+    const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx, const int* __restrict__ seq_state, int nseq, int T_,
+    int heads, int kv_heads, int dim, int vdim, int taps_, int off_a, int off_b) {
+  const int lane = threadIdx.x & 63;
+  const int nqk = kv_heads * dim, nv = heads * vdim, C = 2 * nqk + nv;
+  const int vparts = (nv + 64 * kPrepCh - 1) / (64 * kPrepCh), dparts = CH ? heads : 1;
+  int item = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int t0 = blockIdx.x * kPrepTokens, t1 = min(t0 + kPrepTokens, T_);
+  if (item >= 2 * kv_heads + vparts) {
+    item -= 2 * kv_heads + vparts;
+    if (item < dparts) {
+      if constexpr (CH) {
+        const float ea = expf(a_log[item]);
+        for (int t = t0; t < t1; ++t)
+          for (int e = lane; e < dim; e += 64) {
+            const long i = (long)item * dim + e;
+            gg[(long)t * heads * dim + i] = expf(-ea * softplus_f(dec[(long)t * heads * dim + i] + dt_bias[i]));
+          }
+      } else {
+        for (int t = t0; t < t1; ++t)
+          for (int h = lane; h < heads; h += 64)
+            gg[(long)t * heads + h] = expf(-expf(a_log[h]) * softplus_f(ldf<T>(proj, (long)t * ld + off_a + h) + dt_bias[h]));
+      }
+    } else if (item == dparts) {
+      for (int t = t0; t < t1; ++t)
+        for (int h = lane; h < heads; h += 64) bb[(long)t * heads + h] = sigmoid_f(ldf<T>(proj, (long)t * ld + off_b + h));
     }
-    xs[c] = a * sigmoid_f(a);
+    return;
   }
-  __syncthreads();
-  for (int h = wave; h < 2 * kv_heads; h += 4) {  // unit q heads, then unit k heads
-    float a = 0.f;
-    for (int e = lane; e < dim; e += 64) { const float v = xs[h * dim + e]; a += v * v; }
-    float inv = 1.f / sqrtf(wave_sum(a) + 1e-6f);
-    if (h < kv_heads) inv *= 1.f / sqrtf((float)dim);
-    for (int e = lane; e < dim; e += 64) qk[(long)t * 2 * nqk + h * dim + e] = xs[h * dim + e] * inv;
+  const bool value = item >= 2 * kv_heads;
+  const int c0 = value ? 2 * nqk + (item - 2 * kv_heads) * 64 * kPrepCh : item * dim;   // the item's first channel
+  const int nc = value ? min(64 * kPrepCh, C - c0) : dim;
+  const int taps = TAPS > 0 ? TAPS : taps_, hist = taps - 1;
+  constexpr int kW = TAPS > 0 ? TAPS : 1, kX = TAPS > 1 ? TAPS - 1 : 1;
+  float w[kPrepCh][kW], x[kPrepCh][kX];
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int i = 0; i < kPrepCh; ++i)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[i][j] = lane + 64 * i < nc ? conv_w[(long)(c0 + lane + 64 * i) * TAPS + j] : 0.f;
   }
-  const int nv = heads * vdim;
-  for (int e = tid; e < nv; e += 256) vv[(long)t * nv + e] = xs[2 * nqk + e];
-  for (int h = tid; h < heads; h += 256) {
-    const T* p = proj + (long)t * ld + C;
-    bg[(long)t * 2 * heads + h] = sigmoid_f(ldf<T>(p, h));
-    bg[(long)t * 2 * heads + heads + h] = expf(-expf(a_log[h]) * softplus_f(ldf<T>(p, heads + h) + dt_bias[h]));
+  int s = find_seq(seq_cu, nseq, t0), r0 = 0, end = 0;
+  const float* cs = nullptr;
+  bool carried = false, fresh = true;
+  if (s < 0) return;
+  end = seq_cu[s + 1];
+  for (int t = t0; t < t1; ++t) {
+    while (t >= end) {   // the next sequence that has rows
+      if (++s >= nseq) return;
+      end = seq_cu[s + 1];
+      fresh = true;
+    }
+    // the input `back` rows before row t: an earlier row of the step, or one of the sequence's kept inputs, or zero
+    auto before = [&](int c, int back) {
+      const int r = t - back;
+      if (r >= r0) return ldf<T>(proj, (long)r * ld + c);
+      return carried ? cs[(long)(hist + r - r0) * C + c] : 0.f;
+    };
+    if (fresh) {
+      r0 = seq_cu[s];
+      carried = seq_ctx[s] - (end - r0) > 0;
+      cs = conv_state + (long)seq_state[s] * max(hist, 1) * C;
+      fresh = false;
+      if constexpr (TAPS > 1) {
+#pragma unroll
+        for (int i = 0; i < kPrepCh; ++i)
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) x[i][j] = lane + 64 * i < nc ? before(c0 + lane + 64 * i, TAPS - 1 - j) : 0.f;
+      }
+    }
+    float y[kPrepCh];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < kPrepCh; ++i) {
+      y[i] = 0.f;
+      if (64 * i >= nc) continue;
+      const int c = c0 + lane + 64 * i;
+      if (lane + 64 * i < nc) {
+        const float cur = ldf<T>(proj, (long)t * ld + c);
+        float a = 0.f;
+        if constexpr (TAPS > 0) {
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) a = __builtin_fmaf(w[i][j], x[i][j], a);
+          a = __builtin_fmaf(w[i][TAPS - 1], cur, a);
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS - 1; ++j) x[i][j] = x[i][j + 1];
+          if constexpr (TAPS > 1) x[i][TAPS - 2] = cur;
+        } else {
+          for (int j = 0; j < taps; ++j)
+            a = __builtin_fmaf(conv_w[(long)c * taps + j], j == hist ? cur : before(c, hist - j), a);
+        }
+        y[i] = a * sigmoid_f(a);
+        ss = __builtin_fmaf(y[i], y[i], ss);
+      }
+    }
+    float f = 1.f;
+    if (!value) {
+      f = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+      if (item < kv_heads) f *= 1.f / sqrtf((float)dim);
+    }
+    float* dst = value ? vv + (long)t * nv + (c0 - 2 * nqk) : qk + (long)t * 2 * nqk + c0;
+#pragma unroll
+    for (int i = 0; i < kPrepCh; ++i)
+      if (lane + 64 * i < nc) dst[lane + 64 * i] = y[i] * f;
   }
 }
 
@@ -122,14 +201,15 @@ HS_DEVICE float row_sum(float v) {
 // state is DS multiply-adds per lane and four DPP steps, so the chain from one token to the next is short.
 // Every lane row holds kCV columns (independent chains that fill each other's stalls and share the LDS reads
 // of the per-token vectors, which bound the kernel otherwise); the waves share the staging.
-template <int DS>
+// CH: a decay per key channel, staged beside q and k.
+template <int DS, bool CH>
 __global__ __launch_bounds__(kScanThreads) void gated_delta_scan_kernel(
     float* __restrict__ o, float* __restrict__ S, const float* __restrict__ qk, const float* __restrict__ vv,
-    const float* __restrict__ bg, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx,
+    const float* __restrict__ gg, const float* __restrict__ bb, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx,
     const int* __restrict__ seq_state, int heads, int kv_heads, int dim, int vdim) {
   constexpr int DP = kSeg * DS;
-  __shared__ __attribute__((aligned(16))) float sq[kTB][DP], sk[kTB][DP];
-  __shared__ float sb[kTB][2];
+  __shared__ __attribute__((aligned(16))) float sq[kTB][DP], sk[kTB][DP], sg[CH ? kTB : 1][CH ? DP : 1];
+  __shared__ float sb[kTB][2];   // beta, and the head's decay without CH
   const int s = blockIdx.z, h = blockIdx.x, zb = blockIdx.y, tid = threadIdx.x;
   const int r0 = seq_cu[s], n = seq_cu[s + 1] - r0;
   if (n <= 0) return;
@@ -146,7 +226,7 @@ __global__ __launch_bounds__(kScanThreads) void gated_delta_scan_kernel(
       st[cv][i] = (carried && v0 + cv < vdim && k0 + i < dim) ? Sp[(long)(k0 + i) * vdim + v0 + cv] : 0.f;
   // the next batch of tokens is loaded into registers while this batch is computed
   constexpr int kLd = (kTB * DP + kScanThreads - 1) / kScanThreads;
-  float rq[kLd], rk[kLd], rv[kTB][kCV], rb = 0.f;
+  float rq[kLd], rk[kLd], rg[CH ? kLd : 1], rv[kTB][kCV], rb = 0.f;
   auto fetch = [&](int t0) {
     const int nt = min(kTB, n - t0);
 #pragma unroll
@@ -157,8 +237,13 @@ __global__ __launch_bounds__(kScanThreads) void gated_delta_scan_kernel(
       const bool in = tt < nt && k < dim;
       rq[it] = in ? qk[row + kh * dim + k] : 0.f;
       rk[it] = in ? qk[row + nqk + kh * dim + k] : 0.f;
+      if constexpr (CH) rg[it] = in ? gg[((long)(r0 + t0 + tt) * heads + h) * dim + k] : 0.f;
     }
-    if (tid < 2 * nt) rb = bg[(long)(r0 + t0 + (tid >> 1)) * 2 * heads + (tid & 1) * heads + h];
+    if (tid < 2 * nt) {
+      const long i = (long)(r0 + t0 + (tid >> 1)) * heads + h;
+      if (!(tid & 1)) rb = bb[i];
+      else if (!CH) rb = gg[i];
+    }
 #pragma unroll
     for (int tt = 0; tt < kTB; ++tt)
 #pragma unroll
@@ -176,6 +261,7 @@ __global__ __launch_bounds__(kScanThreads) void gated_delta_scan_kernel(
       if (i < kTB * DP) {
         sq[i / DP][i % DP] = rq[it];
         sk[i / DP][i % DP] = rk[it];
+        if constexpr (CH) sg[i / DP][i % DP] = rg[it];
       }
     }
     if (tid < 2 * kTB) sb[tid >> 1][tid & 1] = rb;
@@ -190,16 +276,20 @@ __global__ __launch_bounds__(kScanThreads) void gated_delta_scan_kernel(
     for (int tt = 0; tt < kTB; ++tt) {
       if (tt < nt) {
         const float beta = sb[tt][0], g = sb[tt][1];
-        float kk[DS], qq[DS];
+        float kk[DS], qq[DS], gd[CH ? DS : 1];
 #pragma unroll
-        for (int i = 0; i < DS; ++i) { kk[i] = sk[tt][k0 + i]; qq[i] = sq[tt][k0 + i]; }
+        for (int i = 0; i < DS; ++i) {
+          kk[i] = sk[tt][k0 + i];
+          qq[i] = sq[tt][k0 + i];
+          if constexpr (CH) gd[i] = sg[tt][k0 + i];
+        }
         float outs[kCV];
 #pragma unroll
         for (int cv = 0; cv < kCV; ++cv) {
           float pred = 0.f, pred2 = 0.f;
 #pragma unroll
           for (int i = 0; i < DS; ++i) {
-            st[cv][i] *= g;
+            st[cv][i] *= CH ? gd[CH ? i : 0] : g;
             if (i & 1) pred2 = __builtin_fmaf(st[cv][i], kk[i], pred2);
             else pred = __builtin_fmaf(st[cv][i], kk[i], pred);
           }
@@ -563,6 +653,190 @@ __global__ __launch_bounds__(256) void wkv_step_kernel(
   }
 }
 
+// Decode rows (one row per sequence): the whole gated rule of one (sequence, head) in one workgroup: convolution, unit
+// query and key, decays and output gate (CH: with their bottlenecks' up-projections), recurrence, norm, gate. The
+// state is read and written once: with VEC 4 and at most kStepIt rows per thread it waits in registers (loaded
+// before anything else), else it is read once more from the caches. Per element of the OLD state the two sums
+//   pred_v = sum_k g_k k_k S_kv,  read_v = sum_k g_k q_k S_kv
+// give u_v = beta (v - pred_v) and o_v = read_v + (q . k) u_v, the read-out of the new state S' = g S + k u^T.
+// Thread (r, w) owns columns VEC w .. of rows r, r + R, ...
+constexpr int kStepIt = 16, kStepRank = 1024;
+
+// sum_j w[j] x[j] over a bottleneck; x in LDS
+template <typename T>
+HS_DEVICE float low_dot(const T* __restrict__ w, const float* x, int n, bool vec) {
+  float a = 0.f, b = 0.f;
+  if (vec) {
+#pragma unroll 4
+    for (int j = 0; j < n; j += 8) {
+      float v[8];
+      Row<T, 8>::ld(w + j, v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        a = __builtin_fmaf(v[i], x[j + i], a);
+        b = __builtin_fmaf(v[4 + i], x[j + 4 + i], b);
+      }
+    }
+  } else {
+    for (int j = 0; j < n; ++j) a = __builtin_fmaf(ldf<T>(w, j), x[j], a);
+  }
+  return a + b;
+}
+
+template <typename T, bool CH, int VEC>
+__global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta p, bool own_conv, bool vec_a, bool vec_g) {
+  __shared__ float low[CH ? kStepRank : 1];                                 // [decay bottleneck | gate bottleneck]
+  __shared__ float xs[3 * 256];                                             // silu(conv): q | k | v
+  __shared__ float sg[256], su[256];                                        // decays, u
+  __shared__ float red[2][1024];                                            // partial sums [r][column]: pred, read
+  __shared__ float sc[16], sn[4];
+  const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int t = p.seq_cu[s];
+  if (p.seq_cu[s + 1] - t != 1) return;   // sequences without a row in this step
+  const int dim = p.dim, vdim = p.vdim, taps = p.taps, hist = taps - 1;
+  const int nqk = p.kv_heads * dim, C = 2 * nqk + p.heads * vdim, kh = h / (p.heads / p.kv_heads);
+  const bool carried = p.seq_ctx[s] - 1 > 0;
+  const T* row = (const T*)p.proj + (long)t * p.ld;
+  float* Sp = p.S + ((long)p.seq_state[s] * p.heads + h) * dim * vdim;
+  const int W = vdim / VEC, R = 256 / W, r = tid / W, w = tid - r * W;
+  const bool active = r < R;
+  const bool kept = VEC == 4 && dim <= R * kStepIt;
+  f32x4 st[VEC == 4 ? kStepIt : 1];
+  if constexpr (VEC == 4) {
+    if (kept) {
+#pragma unroll
+      for (int i = 0; i < kStepIt; ++i) {
+        const int k = r + i * R;
+        st[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (active && k < dim && carried) st[i] = *reinterpret_cast<const f32x4*>(Sp + (long)k * vdim + 4 * w);
+      }
+    }
+  }
+  if constexpr (CH) {
+    for (int j = tid; j < p.ra + p.rg; j += 256)
+      low[j] = j < p.ra ? ldf<T>(row, p.off_a + j) : ldf<T>(row, p.off_g + j - p.ra);
+  }
+  // the convolution of the head's channels; with heads of their own queries and keys the kept inputs move on here
+  float* cs = p.conv_state + (long)p.seq_state[s] * max(hist, 1) * C;
+  for (int i = tid; i < 2 * dim + vdim; i += 256) {
+    const int c = i < dim ? kh * dim + i : i < 2 * dim ? nqk + kh * dim + i - dim : 2 * nqk + h * vdim + i - 2 * dim;
+    const float cur = ldf<T>(row, c);
+    const float* cw = p.conv_w + (long)c * taps;
+    float a = 0.f;
+    for (int j = 0; j < hist; ++j) {
+      const float x = carried ? cs[(long)j * C + c] : 0.f;
+      a = __builtin_fmaf(cw[j], x, a);
+      if (own_conv && j > 0) cs[(long)(j - 1) * C + c] = x;
+    }
+    if (own_conv && hist > 0) cs[(long)(hist - 1) * C + c] = cur;
+    a = __builtin_fmaf(cw[hist], cur, a);
+    xs[i] = a * sigmoid_f(a);
+  }
+  __syncthreads();
+  // unit query and key and their product (waves 0 - 2), decays
+  if (wave < 3) {
+    float a = 0.f;
+    for (int e = lane; e < dim; e += 64) a = __builtin_fmaf(xs[(wave == 1 ? dim : 0) + e], xs[(wave == 0 ? 0 : dim) + e], a);
+    a = wave_sum(a);
+    if (lane == 0) sn[wave] = a;   // q . q, k . k, q . k
+  }
+  if constexpr (CH) {
+    const float ea = expf(p.a_log[h]);
+    for (int e = tid; e < dim; e += 256) {
+      const long i = (long)h * dim + e;
+      const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, vec_a);
+      sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
+    }
+  } else {
+    const float g = expf(-expf(p.a_log[h]) * softplus_f(ldf<T>(row, p.off_a + h) + p.dt_bias[h]));
+    for (int e = tid; e < dim; e += 256) sg[e] = g;
+  }
+  float gp = 0.f;
+  if (tid < vdim) {
+    if constexpr (CH) gp = low_dot<T>((const T*)p.g2 + ((long)h * vdim + tid) * p.rg, low + p.ra, p.rg, vec_g);
+    else gp = ldf<T>(row, p.off_g + h * vdim + tid);
+  }
+  __syncthreads();
+  const float fq = 1.f / sqrtf(sn[0] + 1e-6f) / sqrtf((float)dim), fk = 1.f / sqrtf(sn[1] + 1e-6f);
+  const float qk = sn[2] * fq * fk;
+  const float* xq = xs;
+  const float* xk = xs + dim;
+  float pr[VEC], rd[VEC];
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) pr[i] = rd[i] = 0.f;
+  if (active && carried) {
+    if (kept) {
+      if constexpr (VEC == 4) {
+#pragma unroll
+        for (int i = 0; i < kStepIt; ++i) {
+          const int k = r + i * R;
+          if (k < dim) {
+            const float g = sg[k], gk = g * xk[k], gq = g * xq[k];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { pr[e] = __builtin_fmaf(gk, st[i][e], pr[e]); rd[e] = __builtin_fmaf(gq, st[i][e], rd[e]); }
+          }
+        }
+      }
+    } else {
+      for (int k = r; k < dim; k += R) {
+        const float g = sg[k], gk = g * xk[k], gq = g * xq[k];
+        float v[VEC];
+        Row<float, VEC>::ld(Sp + (long)k * vdim + VEC * w, v);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) { pr[e] = __builtin_fmaf(gk, v[e], pr[e]); rd[e] = __builtin_fmaf(gq, v[e], rd[e]); }
+      }
+    }
+  }
+  if (active) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) { red[0][r * vdim + VEC * w + e] = pr[e]; red[1][r * vdim + VEC * w + e] = rd[e]; }
+  }
+  __syncthreads();
+  float o = 0.f;
+  if (tid < vdim) {
+    float a = 0.f, b = 0.f;
+    for (int i = 0; i < R; ++i) { a += red[0][i * vdim + tid]; b += red[1][i * vdim + tid]; }
+    const float u = sigmoid_f(ldf<T>(row, p.off_b + h)) * (xs[2 * dim + tid] - fk * a);
+    su[tid] = u;
+    o = fq * b + qk * u;
+  }
+  const float ss = block_sum(tid < vdim ? o * o : 0.f, sc);   // also orders the writes of su before the reads below
+  if (tid < vdim) {
+    const float gv = sigmoid_f(gp) * (p.silu ? gp : 1.f);
+    stf<T>((T*)p.y, (long)t * p.y_ld + (long)h * vdim + tid, o / sqrtf(ss / (float)vdim + p.eps) * p.norm_w[tid] * gv);
+  }
+  if (!active) return;
+  float u[VEC];
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) u[e] = fk * su[VEC * w + e];
+  if (kept) {
+    if constexpr (VEC == 4) {
+#pragma unroll
+      for (int i = 0; i < kStepIt; ++i) {
+        const int k = r + i * R;
+        if (k < dim) {
+          const float g = sg[k], kk = xk[k];
+          f32x4 v;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = __builtin_fmaf(kk, u[e], g * st[i][e]);
+          *reinterpret_cast<f32x4*>(Sp + (long)k * vdim + 4 * w) = v;
+        }
+      }
+    }
+  } else {
+    for (int k = r; k < dim; k += R) {
+      const float g = sg[k], kk = xk[k];
+      float v[VEC];
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+      if (carried) Row<float, VEC>::ld(Sp + (long)k * vdim + VEC * w, v);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] = __builtin_fmaf(kk, u[e], g * v[e]);
+      Row<float, VEC>::st(Sp + (long)k * vdim + VEC * w, v);
+    }
+  }
+}
+
 // One wave per (token, head): out = o / rms(o) * w[head * w_stride + e] * act(gate) * scale.
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
@@ -600,44 +874,76 @@ int ds_of(int dim) { return dim <= 16 ? 1 : dim <= 32 ? 2 : dim <= 64 ? 4 : dim 
 int delta_max_dim() { return 256; }
 int delta_max_taps() { return kMaxHist + 1; }
 
-void launch_gated_delta(void* y, float* S, float* conv_state, const void* proj, long ld, const float* conv_w,
-                        const float* a_log, const float* dt_bias, const float* norm_w, const int* seq_cu,
-                        const int* seq_ctx, const int* seq_state, int nseq, int T, float* scratch, int heads,
-                        int kv_heads, int dim, int vdim, int taps, float eps, bool f32, hipStream_t s) {
-  if (nseq <= 0 || T <= 0) return;
-  const int nqk = kv_heads * dim, nv = heads * vdim, C = 2 * nqk + nv;
-  float* qk = scratch;                       // [T, 2 nqk]
-  float* vv = qk + (long)T * 2 * nqk;        // [T, nv]
-  float* bg = vv + (long)T * nv;             // [T, 2 heads]
-  float* o = bg + (long)T * 2 * heads;       // [T, nv]
-  const size_t smem = (size_t)C * sizeof(float);
-  dim3 ugrid(nseq, (C + 255) / 256);
-  if (f32) {
-    gated_delta_prepare_kernel<float><<<T, 256, smem, s>>>(qk, vv, bg, (const float*)proj, ld, conv_state, conv_w,
-                                                           a_log, dt_bias, seq_cu, seq_ctx, seq_state, nseq, heads,
-                                                           kv_heads, dim, vdim, taps);
-    conv_state_update_kernel<float><<<ugrid, 256, 0, s>>>(conv_state, (const float*)proj, ld, seq_cu, seq_ctx,
-                                                          seq_state, C, taps);
-  } else {
-    gated_delta_prepare_kernel<unsigned short><<<T, 256, smem, s>>>(
-        qk, vv, bg, (const unsigned short*)proj, ld, conv_state, conv_w, a_log, dt_bias, seq_cu, seq_ctx, seq_state,
-        nseq, heads, kv_heads, dim, vdim, taps);
-    conv_state_update_kernel<unsigned short><<<ugrid, 256, 0, s>>>(conv_state, (const unsigned short*)proj, ld, seq_cu,
-                                                                   seq_ctx, seq_state, C, taps);
-  }
-  dim3 grid(heads, (vdim + kCols - 1) / kCols, nseq);
-  switch (ds_of(dim)) {
+int gated_delta_step_max_rank() { return kStepRank; }
+
+namespace {
+
+template <typename T>
+void conv_state_update(const GatedDelta& p, hipStream_t s) {
+  const int C = 2 * p.kv_heads * p.dim + p.heads * p.vdim;
+  conv_state_update_kernel<T><<<dim3(p.nseq, (C + 255) / 256), 256, 0, s>>>(p.conv_state, (const T*)p.proj, p.ld, p.seq_cu,
+                                                                             p.seq_ctx, p.seq_state, C, p.taps);
+}
+
+template <typename T, bool CH>
+void gated_delta(const GatedDelta& p, float* scratch, hipStream_t s) {
+  const int nqk = p.kv_heads * p.dim, nv = p.heads * p.vdim, ng = CH ? p.heads * p.dim : p.heads;
+  const long T_ = p.T;
+  float* qk = scratch;            // [T, 2 nqk]
+  float* vv = qk + T_ * 2 * nqk;  // [T, nv]
+  float* gg = vv + T_ * nv;       // [T, ng]
+  float* bb = gg + T_ * ng;       // [T, heads]
+  float* o = bb + T_ * p.heads;   // [T, nv]
+  const int items = 2 * p.kv_heads + (nv + 64 * kPrepCh - 1) / (64 * kPrepCh) + (CH ? p.heads : 1) + 1;
+  dim3 pgrid((p.T + kPrepTokens - 1) / kPrepTokens, (items + 3) / 4);
+#define HS_GP(N)                                                                                                       \
+  gated_delta_prepare_kernel<T, N, CH><<<pgrid, 256, 0, s>>>(qk, vv, gg, bb, (const T*)p.proj, p.ld, p.decay,           \
+                                                             p.conv_state, p.conv_w, p.a_log, p.dt_bias, p.seq_cu,      \
+                                                             p.seq_ctx, p.seq_state, p.nseq, p.T, p.heads, p.kv_heads,  \
+                                                             p.dim, p.vdim, p.taps, p.off_a, p.off_b)
+  if (p.taps == 4) HS_GP(4); else if (p.taps == 3) HS_GP(3); else if (p.taps == 2) HS_GP(2); else HS_GP(0);
+#undef HS_GP
+  conv_state_update<T>(p, s);
+  dim3 grid(p.heads, (p.vdim + kCols - 1) / kCols, p.nseq);
+  switch (ds_of(p.dim)) {
 #define HS_GD(D)                                                                                                     \
   case D:                                                                                                            \
-    gated_delta_scan_kernel<D><<<grid, kScanThreads, 0, s>>>(o, S, qk, vv, bg, seq_cu, seq_ctx, seq_state, heads, kv_heads, dim, \
-                                                   vdim);                                                            \
+    gated_delta_scan_kernel<D, CH><<<grid, kScanThreads, 0, s>>>(o, p.S, qk, vv, gg, bb, p.seq_cu, p.seq_ctx,          \
+                                                                 p.seq_state, p.heads, p.kv_heads, p.dim, p.vdim);    \
     break;
     HS_GD(1) HS_GD(2) HS_GD(4) HS_GD(8) HS_GD(16)
 #undef HS_GD
   }
-  const int gate_off = C + 2 * heads;
-  if (f32) head_norm_gate<float>(y, nv, o, proj, ld, gate_off, norm_w, 0, T, heads, vdim, eps, true, 1.f, s);
-  else head_norm_gate<unsigned short>(y, nv, o, proj, ld, gate_off, norm_w, 0, T, heads, vdim, eps, true, 1.f, s);
+  const bool own = p.gate != nullptr;   // the gate's rows: the bottleneck's result, or columns of the projection
+  head_norm_gate<T>(p.y, p.y_ld, o, own ? p.gate : p.proj, own ? nv : p.ld, own ? 0 : p.off_g, p.norm_w, 0, p.T, p.heads,
+                    p.vdim, p.eps, p.silu, 1.f, s);
+}
+
+template <typename T, bool CH>
+void gated_delta_step(const GatedDelta& p, hipStream_t s) {
+  const bool own_conv = p.heads == p.kv_heads;
+  auto ok = [](const void* q, int n) { return n % 8 == 0 && reinterpret_cast<uintptr_t>(q) % 16 == 0; };
+  const bool va = ok(p.a2, p.ra), vg = ok(p.g2, p.rg);
+  dim3 grid(p.heads, p.nseq);
+  if (p.vdim % 4 == 0) gated_delta_step_kernel<T, CH, 4><<<grid, 256, 0, s>>>(p, own_conv, va, vg);
+  else gated_delta_step_kernel<T, CH, 1><<<grid, 256, 0, s>>>(p, own_conv, va, vg);
+  if (!own_conv) conv_state_update<T>(p, s);   // its readers are other workgroups too: after all of them
+}
+
+}  // namespace
+
+void launch_gated_delta(const GatedDelta& p, float* scratch, bool f32, hipStream_t s) {
+  if (p.nseq <= 0 || p.T <= 0) return;
+  if (f32) { if (p.channel) gated_delta<float, true>(p, scratch, s); else gated_delta<float, false>(p, scratch, s); }
+  else if (p.channel) gated_delta<unsigned short, true>(p, scratch, s);
+  else gated_delta<unsigned short, false>(p, scratch, s);
+}
+
+void launch_gated_delta_step(const GatedDelta& p, bool f32, hipStream_t s) {
+  if (p.nseq <= 0 || p.T <= 0) return;
+  if (f32) { if (p.channel) gated_delta_step<float, true>(p, s); else gated_delta_step<float, false>(p, s); }
+  else if (p.channel) gated_delta_step<unsigned short, true>(p, s);
+  else gated_delta_step<unsigned short, false>(p, s);
 }
 
 void launch_delta_rule(void* out, long out_ld, float* S, const void* proj, long ld, const float* wl, const float* a_b,

@@ -4,7 +4,8 @@
 // expert without weights) is written as E, so the expert alignment sees them as one bucket that
 // no GEMM tile serves. One wave per token, output e on lane e % 64, slot e / 64 (n <= 256).
 // groups > 1 (at most 64): the outputs form equal groups of neighbours; a group scores the largest
-// corrected score in it (group g's on lane g), and the outputs outside the `keep` best groups (ties:
+// corrected score in it, or with top2 the sum of its two largest (of the scores s alone without a correction;
+// group g's on lane g), and the outputs outside the `keep` best groups (ties:
 // the lower group) cannot be chosen. Without a correction the choice is made by the logits, which have the order of
 // s but do not saturate. renorm: the chosen scores are divided by their sum + 1e-20.
 #include "seq_common.h"
@@ -18,7 +19,7 @@ constexpr int kSlots = 4;
 // One wave routes token t; ids_row / wts_row take its `top` choices, lds_ids (may be null) the ids once more.
 HS_DEVICE void route_token(int* __restrict__ ids_row, float* __restrict__ wts_row, int* lds_ids,
                            const float* __restrict__ row, const float* __restrict__ correction, int n, int top,
-                           float scale, int E, int groups, int keep, bool renorm, bool sigmoid) {
+                           float scale, int E, int groups, int keep, bool renorm, bool sigmoid, bool top2) {
   const int lane = threadIdx.x & 63;
   float p[kSlots], c[kSlots];
   float z[kSlots];
@@ -48,10 +49,29 @@ HS_DEVICE void route_token(int* __restrict__ ids_row, float* __restrict__ wts_ro
     float gbest = -INFINITY;   // lane g: group g's score
     for (int g = 0; g < groups; ++g) {
       float v = -INFINITY;
+      if (!top2) {
 #pragma unroll
-      for (int s = 0; s < kSlots; ++s)
-        if ((lane + 64 * s) / per == g) v = fmaxf(v, c[s]);
-      v = wave_max(v);
+        for (int s = 0; s < kSlots; ++s)
+          if ((lane + 64 * s) / per == g) v = fmaxf(v, c[s]);
+        v = wave_max(v);
+      } else {
+        // the largest and the second largest (ties count as two) of the lanes' own largest pairs
+        float a = -INFINITY, b = -INFINITY;
+#pragma unroll
+        for (int s = 0; s < kSlots; ++s) {
+          const int e = lane + 64 * s;
+          if (e / per == g && e < n) {
+            const float x = correction != nullptr ? c[s] : p[s];
+            b = fmaxf(b, fminf(a, x));
+            a = fmaxf(a, x);
+          }
+        }
+        v = wave_max(a);
+        if (per > 1) {
+          const int who = __builtin_ctzll(__ballot(a == v));
+          v += wave_max(lane == who ? b : a);
+        }
+      }
       if (lane == g) gbest = v;
     }
     unsigned long long allowed = 0;
@@ -106,11 +126,11 @@ __global__ __launch_bounds__(256) void route_topk_kernel(int* __restrict__ ids, 
                                                          const float* __restrict__ logits, long ld,
                                                          const float* __restrict__ correction, int T, int n, int top,
                                                          float scale, int E, int groups, int keep, bool renorm,
-                                                         bool sigmoid) {
+                                                         bool sigmoid, bool top2) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= T) return;
   route_token(ids + (long)t * top, wts + (long)t * top, nullptr, logits + (long)t * ld, correction, n, top, scale, E,
-              groups, keep, renorm, sigmoid);
+              groups, keep, renorm, sigmoid, top2);
 }
 
 // ---- router and alignment of a small batch in one workgroup: the choices go to LDS, pair p's place among the
@@ -122,13 +142,13 @@ __global__ __launch_bounds__(kAlignThreads) void route_align_kernel(
     int* __restrict__ ids, float* __restrict__ wts, int* __restrict__ slots, int cap, int* __restrict__ tile_expert,
     int tile, int* __restrict__ pair_slot, const float* __restrict__ logits, long ld,
     const float* __restrict__ correction, int T, int n, int top, float scale, int E, int nb, int groups, int keep,
-    bool renorm, bool sigmoid) {
+    bool renorm, bool sigmoid, bool top2) {
   __shared__ int sid[kMaxPairs], cnt[kMaxBuckets], off[kMaxBuckets];
   extern __shared__ int tab[];   // [cap] slots, [cap / tile] experts
   const int tid = threadIdx.x, P = T * top, nt = cap / tile;
   for (int t = tid >> 6; t < T; t += kAlignThreads / 64)
     route_token(ids + (long)t * top, wts + (long)t * top, sid + t * top, logits + (long)t * ld, correction, n, top, scale,
-                E, groups, keep, renorm, sigmoid);
+                E, groups, keep, renorm, sigmoid, top2);
   for (int i = tid; i < cap + nt; i += kAlignThreads) tab[i] = -1;
   __syncthreads();
   int rank = 0;
@@ -165,20 +185,21 @@ int route_align_max_slots() { return kMaxSlots; }
 
 void launch_route_align(int* ids, float* wts, int* slots, int cap, int* tile_expert, int tile, int* pair_slot,
                         const float* logits, long ld, const float* correction, int T, int n, int top, float scale, int E,
-                        int nb, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s) {
+                        int nb, int groups, int keep, bool renorm, bool sigmoid, bool top2, hipStream_t s) {
   if (T <= 0) return;
   route_align_kernel<<<1, kAlignThreads, (size_t)(cap + cap / tile) * sizeof(int), s>>>(
       ids, wts, slots, cap, tile_expert, tile, pair_slot, logits, ld, correction, T, n, top, scale, E, nb, groups, keep,
-      renorm, sigmoid);
+      renorm, sigmoid, top2);
 }
 
 int route_topk_max_outputs() { return 64 * kSlots; }
 
 void launch_route_topk(int* ids, float* wts, const float* logits, long ld, const float* correction, int T, int n,
-                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, hipStream_t s) {
+                       int top, float scale, int E, int groups, int keep, bool renorm, bool sigmoid, bool top2,
+                       hipStream_t s) {
   if (T <= 0) return;
   route_topk_kernel<<<(T + 3) / 4, 256, 0, s>>>(ids, wts, logits, ld, correction, T, n, top, scale, E, groups, keep, renorm,
-                                               sigmoid);
+                                               sigmoid, top2);
 }
 
 }  // namespace hipserve

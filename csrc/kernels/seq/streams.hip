@@ -16,37 +16,6 @@ namespace {
 constexpr int kNT = 256;
 constexpr int kMaxStreams = 32;   // of the run-time sized instantiation
 
-template <typename T, int V> struct Row;
-template <> struct Row<float, 1> {
-  static HS_DEVICE void ld(const float* p, float (&v)[1]) { v[0] = *p; }
-  static HS_DEVICE void st(float* p, const float (&v)[1]) { *p = v[0]; }
-};
-template <> struct Row<float, 4> {
-  static HS_DEVICE void ld(const float* p, float (&v)[4]) {
-    const f32x4 a = *reinterpret_cast<const f32x4*>(p);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = a[i];
-  }
-  static HS_DEVICE void st(float* p, const float (&v)[4]) { *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]}; }
-};
-template <> struct Row<unsigned short, 1> {
-  static HS_DEVICE void ld(const unsigned short* p, float (&v)[1]) { v[0] = bf16_to_f32(*p); }
-  static HS_DEVICE void st(unsigned short* p, const float (&v)[1]) { *p = f32_to_bf16(v[0]); }
-};
-template <> struct Row<unsigned short, 4> {
-  static HS_DEVICE void ld(const unsigned short* p, float (&v)[4]) {
-    const u16x4 a = *reinterpret_cast<const u16x4*>(p);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = bf16_to_f32(a[i]);
-  }
-  static HS_DEVICE void st(unsigned short* p, const float (&v)[4]) {
-    u16x4 a;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) a[i] = f32_to_bf16(v[i]);
-    *reinterpret_cast<u16x4*>(p) = a;
-  }
-};
-
 // SS streams (0: n_streams, at most kMaxStreams); V channels per thread and step (H % V == 0).
 template <typename T, int SS, int V>
 __global__ __launch_bounds__(kNT) void stream_update_kernel(

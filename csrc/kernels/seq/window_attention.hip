@@ -7,7 +7,8 @@
 // every head of `dim` elements with one weight of `dim` elements for all heads), the
 // rotate-half rotation of the first 2 * nfreq dims of every q / k head (angle = pos * inv_freq[i],
 // cos and sin times amp, fp32), the optional division of every rotated q / k head by its root mean
-// square (which the rotation changes only by amp, so it is taken from the unrotated head), the optional division of every value head by its root mean square, q written back in
+// square (which the rotation changes only by amp, so it is taken from the unrotated head), the optional
+// growth of the queries with their position, the optional division of every value head by its root mean square, q written back in
 // place, k and v into the cache row. Without a cache (a layer that reads another layer's keys and
 // values) the row is [q | ...] and only q is prepared.
 //
@@ -34,18 +35,18 @@ namespace {
 
 // One head's rotation work items: `dim - nfreq` per head; item i < nfreq is the pair (i, i + nfreq),
 // item i >= nfreq the unrotated element i + nfreq. Every element belongs to exactly one item.
-// `hinv` (per-head inverse rms, or null: `inv` for all) and `w` (null: none; wmod > 0: one weight of wmod
+// mul: a factor of every element. `hinv` (per-head inverse rms, or null: `inv` for all) and `w` (null: none; wmod > 0: one weight of wmod
 // elements shared by all heads, else a weight per element of the projection).
 template <typename T, typename F>
 HS_DEVICE void rotate_heads(const T* __restrict__ src, int nheads, int dim, int nfreq, float pos,
                             const float* __restrict__ inv_freq, float inv, const float* __restrict__ hinv,
-                            const float* __restrict__ w, int wmod, float amp, int tid, F&& store) {
+                            const float* __restrict__ w, int wmod, float amp, float mul, int tid, F&& store) {
   const int per = dim - nfreq;
   for (int it = tid; it < nheads * per; it += 256) {
     const int h = it / per, i = it % per;
     const int off = i < nfreq ? i : i + nfreq;
     const int e0 = h * dim + off;
-    const float sc = hinv != nullptr ? hinv[h] : inv;
+    const float sc = (hinv != nullptr ? hinv[h] : inv) * mul;
     float a = ldf<T>(src, e0) * sc;
     if (w != nullptr) a *= w[wmod > 0 ? off : e0];
     if (i < nfreq) {
@@ -72,7 +73,7 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
     T* __restrict__ proj, long ld, T* __restrict__ cache, const long* __restrict__ positions,
     const long* __restrict__ slots, const float* __restrict__ inv_freq, int nfreq, int heads, int kv_heads, int vheads,
     int dim, int vdim, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int norm_mode, bool v_norm,
-    float eps, float amp) {
+    float eps, float amp, float temp_coef, int temp_every) {
   extern __shared__ float hinv[];  // norm_mode 2, 3: [heads + kv_heads] inverse rms per head
   __shared__ float scratch[16];
   const long t = blockIdx.x;
@@ -106,14 +107,16 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
   const float* hq = norm_mode >= 2 ? hinv : nullptr;
   const int wmod = norm_mode == 2 ? dim : 0;
   const float pos = (float)positions[t];
-  rotate_heads<T>(row, heads, dim, nfreq, pos, inv_freq, iq, hq, q_norm, wmod, amp, tid,
+  // the query's factor: floor((p + 1) / every) in integers, the logarithm in fp32
+  const float temp = temp_every > 0 ? 1.f + temp_coef * logf((float)((positions[t] + 1) / temp_every) + 1.f) : 1.f;
+  rotate_heads<T>(row, heads, dim, nfreq, pos, inv_freq, iq, hq, q_norm, wmod, amp, temp, tid,
                   [&](int e, float v) { stf<T>(row, e, v); });
   if (!own_kv) return;
   const long slot = slots[t];
   if (slot < 0) return;
   T* dst = cache + slot * (long)(nk + nv);
   rotate_heads<T>(row + nq, kv_heads, dim, nfreq, pos, inv_freq, ik, hq != nullptr ? hq + heads : nullptr, k_norm,
-                  wmod, amp, tid, [&](int e, float v) { stf<T>(dst, e, v); });
+                  wmod, amp, 1.f, tid, [&](int e, float v) { stf<T>(dst, e, v); });
   const T* vr = row + nq + nk;
   for (int g = wave; g < vheads; g += 4) {  // one wave per value head
     float inv = 1.f;
@@ -156,7 +159,7 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
     int block_size, const int* __restrict__ seq_cu, const int* __restrict__ seq_ctx, const int* __restrict__ seq_bt,
     int bt_width, int seq0, int seq1, int tq, int hc, int hchunks, int heads, int kv_heads, int dim, int vdim,
     int gate_off, float scale, int window, bool sink, float out_scale, float lam, float post, float eps, int keep,
-    float softcap, const float* __restrict__ sink_w, bool channel_gate) {
+    float softcap, const float* __restrict__ sink_w, bool channel_gate, int chunk) {
   extern __shared__ float sm[];
   const int nrows = blockDim.x >> 6;
   const int qd = MAPS * dim;                       // a row's query elements
@@ -184,8 +187,7 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
     for (int e = lane; e < qd; e += 64) qs[wave * qd + e] = ldf<T>(q, e);
   }
   const int p_first = ctx - n + tok0, p_last = p_first + ntok - 1;
-  const int lo = window > 0 ? max(0, p_first - window + 1) : 0;
-  const int my_lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = first_key(p_first, window, chunk), my_lo = first_key(pos, window, chunk);
   const int nk = (window > 0 && keep > 0) ? min(keep, lo) : 0;   // kept keys below the workgroup's window
   const int total = nk + p_last - lo + 1;
   const float sink0 = (sink && sink_w != nullptr) ? sink_w[head] : 0.f;
@@ -298,17 +300,19 @@ __global__ __launch_bounds__(64 * kMaxRows) void window_attention_kernel(
 void launch_attn_prepare(void* proj, long ld, void* cache, const long* positions, const long* slots,
                          const float* inv_freq, int nfreq, int T, int heads, int kv_heads, int maps, int dim, int vdim,
                          const float* q_norm, const float* k_norm, int norm_mode, bool v_norm, float eps, float amp,
-                         bool f32, hipStream_t s) {
+                         float temp_coef, int temp_every, bool f32, hipStream_t s) {
   if (T <= 0) return;
   const int qh = heads * maps, kh = kv_heads * maps;
   const size_t smem = (size_t)(qh + kh) * sizeof(float);
   if (f32)
     attn_prepare_kernel<float><<<T, 256, smem, s>>>((float*)proj, ld, (float*)cache, positions, slots, inv_freq, nfreq,
-                                                    qh, kh, kv_heads, dim, vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp);
+                                                    qh, kh, kv_heads, dim, vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp,
+                                                    temp_coef, temp_every);
   else
     attn_prepare_kernel<unsigned short><<<T, 256, smem, s>>>((unsigned short*)proj, ld, (unsigned short*)cache,
                                                              positions, slots, inv_freq, nfreq, qh, kh, kv_heads, dim,
-                                                             vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp);
+                                                             vdim, q_norm, k_norm, norm_mode, v_norm, eps, amp, temp_coef,
+                                                             temp_every);
 }
 
 int window_attention_max_vdim() { return kMaxCh * kDC; }
@@ -319,7 +323,7 @@ void launch_generic(void* out, long out_ld, const void* proj, long proj_ld, cons
                     const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                     int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale,
                     int window, bool sink, float out_scale, float lam, float post, float eps, int keep, float softcap,
-                    const float* sink_w, bool channel_gate, hipStream_t s) {
+                    const float* sink_w, bool channel_gate, int chunk, hipStream_t s) {
   const int group = heads / kv_heads;
   auto lds = [&](int rows) {
     return ((size_t)rows * MAPS * dim + kKT * (kDC + 1) + (size_t)rows * MAPS * kKT) * sizeof(float) +
@@ -335,7 +339,7 @@ void launch_generic(void* out, long out_ld, const void* proj, long proj_ld, cons
   window_attention_kernel<T, MAPS><<<grid, block, lds(nrows), s>>>(
       (T*)out, out_ld, (const T*)proj, proj_ld, (const T*)cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0,
       seq1, tq, hc, hchunks, heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, lam, post, eps, keep,
-      softcap, sink_w, channel_gate);
+      softcap, sink_w, channel_gate, chunk);
 }
 }  // namespace
 
@@ -343,13 +347,13 @@ void launch_window_attention(void* out, long out_ld, const void* proj, long proj
                              const int* seq_cu, const int* seq_ctx, const int* seq_bt, int bt_width, int seq0, int seq1,
                              int rows_bound, int tq, int heads, int kv_heads, int dim, int vdim, int gate_off,
                              float scale, int window, bool sink, float out_scale, int maps, float lam, float post,
-                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, bool f32,
-                             hipStream_t s) {
+                             float eps, int keep, float softcap, const float* sink_w, bool channel_gate, int chunk,
+                             bool f32, hipStream_t s) {
   if (seq1 <= seq0 || rows_bound <= 0) return;
 #define HS_GA(T, M)                                                                                                  \
   launch_generic<T, M>(out, out_ld, proj, proj_ld, cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0, seq1,  \
                        rows_bound, tq, heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, lam, post, \
-                       eps, keep, softcap, sink_w, channel_gate, s)
+                       eps, keep, softcap, sink_w, channel_gate, chunk, s)
   if (f32) { if (maps == 2) HS_GA(float, 2); else HS_GA(float, 1); }
   else { if (maps == 2) HS_GA(unsigned short, 2); else HS_GA(unsigned short, 1); }
 #undef HS_GA

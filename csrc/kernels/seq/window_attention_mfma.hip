@@ -19,6 +19,8 @@
 //      both where P's registers already are and one 16-byte read of the transposed value tile.
 // Rows with few tokens and many keys (decode) split their keys over grid.z; the runs' unnormalised
 // outputs and (max, sum) are merged by window_attention_reduce.
+// chunk > 0 (no window): a row sees its own chunk of that many positions; the workgroup's run starts at its first
+// row's chunk.
 // keep > 0: the sequence's first `keep` keys stay visible behind the window. Tiles and runs walk a compacted
 // key index u: the nk kept keys below the workgroup's window first, then the window (key = u - nk + lo).
 //
@@ -68,7 +70,7 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
     int hchunks, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale, int window, bool sink,
     float out_scale, int part_keys, float* __restrict__ ws_acc, float* __restrict__ ws_ml, int row_base, int ws_rows,
     float lam, float post, float eps, bool one_row_seqs, bool qvec, int keep, float softcap,
-    const float* __restrict__ sink_w, bool channel_gate) {
+    const float* __restrict__ sink_w, bool channel_gate, int chunk) {
   static_assert(!DIFF || MT % 2 == 0, "a wave's row tiles come in pairs: the two maps of the same 16 rows");
   constexpr int RT = DIFF ? MT / 2 : MT;   // distinct 16-row tiles per wave; tile mt is rows mt / kMaps, map mt % kMaps
   constexpr int kLd = KLd<KS>::v;
@@ -92,7 +94,7 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
   const int r0 = seq_cu[s], n = seq_cu[s + 1] - r0, ctx = seq_ctx[s];
   const int ntok = min(tq, n - tok0);
   const int p_first = ctx - n + tok0, p_last = p_first + ntok - 1;
-  const int lo_all = window > 0 ? max(0, p_first - window + 1) : 0;
+  const int lo_all = first_key(p_first, window, chunk);
   const int nk = (window > 0 && keep > 0) ? min(keep, lo_all) : 0;   // kept keys below the workgroup's window
   const int total = nk + p_last - lo_all + 1;
   const int lo = blockIdx.z * part_keys;                              // compacted key indices from here on
@@ -118,7 +120,7 @@ __global__ __launch_bounds__(kThreads, 2) void window_attention_mfma_kernel(
     head[mt] = kvh * group + h0 + (sact[mt] ? srh : 0);
     trow[mt] = r0 + tok0 + (sact[mt] ? srt : 0);
     spos[mt] = p_first + srt;
-    s_lo[mt] = window > 0 ? max(0, spos[mt] - window + 1) : 0;
+    s_lo[mt] = first_key(spos[mt], window, chunk);
     const unsigned short* src = proj + trow[mt] * proj_ld + ((long)head[mt] * kMaps + (DIFF ? mt & 1 : 0)) * dim;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -420,7 +422,7 @@ void launch_mfma(unsigned short* out, long out_ld, const unsigned short* proj, l
                  int seq1, int rows_bound, int heads, int kv_heads, int dim, int vdim, int gate_off, float scale,
                  int window, bool sink, float out_scale, int nparts, int part_keys, float* ws_acc, float* ws_ml,
                  int row_base, float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                 bool channel_gate, hipStream_t s) {
+                 bool channel_gate, int chunk, hipStream_t s) {
   const int group = heads / kv_heads;
   const int rows = kRows * (DIFF ? MT / 2 : MT);
   const int hc = min(group, rows);
@@ -434,7 +436,7 @@ void launch_mfma(unsigned short* out, long out_ld, const unsigned short* proj, l
   window_attention_mfma_kernel<KS, NV, MT, DIFF><<<grid, kThreads, 0, s>>>(
       out, out_ld, proj, proj_ld, cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0, seq1, tq, hc, hchunks,
       heads, kv_heads, dim, vdim, gate_off, scale, window, sink, out_scale, part_keys, ws_acc, ws_ml, row_base,
-      rows_bound, lam, post, eps, one_row_seqs, qvec, keep, softcap, sink_w, channel_gate);
+      rows_bound, lam, post, eps, one_row_seqs, qvec, keep, softcap, sink_w, channel_gate, chunk);
   if (nparts > 1 && DIFF)
     window_attention_diff_reduce_kernel<<<dim3(rows_bound, heads), 128, 0, s>>>(
         out, out_ld, ws_acc, ws_ml, proj, proj_ld, gate_off, nparts, heads, rows_bound, row_base, vdim, out_scale, lam,
@@ -459,14 +461,14 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
                                   int vdim, int gate_off, float scale, int window, bool sink, float out_scale,
                                   int nparts, int part_keys, float* ws_acc, float* ws_ml, int row_base, int maps,
                                   float lam, float post, float eps, int keep, float softcap, const float* sink_w,
-                                  bool channel_gate, hipStream_t s) {
+                                  bool channel_gate, int chunk, hipStream_t s) {
   if (seq1 <= seq0 || rows_bound <= 0) return;
 #define HS_WA(KS, NV, MT, DIFF)                                                                                     \
   launch_mfma<KS, NV, MT, DIFF>((unsigned short*)out, out_ld, (const unsigned short*)proj, proj_ld,                  \
                                 (const unsigned short*)cache, block_size, seq_cu, seq_ctx, seq_bt, bt_width, seq0,    \
                                 seq1, rows_bound, heads, kv_heads, dim, vdim, gate_off, scale, window, sink,          \
                                 out_scale, nparts, part_keys, ws_acc, ws_ml, row_base, lam, post, eps, keep, softcap,  \
-                                sink_w, channel_gate, s)
+                                sink_w, channel_gate, chunk, s)
   // two row tiles per wave where a prompt portion brings enough rows and the accumulators fit the registers, except
   // where 128-row workgroups would all be resident at once (two per CU): the rows with few visible keys then leave their
   // CU idle, and twice as many smaller workgroups even that out (8192 rows x 8 heads: 183 -> 143 us)

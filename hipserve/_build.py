@@ -40,8 +40,8 @@ HIP_FLAGS = [
 # kernel libraries: name -> (shared object, kernel sources, host bindings). "core" is every
 # dense-transformer / sampling / quantisation kernel; "seq" the latent-attention / minGRU / table-MoE
 # kernels of the layer-list decoders (plus the expert alignment of moe.hip); "delta" their window and
-# differential attention, delta-rule and decayed linear-attention recurrences, softmax router and
-# activations; "cell" the parallel block with gated sublayer results, the mLSTM matrix memory, PolyNorm and
+# differential attention, delta-rule and decayed linear-attention recurrences, the residual updates with norms on
+# both sides, softmax router and activations; "cell" the parallel block with gated sublayer results, the mLSTM matrix memory, PolyNorm and
 # the gate multiply, plus the latent and window attention, router and activations that such a model also
 # runs; "stream" the residual streams' update and lightning attention beside the window attention, router and
 # experts. Kernel files shared by several libraries are compiled once and linked into each, so a model of
@@ -51,7 +51,7 @@ LIBS = {
     "seq": ("_C_seq.so", ["kernels/seq/group_norm.hip", "kernels/seq/latent_attention*.hip", "kernels/seq/mingru.hip",
                           "kernels/seq/expert_ffn.hip", "kernels/moe.hip"], "seq_bindings.cpp"),
     "delta": ("_C_delta.so", ["kernels/seq/group_norm.hip", "kernels/seq/window_attention*.hip",
-                              "kernels/seq/delta_scan.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",
+                              "kernels/seq/delta_scan.hip", "kernels/seq/sandwich.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",
                               "kernels/seq/elementwise.hip", "kernels/moe.hip"], "seq_delta_bindings.cpp"),
     "cell": ("_C_cell.so", ["kernels/seq/gated_block.hip", "kernels/seq/mlstm.hip", "kernels/seq/latent_attention*.hip",
                             "kernels/seq/window_attention*.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",

@@ -642,6 +642,33 @@ class YarnScaling:
 
 
 @dataclass(frozen=True)
+class LlamaScaling:
+    """Stretching of rotary frequencies as in Llama 3.1: pairs whose wave is longer than ``original / low`` positions are
+    slowed down by ``factor``, waves shorter than ``original / high`` are kept, and between the two the slowed and the kept
+    frequency are blended by the number of turns over ``original``. cos and sin keep their size."""
+    factor: float
+    original: float
+    low: float
+    high: float
+
+    amplitude = 1.0
+
+    def frequencies(self, base: float, dims: int) -> list:
+        """Angle per position of every pair i < dims / 2 (computed in double precision)."""
+        out = []
+        for i in range(dims // 2):
+            f = base ** (-2.0 * i / dims)
+            turns = self.original * f / (2.0 * math.pi)
+            if turns < self.low:
+                f /= self.factor
+            elif turns <= self.high:
+                blend = (turns - self.low) / (self.high - self.low)
+                f *= (1.0 - blend) / self.factor + blend
+            out.append(f)
+        return out
+
+
+@dataclass(frozen=True)
 class WindowAttentionSpec:
     """Grouped-query attention over a sliding window (``window`` keys: the token itself and
     the ``window - 1`` before it; 0 = plain causal) with rotate-half rotary positions on the
@@ -658,7 +685,10 @@ class WindowAttentionSpec:
     every query / key head by its root mean square AFTER the rotation (no weight), ``v_norm`` divides
     every value head by its root mean square (cached so), ``out_bias`` adds a bias in the
     output projection. ``interleaved``: the rotation pairs coordinate 2i with 2i + 1 (else i with
-    i + rot_dims / 2); ``yarn`` stretches its frequencies and its cos / sin.
+    i + rot_dims / 2); ``yarn`` stretches its frequencies and its cos / sin, ``llama`` its frequencies.
+    ``chunk`` > 0 (instead of a window): positions fall into chunks of that many, counted from the
+    sequence's start, and a token sees only its own chunk. ``temp_every`` > 0: the query at position p
+    is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1).
 
     ``maps`` = 2 is differential attention: every query head and every key head carries two
     maps side by side ([map 1 | map 2], ``dim`` each); each map is a softmax attention of its
@@ -690,8 +720,22 @@ class WindowAttentionSpec:
     unit_qk: bool = False
     interleaved: bool = False
     yarn: YarnScaling | None = None
+    llama: LlamaScaling | None = None
+    chunk: int = 0
+    temp_coef: float = 0.0
+    temp_every: int = 0
 
     kind = "attention"
+
+    @property
+    def scaling(self):
+        """The stretching of the rotary frequencies, if any."""
+        return self.yarn or self.llama
+
+    @property
+    def reach(self) -> int:
+        """Most keys a row can see behind a window or in a chunk (0: no bound)."""
+        return self.window + self.keep_first if self.window > 0 else self.chunk
 
     @property
     def gate_size(self) -> int:
@@ -739,12 +783,17 @@ class GatedDeltaSpec:
     """Gated delta rule: per head a ``dim x vdim`` state that decays by one number per token
     and is corrected towards the token's value along its unit key; q, k and v pass a causal
     convolution of ``conv`` taps and SiLU first. ``kv_heads`` query / key heads serve ``heads``
-    value heads."""
+    value heads. ``channel_decay``: a decay per head and key channel instead, from a bottleneck
+    (its width is read from the checkpoint). ``gate_bottleneck``: the output gate comes from a
+    bottleneck too. ``gate_act``: ``silu`` or ``sigmoid`` of the output gate."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv: int
+    channel_decay: bool = False
+    gate_bottleneck: bool = False
+    gate_act: str = "silu"
 
     kind = "delta"
 
@@ -753,9 +802,13 @@ class GatedDeltaSpec:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
     @property
+    def out_size(self) -> int:
+        return self.heads * self.vdim
+
+    @property
     def proj_size(self) -> int:
-        """Merged input projection: q | k | v | beta | decay | output gate."""
-        return self.conv_channels + 2 * self.heads + self.heads * self.vdim
+        """Merged input projection: q | k | v | beta | decay | output gate (the last two without bottlenecks)."""
+        return self.conv_channels + self.heads * (1 if self.channel_decay else 2) + (0 if self.gate_bottleneck else self.out_size)
 
 
 @dataclass(frozen=True)
@@ -816,11 +869,13 @@ class LightningSpec:
 
 @dataclass(frozen=True)
 class ParallelMixerSpec:
-    """Two mixers on the same input, their outputs summed with fixed weights."""
+    """Two mixers on the same input, their outputs summed with fixed weights. ``out_norms``: each output
+    is RMS-normed over the model width with a weight of its own first."""
     left: object
     right: object
     left_scale: float = 1.0
     right_scale: float = 1.0
+    out_norms: bool = False
 
     kind = "parallel"
 
@@ -829,9 +884,11 @@ class ParallelMixerSpec:
 class DenseFFSpec:
     """down(act(up(x))) with one of the op set's elementwise activations (``xielu``, ``relu2``) or
     ``polynorm``: a N(z) + b N(z^2) + c N(z^3) + e with four learned numbers, N dividing a token's
-    vector by its root mean square."""
+    vector by its root mean square. ``clamped_glu``: down(g sigmoid(1.702 g) (u + 1)) with
+    g = min(gate(x), limit), u = clamp(up(x), -limit, limit)."""
     ff: int
     act: str = "xielu"
+    limit: float = 0.0
 
     kind = "dense"
 
@@ -848,8 +905,8 @@ class RoutedMoESpec:
     number per token. The last ``identity`` router outputs are experts
     without weights that return their input; ``shared_ff`` > 0 adds a gated feed-forward that
     every token runs. ``groups`` > 1: the router outputs form that many equal groups of
-    neighbours, a group scores the largest corrected score in it, and only the experts of the
-    ``keep_groups`` best groups can be chosen. ``renorm``: the chosen scores are divided by
+    neighbours, a group scores the largest corrected score in it (``group_top2``: the sum of the two
+    largest), and only the experts of the ``keep_groups`` best groups can be chosen. ``renorm``: the chosen scores are divided by
     their sum before the scaling."""
     experts: int
     top: int
@@ -867,6 +924,7 @@ class RoutedMoESpec:
     limit: float = 0.0
     shared_limit: float = 0.0
     shared_gate: bool = False
+    group_top2: bool = False
 
     kind = "routed_moe"
 
@@ -1366,6 +1424,118 @@ class ZinavikConfig:
             eos_token_id=eos)
 
 
+@dataclass(frozen=True)
+class LugetarConfig:
+    """Lugetar: a decoder given as a list of layers with a norm before AND after every sublayer,
+
+        x <- x + m norm1b(mixer(norm1 x));  x <- x + m norm2b(ff(norm2 x))
+
+    with one multiplier m for the model. Mixers: chunked grouped-query attention (Llama 3.1 rotation)
+    beside a gated delta rule with a decay per key channel, each half's output normed over the width
+    before they are averaged; or plain causal attention without positions whose queries grow with
+    their position. Both kinds of attention norm the whole query / key projection. Feed-forwards: a
+    clamped gated one, or sigmoid-routed experts (the groups score the sum of their two best) with a
+    gated shared expert; a layer may have none. The embedding is scaled by ``embed_scale``; the logits
+    read the unscaled table."""
+    name: str = "lugetar"
+    architecture: str = "lugetar"
+    family: str = "lugetar"
+    hidden_size: int = 256
+    vocab_size: int = 512
+    layers: tuple = ()
+    norm_eps: float = 1e-6
+    embed_scale: float = 1.0
+    residual_mult: float = 1.0
+    max_position_embeddings: int = 1 << 20   # rotary angles are computed, not tabulated
+    default_model_len: int = 32768
+    bos_token_id: int | None = None
+    eos_token_id: tuple = ()
+    vision: object = None
+    num_experts: int = 0                      # engine start-up tuning of the dense families keys on it
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list:
+        """Layer runs in execution order: (layer index, 0, False); every layer runs once."""
+        return [(i, 0, False) for i in range(len(self.layers))]
+
+    def num_params(self) -> int:
+        """Without the bottlenecks' weights, whose widths only the checkpoint has."""
+        H, n = self.hidden_size, self.vocab_size * self.hidden_size
+
+        def mixer(m):
+            if isinstance(m, ParallelMixerSpec):
+                return mixer(m.left) + mixer(m.right)
+            if isinstance(m, GatedDeltaSpec):
+                return H * (m.proj_size + m.out_size)
+            return H * (m.q_size + m.cache_dim + m.heads * m.vdim)
+
+        for l in self.layers:
+            f = l.mlp
+            n += mixer(l.mixer)
+            if isinstance(f, DenseFFSpec):
+                n += 3 * f.ff * H
+            elif f is not None:
+                n += 3 * H * (f.experts * f.ff + f.shared_ff) + H * (f.experts + (1 if f.shared_gate else 0))
+        return n
+
+    def replace(self, **kw) -> "LugetarConfig":
+        return dataclasses.replace(self, **kw)
+
+    @staticmethod
+    def attention_spec(m: dict) -> WindowAttentionSpec:
+        rot, temp = m.get("rot") or {}, m.get("q_temp") or {}
+        sc = rot.get("scaling")
+        llama = LlamaScaling(float(sc["factor"]), float(sc["original"]), float(sc["low"]), float(sc["high"])) if sc else None
+        return WindowAttentionSpec(
+            heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+            scale=float(m["scale"]), chunk=int((m.get("mask") or {}).get("size") or 0), rot_dims=int(rot.get("dims") or 0),
+            rot_base=float(rot.get("base", 10000.0)), llama=llama, qk_norm=True, temp_coef=float(temp.get("coef") or 0.0),
+            temp_every=int(temp.get("every") or 0))
+
+    @staticmethod
+    def mlp_spec(f: dict):
+        if f.get("kind") == "dense":
+            return DenseFFSpec(ff=int(f["ff"]), act="clamped_glu", limit=float(f["limit"]))
+        if f.get("kind") != "moe":
+            raise NotImplementedError(f"unknown feed-forward {f.get('kind')!r}")
+        r, sh = f["router"], f.get("shared") or {}
+        g = r.get("groups") or {}
+        count = int(g.get("count") or 1)
+        keep = int(g.get("keep") or count)
+        if int(r["experts"]) % count or not 1 <= keep <= count or keep * (int(r["experts"]) // count) < int(r["top"]):
+            raise ValueError("the experts do not divide into equal groups that can hold the choice")
+        return RoutedMoESpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(f["expert"]["ff"]),
+                             scale=float(r.get("scale", 1.0)), shared_ff=int(sh.get("ff") or 0), shared_gate=bool(sh),
+                             groups=count, keep_groups=keep, group_top2=True, score="sigmoid", correction=False)
+
+    @staticmethod
+    def from_dict(d: dict, name: str = "model") -> "LugetarConfig":
+        layers = []
+        for l in d["layers"]:
+            m = l["mixer"]
+            if l["type"] == "parallel":
+                r = m["right"]
+                right = GatedDeltaSpec(heads=int(r["heads"]), kv_heads=int(r["kv_heads"]), dim=int(r["dim"]),
+                                       vdim=int(r["vdim"]), conv=int(r["conv"]), channel_decay=True, gate_bottleneck=True,
+                                       gate_act="sigmoid")
+                mixer = ParallelMixerSpec(LugetarConfig.attention_spec(m["left"]), right, 0.5, 0.5, out_norms=True)
+            elif l["type"] == "attention":
+                mixer = LugetarConfig.attention_spec(m)
+            else:
+                raise NotImplementedError(f"unknown mixer {l['type']!r}")
+            layers.append(HybridLayerSpec(mixer, LugetarConfig.mlp_spec(l["mlp"]) if l.get("mlp") is not None else None))
+        eos = d.get("eos_token_id", ())
+        eos = tuple(eos) if isinstance(eos, (list, tuple)) else (eos,)
+        return LugetarConfig(
+            name=name, hidden_size=int(d["width"]), vocab_size=int(d["vocab"]), layers=tuple(layers),
+            norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)),
+            embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+            residual_mult=float(d.get("residual_mult", 1.0)), bos_token_id=d.get("bos_token_id"), eos_token_id=eos)
+
+
 def check_kv_sources(layers):
     """A layer that reads another layer's keys and values must name an earlier attention layer
     with a cache of its own and the same key / value head layout."""
@@ -1394,6 +1564,8 @@ def config_from_dict(d: dict, name: str = "model"):
         return TopezenConfig.from_dict(d, name=name)
     if arch == "zinavik":
         return ZinavikConfig.from_dict(d, name=name)
+    if arch == "lugetar":
+        return LugetarConfig.from_dict(d, name=name)
     return ModelConfig.from_hf_dict(d, name=name)
 
 
@@ -1536,4 +1708,37 @@ PRESETS.update({
                                    dict(heads=4, dim=64, vdim=64),
                                    dict(experts=8, top=2, ff=256, limit=7.0, shared_ff=512, shared_limit=7.0), "ppn",
                                    loop=(0, 2, 2), streams=4),
+})
+
+
+def _mini_lugetar(name, H, V, left, right, attn, ff, moe, order, limit=5.0, embed_scale=4.0, mult=0.5):
+    """order: 'p' parallel mixer + clamped feed-forward, 'a' causal attention + routed experts, 'n' parallel mixer
+    without a feed-forward, 'd' causal attention + clamped feed-forward."""
+    p = ParallelMixerSpec(WindowAttentionSpec(qk_norm=True, **left),
+                          GatedDeltaSpec(channel_decay=True, gate_bottleneck=True, gate_act="sigmoid", **right), 0.5, 0.5,
+                          out_norms=True)
+    a = WindowAttentionSpec(qk_norm=True, **attn)
+    f = DenseFFSpec(ff, "clamped_glu", limit)
+    e = RoutedMoESpec(score="sigmoid", correction=False, shared_gate=True, group_top2=True, **moe)
+    spec = {"p": HybridLayerSpec(p, f), "a": HybridLayerSpec(a, e), "n": HybridLayerSpec(p, None), "d": HybridLayerSpec(a, f)}
+    return LugetarConfig(name=name, hidden_size=H, vocab_size=V, layers=tuple(spec[c] for c in order),
+                         embed_scale=embed_scale, residual_mult=mult, eos_token_id=(2,), bos_token_id=1)
+
+
+PRESETS.update({
+    # CPU plumbing size
+    "tiny-lugetar": _mini_lugetar("tiny-lugetar", 64, 320,
+                                  dict(heads=4, kv_heads=2, dim=16, vdim=24, scale=0.3, chunk=20, rot_dims=12,
+                                       llama=LlamaScaling(2.0, 64, 1.0, 4.0)),
+                                  dict(heads=4, kv_heads=2, dim=16, vdim=24, conv=4),
+                                  dict(heads=4, kv_heads=1, dim=24, vdim=16, scale=0.2, temp_coef=0.3, temp_every=10), 96,
+                                  dict(experts=6, top=2, ff=24, scale=1.5, shared_ff=40, groups=3, keep_groups=2), "pand"),
+    # GPU-test size
+    "small-lugetar": _mini_lugetar("small-lugetar", 512, 1024,
+                                   dict(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.125, chunk=160, rot_dims=64,
+                                        rot_base=50000.0, llama=LlamaScaling(4.0, 1024, 1.0, 4.0)),
+                                   dict(heads=4, kv_heads=4, dim=64, vdim=64, conv=4),
+                                   dict(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.125, temp_coef=0.2, temp_every=128),
+                                   1024, dict(experts=8, top=2, ff=256, scale=1.5, shared_ff=512, groups=4, keep_groups=2),
+                                   "papa"),
 })

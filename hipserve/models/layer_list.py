@@ -20,6 +20,7 @@ from .mixers import make_ff, make_mixer
 class _Layer:
     def __init__(self):
         self.norm1 = self.norm2 = None   # [hidden] fp32 (one number each in designs with single-weight norms)
+        self.norm1b = self.norm2b = None  # [hidden] fp32: norms of the sublayers' results, in designs that have both
         self.b1 = self.b2 = None         # [hidden] fp32: biases of the gates on the sublayers' results, where a design has them
         self.mixer = None
         self.mlp = None

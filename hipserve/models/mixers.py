@@ -35,7 +35,11 @@ them is one op of the op set:
   expert are folded into the residual update (``add_normed``).
 * gated delta rule: merged [q | k | v | beta | decay | gate] projection -> ``gated_delta``
   (causal convolution + SiLU, unit q / k, the recurrence from the sequence's state slot,
-  per-head output norm and SiLU gate) -> output projection.
+  per-head output norm and SiLU or sigmoid gate) -> output projection. With a decay per key channel
+  and an output gate that come from bottlenecks, the merged projection is [q | k | v | decay
+  bottleneck | gate bottleneck | beta] and the up-projections follow as GEMMs (the decay's with a
+  32-bit result); steps in which every sequence brings one row run ``gated_delta_step`` instead, the
+  bottlenecks' up-projections included.
 * generalized delta rule: merged [r | k | v | a | g | decay bottleneck] projection -> tanh ->
   decay up-projection (32-bit result) -> ``delta_rule`` (decay, removal rate, unit key, the
   recurrence, per-head output norm and sigmoid gate) -> output projection.
@@ -45,7 +49,11 @@ them is one op of the op set:
 * parallel mixer: both halves write their scaled head outputs side by side into one
   buffer, and ONE output projection over the concatenated weights sums them; where both
   halves can take their input projection from outside, ONE input projection serves both.
-* dense feed-forward: up projection -> ``activation`` -> down projection.
+  Where each half's output is normed first, the halves keep their output projections and
+  ``forward`` returns both results with the norms' weights (``NormedPair``) for the residual
+  update (``sandwich_update``), which norms and sums them.
+* dense feed-forward: up projection ([gate | up] for the clamped gate) -> ``activation`` -> down
+  projection.
 
 * matrix memory (``MLstm``): merged [q | k | v | gate] projection and a 32-bit [input gate | forget
   gate] projection -> ``mlstm`` (capped log gates, running maximum, the recurrence of the matrix
@@ -60,6 +68,8 @@ the sublayer's result, say) attaches its rows to the sublayer's merged input GEM
 ``attach_side``; after ``forward`` the sublayer's ``side_out`` holds those columns.
 """
 from __future__ import annotations
+
+from typing import NamedTuple
 
 import torch
 import torch.nn.functional as F
@@ -344,11 +354,12 @@ class WindowAttention:
         # f_i = base^(-2i / dims), 32-bit
         self.inv_freq = torch.pow(torch.tensor(spec.rot_base, dtype=torch.float32),
                                   -2.0 * i / max(spec.rot_dims, 1)).to(device)
-        if spec.yarn is not None:
-            self.inv_freq = torch.tensor(spec.yarn.frequencies(spec.rot_base, spec.rot_dims), dtype=torch.float32).to(device)
+        if spec.scaling is not None:
+            self.inv_freq = torch.tensor(spec.scaling.frequencies(spec.rot_base, spec.rot_dims), dtype=torch.float32).to(device)
         self.gate_off = spec.q_size + spec.cache_dim if spec.gate_size else -1
         assert spec.maps in (1, 2) and not (spec.gate_size and spec.kv_from is not None)
         assert not (spec.channel_gate and spec.maps == 2) and not (spec.unit_qk and (spec.qk_norm or spec.head_norm))
+        assert not (spec.chunk and (spec.window or spec.keep_first)) and not (spec.yarn and spec.llama)
 
     @property
     def out_size(self) -> int:
@@ -494,26 +505,48 @@ class Wkv:
 
 class GatedDelta:
     cache_dim = 0
+    takes_proj = True
+    STEP_MAX_DIM, STEP_MAX_RANK = 256, 1024   # sizes the one-row-per-sequence kernel takes
 
     def __init__(self, spec: GatedDeltaSpec, hidden: int, eps: float, device, dtype, ops):
         self.spec, self.hidden, self.eps, self.device, self.dtype, self.ops = spec, hidden, eps, device, dtype, ops
-        self.w_in = None      # [q | k | v | beta | decay | gate, hidden]
+        # [q | k | v | beta | decay | gate, hidden]; with bottlenecks [q | k | v | decay bottleneck | gate bottleneck |
+        # beta, hidden], every part but the first two of the convolution's padded to a multiple of 8 rows
+        self.w_in = None
         self.conv_w = None    # fp32 [conv channels, taps]
-        self.a_log = self.dt_bias = None  # fp32 [heads]
+        self.a_log = self.dt_bias = None  # fp32 [heads]; [heads], or [heads * dim] with a decay per channel
         self.norm = None      # fp32 [vdim]
         self.w_o = None
+        self.w_a2 = self.w_g2 = None   # the bottlenecks' up-projections [heads * dim, rank], [heads * vdim, rank]
+        self.off_a = self.off_g = self.off_b = 0   # columns of the projection: decay (bottleneck), gate (bottleneck), beta
+        assert spec.gate_bottleneck == spec.channel_decay and spec.gate_act in ("silu", "sigmoid")
 
     @property
     def out_size(self) -> int:
-        return self.spec.heads * self.spec.vdim
+        return self.spec.out_size
 
     def state_shapes(self, slots: int):
         s = self.spec
         return [(slots, s.heads, s.dim, s.vdim), (slots, max(s.conv - 1, 1), s.conv_channels)]
 
     def load(self, get, prefix: str):
-        dt, dev = self.dtype, self.device
-        self.w_in = torch.cat([get(prefix + n) for n in ("q", "k", "v", "b", "a", "g")], 0).to(dev, dt).contiguous()
+        s, dt, dev = self.spec, self.dtype, self.device
+        if s.channel_decay:
+            qkv = torch.cat([get(prefix + n) for n in ("q", "k", "v")], 0)
+            parts, at, offs = [], 0, []
+            for w in (qkv, get(prefix + "a1"), get(prefix + "g1"), get(prefix + "b")):
+                offs.append(at)
+                n = -(-w.shape[0] // 8) * 8   # 16-byte aligned columns in bf16
+                parts.append(F.pad(w, (0, 0, 0, n - w.shape[0])))
+                at += n
+            self.off_a, self.off_g, self.off_b = offs[1:]
+            self.w_in = torch.cat(parts, 0).to(dev, dt).contiguous()
+            self.w_a2 = get(prefix + "a2").to(dev, dt).contiguous()
+            self.w_g2 = get(prefix + "g2").to(dev, dt).contiguous()
+        else:
+            self.off_b = s.conv_channels
+            self.off_a, self.off_g = self.off_b + s.heads, self.off_b + 2 * s.heads
+            self.w_in = torch.cat([get(prefix + n) for n in ("q", "k", "v", "b", "a", "g")], 0).to(dev, dt).contiguous()
         self.conv_w = torch.cat([get(prefix + n + ".conv") for n in ("q", "k", "v")], 0).to(dev, torch.float32).contiguous()
         self.a_log = get(prefix + "A_log").to(dev, torch.float32)
         self.dt_bias = get(prefix + "dt_bias").to(dev, torch.float32)
@@ -525,17 +558,37 @@ class GatedDelta:
         qk = s.kv_heads * s.dim
         t = {"q": _rand(gen, qk, H, std=std * 4), "k": _rand(gen, qk, H, std=std * 4),
              "v": _rand(gen, self.out_size, H, std=std * 4), "b": _rand(gen, s.heads, H, std=std * 4),
-             "a": _rand(gen, s.heads, H, std=std * 4), "g": _rand(gen, self.out_size, H, std=std * 4),
-             "A_log": _rand(gen, s.heads, std=0.5) - 1.0, "dt_bias": _rand(gen, s.heads, std=0.5),
-             "norm": 1.0 + 0.2 * _rand(gen, s.vdim), "o": _rand(gen, H, self.out_size, std=std)}
+             "A_log": _rand(gen, s.heads, std=0.5) - 1.0, "norm": 1.0 + 0.2 * _rand(gen, s.vdim),
+             "o": _rand(gen, H, self.out_size, std=std)}
+        if s.channel_decay:
+            rank = max(8, s.vdim // 8 * 8)
+            t.update({"a1": _rand(gen, rank, H, std=std * 4), "a2": _rand(gen, s.heads * s.dim, rank, std=0.2),
+                      "dt_bias": _rand(gen, s.heads * s.dim, std=0.5), "g1": _rand(gen, rank, H, std=std * 4),
+                      "g2": _rand(gen, self.out_size, rank, std=0.2)})
+        else:
+            t.update({"a": _rand(gen, s.heads, H, std=std * 4), "g": _rand(gen, self.out_size, H, std=std * 4),
+                      "dt_bias": _rand(gen, s.heads, std=0.5)})
         for n, c in (("q", qk), ("k", qk), ("v", self.out_size)):
             t[n + ".conv"] = _rand(gen, c, s.conv, std=0.5)
         return t
 
-    def mix(self, h, meta, cache, state, out, out_scale: float = 1.0):
+    def mix(self, h, meta, cache, state, out, out_scale: float = 1.0, proj=None):
+        s, ops = self.spec, self.ops
         assert out_scale == 1.0
-        proj = F.linear(h, self.w_in)
-        self.ops.gated_delta(out, state, proj, self.conv_w, self.a_log, self.dt_bias, self.norm, self.spec, self.eps, meta)
+        if proj is None:
+            proj = F.linear(h, self.w_in)
+        weights = (self.conv_w, self.a_log, self.dt_bias, self.norm)
+        offs = (self.off_a, self.off_g, self.off_b)
+        ra, rg = (self.w_a2.shape[1], self.w_g2.shape[1]) if s.channel_decay else (0, 0)
+        if meta.max_q == 1 and max(s.dim, s.vdim) <= self.STEP_MAX_DIM and ra + rg <= self.STEP_MAX_RANK:
+            # every sequence brings one row (decode steps): bottlenecks, convolution, recurrence, norm and gate
+            ops.gated_delta_step(out, state, proj, *weights, self.w_a2, self.w_g2, offs, s, self.eps, meta)
+            return out
+        decay = gate = None
+        if s.channel_decay:
+            decay = _linear32(proj[:, self.off_a:self.off_a + ra], self.w_a2)
+            gate = F.linear(proj[:, self.off_g:self.off_g + rg], self.w_g2)
+        ops.gated_delta(out, state, proj, *weights, decay, gate, offs, s, self.eps, meta)
         return out
 
     def forward(self, h, meta, cache, state):
@@ -685,15 +738,27 @@ class Lightning:
         return F.linear(self.mix(h, meta, cache, state, out), self.w_o)
 
 
+class NormedPair(NamedTuple):
+    """a_scale N(a) a_w + b_scale N(b) b_w of two results a, b [T, hidden], N dividing a row by its root mean square."""
+    a: torch.Tensor
+    a_w: torch.Tensor    # fp32 [hidden]
+    b: torch.Tensor
+    b_w: torch.Tensor
+    a_scale: float
+    b_scale: float
+
+
 class ParallelMixer:
     """left_scale * left(h) + right_scale * right(h): both halves write their scaled head outputs
-    into one [T, left | right] buffer; one GEMM with the concatenated output weights sums them."""
+    into one [T, left | right] buffer; one GEMM with the concatenated output weights sums them.
+    With ``spec.out_norms`` each half has an output GEMM of its own and ``forward`` returns a ``NormedPair``."""
 
     def __init__(self, spec: ParallelMixerSpec, hidden: int, eps: float, device, dtype, ops):
         self.spec, self.hidden, self.device, self.dtype, self.ops = spec, hidden, device, dtype, ops
         self.left = make_mixer(spec.left, hidden, eps, device, dtype, ops)
         self.right = make_mixer(spec.right, hidden, eps, device, dtype, ops)
         self.w_o = None      # [hidden, left out | right out]
+        self.left_norm = self.right_norm = None   # fp32 [hidden] with out_norms
         self.w_in = None     # [left inputs | zero rows up to a multiple of 8 | right inputs, hidden], when one GEMM serves both
         self.split = 0       # rows of w_in before the right half's
 
@@ -710,8 +775,12 @@ class ParallelMixer:
     def load(self, get, prefix: str):
         self.left.load(get, prefix + "left.")
         self.right.load(get, prefix + "right.")
-        self.w_o = torch.cat([self.left.w_o, self.right.w_o], 1).contiguous()
-        self.left.w_o = self.right.w_o = None
+        if self.spec.out_norms:
+            self.left_norm = get(prefix + "left.out").to(self.device, torch.float32).contiguous()
+            self.right_norm = get(prefix + "right.out").to(self.device, torch.float32).contiguous()
+        else:
+            self.w_o = torch.cat([self.left.w_o, self.right.w_o], 1).contiguous()
+            self.left.w_o = self.right.w_o = None
         if getattr(self.left, "takes_proj", False) and getattr(self.right, "takes_proj", False):
             wl, wr = self.left.w_in, self.right.w_in
             self.split = -(-wl.shape[0] // 8) * 8   # 16-byte aligned rows in bf16
@@ -721,9 +790,25 @@ class ParallelMixer:
     def init_random(self, gen, std: float):
         t = {"left." + k: v for k, v in self.left.init_random(gen, std).items()}
         t.update({"right." + k: v for k, v in self.right.init_random(gen, std).items()})
+        if self.spec.out_norms:
+            t.update({n + ".out": 1.0 + 0.2 * _rand(gen, self.hidden) for n in ("left", "right")})
         return t
 
+    def _forward_normed(self, h, meta, cache, state):
+        pl = pr = None
+        if self.w_in is not None:
+            proj = F.linear(h, self.w_in)
+            pl, pr = proj[:, :self.split], proj[:, self.split:]
+        ys = []
+        for m, p in ((self.left, pl), (self.right, pr)):
+            out = torch.empty(h.shape[0], m.out_size, device=h.device, dtype=h.dtype)
+            m.mix(h, meta, cache, state, out, 1.0, **({} if p is None else {"proj": p}))
+            ys.append(F.linear(out, m.w_o, getattr(m, "b_o", None)))
+        return NormedPair(ys[0], self.left_norm, ys[1], self.right_norm, self.spec.left_scale, self.spec.right_scale)
+
     def forward(self, h, meta, cache, state):
+        if self.spec.out_norms:
+            return self._forward_normed(h, meta, cache, state)
         a, b = self.left.out_size, self.right.out_size
         buf = torch.empty(h.shape[0], a + b, device=h.device, dtype=h.dtype)
         if self.w_in is not None:
@@ -747,7 +832,10 @@ class DenseFF:
 
     def load(self, get, prefix: str):
         dt, dev = self.dtype, self.device
-        self.w_up = get(prefix + "up").to(dev, dt).contiguous()
+        up = get(prefix + "up")
+        if self.spec.act == "clamped_glu":
+            up = torch.cat([get(prefix + "gate"), up], 0)
+        self.w_up = up.to(dev, dt).contiguous()
         self.w_down = get(prefix + "down").to(dev, dt).contiguous()
         if self.spec.act == "xielu":
             sp = F.softplus(get(prefix + "act").to(torch.float32))
@@ -761,6 +849,8 @@ class DenseFF:
             t["act"] = _rand(gen, 2, std=0.5)
         if self.spec.act == "polynorm":
             t["act"] = _rand(gen, 4, std=0.5)
+        if self.spec.act == "clamped_glu":
+            t["gate"] = _rand(gen, self.spec.ff, self.hidden, std=std * 4)
         return t
 
     def forward(self, h):
@@ -770,6 +860,10 @@ class DenseFF:
         if self.spec.act == "polynorm":
             act = torch.empty(h.shape[0], ff, device=h.device, dtype=h.dtype)
             self.ops.polynorm(act, up[:, :ff], self.coef, self.eps)
+            return F.linear(act, self.w_down)
+        if self.spec.act == "clamped_glu":
+            act = torch.empty(h.shape[0], ff, device=h.device, dtype=h.dtype)
+            self.ops.activation(act, up[:, :2 * ff], "clamped_glu", self.spec.limit)
             return F.linear(act, self.w_down)
         if self.side_rows:
             act = torch.empty(h.shape[0], ff, device=h.device, dtype=h.dtype)
@@ -844,7 +938,7 @@ class RoutedMoE:
             n = s.experts + s.identity
             logits, self.shared_gate = logits[:, :n], logits[:, n:]
         router = (logits, self.correction, s.top, s.scale, s.experts)
-        options = (s.groups, s.keep_groups, s.renorm, s.score)
+        options = (s.groups, s.keep_groups, s.renorm, s.score, s.group_top2)
         scale = wts if s.weight_input else None
         # the identity experts share one bucket (s.experts) that no GEMM tile serves
         P, nb = T * s.top, s.experts + (1 if s.identity else 0)

@@ -24,6 +24,7 @@ ARCHITECTURES = {
     "fikizen": ("hipserve.models.fikizen", "FikizenModel", "hipserve.weights.safetensors_loader:load_named_tensors"),
     "kemavik": ("hipserve.models.kemavik", "KemavikModel", "hipserve.weights.safetensors_loader:load_named_tensors"),
     "zinavik": ("hipserve.models.zinavik", "ZinavikModel", "hipserve.weights.safetensors_loader:load_named_tensors"),
+    "lugetar": ("hipserve.models.lugetar", "LugetarModel", "hipserve.weights.safetensors_loader:load_named_tensors"),
     "topezen": ("hipserve.models.topezen", "TopezenModel", "hipserve.weights.safetensors_loader:load_named_tensors"),
 }
 

@@ -292,7 +292,7 @@ class KernelOps:
         self._window_lib.attn_prepare(proj, cache if own_kv else None, meta.positions, meta.slot_mapping, inv_freq, sp.heads,
                                  sp.kv_heads, sp.maps, sp.dim, sp.vdim, q_norm if mode in (1, 2) else None,
                                  k_norm if mode in (1, 2) and own_kv else None, mode, sp.v_norm, eps,
-                                 sp.yarn.amplitude if sp.yarn is not None else 1.0)
+                                 sp.scaling.amplitude if sp.scaling is not None else 1.0, sp.temp_coef, sp.temp_every)
 
     WINDOW_PREFILL_TQ = 4  # tokens per workgroup of a prompt portion (x the query heads of one key/value head)
     # bf16 runs the MFMA kernel (HIPSERVE_WINDOW_MFMA=0: the generic kernel, as fp32 does)
@@ -307,7 +307,7 @@ class KernelOps:
         nseq = meta.seq_ctx.shape[0]
         nd = meta.num_decode
         npf, Tp = nseq - nd, meta.num_prefill_tokens
-        diff = (sp.maps, lam, 1.0 - sp.diff, eps, sp.keep_first, sp.softcap, sink_w, sp.channel_gate)
+        diff = (sp.maps, lam, 1.0 - sp.diff, eps, sp.keep_first, sp.softcap, sink_w, sp.channel_gate, sp.chunk)
         if (proj.dtype == torch.bfloat16 and self.WINDOW_MFMA
                 and self._window_lib.window_attention_mfma_ok(sp.dim, sp.vdim, out.stride(0), out.storage_offset(), sp.maps)):
             # bf16: the matrix-core kernel; decode rows split their keys into runs merged by a reduce kernel
@@ -316,9 +316,9 @@ class KernelOps:
                 self._window_lib.window_attention_mfma(out, proj, cache, meta.seq_cu, meta.seq_ctx, meta.seq_bt, 0, npf, Tp,
                                                 *args, 1, 0, None, None, 0, *diff)
             if nd:
-                # keys a row can see: its window and the kept first keys behind it
-                reach = sp.window + sp.keep_first
-                span = min(reach, meta.max_ctx or reach) if sp.window > 0 else meta.max_ctx
+                # keys a row can see: its window and the kept first keys behind it, or its chunk
+                reach = sp.reach
+                span = min(reach, meta.max_ctx or reach) if reach > 0 else meta.max_ctx
                 part = self.WINDOW_DECODE_RUN
                 if span >= 16 * part:   # long runs of keys: fewer, longer runs per row (measured at 2k and 8k keys)
                     part *= 2
@@ -338,12 +338,22 @@ class KernelOps:
                                            sp.heads, sp.kv_heads, sp.dim, sp.vdim, gate_off, sp.scale, sp.window,
                                            sp.sink, out_scale, *diff)
 
-    def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta):
+    def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps, meta):
+        """``decay`` (fp32) / ``gate``: the pre-activations that come from bottlenecks (None: columns of ``proj``);
+        ``offs``: the columns of ``proj`` where the decay, the gate and beta (or the bottlenecks) start."""
         T = proj.shape[0]
-        scratch = torch.empty(T * (2 * sp.kv_heads * sp.dim + 2 * sp.heads * sp.vdim + 2 * sp.heads),
+        scratch = torch.empty(T * (2 * sp.kv_heads * sp.dim + 2 * sp.out_size + sp.heads * (1 + (sp.dim if sp.channel_decay else 1))),
                               device=proj.device, dtype=torch.float32)
-        self._delta.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, meta.seq_cu, meta.seq_ctx,
-                              meta.seq_state, scratch, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.conv, eps)
+        self._delta.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, decay, gate, meta.seq_cu,
+                                meta.seq_ctx, meta.seq_state, scratch, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.conv, eps,
+                                *offs, sp.channel_decay, sp.gate_act == "silu")
+
+    def gated_delta_step(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, w_a2, w_g2, offs, sp, eps, meta):
+        """``gated_delta`` for steps in which every sequence has one row (``meta.max_q`` == 1), the bottlenecks'
+        up-projections ``w_a2`` / ``w_g2`` included."""
+        self._delta.gated_delta_step(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, w_a2, w_g2, meta.seq_cu,
+                                     meta.seq_ctx, meta.seq_state, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.conv, eps,
+                                     *offs, sp.channel_decay, sp.gate_act == "silu")
 
     def delta_rule(self, out, state, proj, wl, a_b, w0, norm_w, sp, eps, meta, out_scale=1.0):
         scratch = torch.empty(proj.shape[0] * 7 * sp.size, device=proj.device, dtype=torch.float32)
@@ -381,25 +391,25 @@ class KernelOps:
     ROUTER_MAX_OUTPUTS = 256
 
     def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False,
-                   score="softmax"):
+                   score="softmax", group_top2=False):
         if logits.shape[1] > self.ROUTER_MAX_OUTPUTS or groups > 64:
             # more router outputs than a wave holds: device-side torch ops
-            ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+            ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score, group_top2)
             return
         self._window_lib.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm,
-                                    score == "sigmoid")
+                                    score == "sigmoid", group_top2)
 
     ROUTE_ALIGN_PAIRS, ROUTE_ALIGN_SLOTS = 256, 8192   # batches whose router and alignment run in one launch
 
     def route_align(self, ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile, groups=1,
-                    keep_groups=1, renorm=False, score="softmax"):
+                    keep_groups=1, renorm=False, score="softmax", group_top2=False):
         """``route_topk`` and ``moe_align`` (``nb`` buckets) of the choices."""
         if (ids.numel() <= self.ROUTE_ALIGN_PAIRS and slots.numel() <= self.ROUTE_ALIGN_SLOTS and nb <= 128 and groups <= 64
                 and logits.shape[1] <= self.ROUTER_MAX_OUTPUTS and self._window_lib is self._moe_lib):
             self._window_lib.route_align(ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile,
-                                         groups, keep_groups, renorm, score == "sigmoid")
+                                         groups, keep_groups, renorm, score == "sigmoid", group_top2)
             return
-        self.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+        self.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score, group_top2)
         self.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
 
     # ---- parallel blocks with gated sublayer results, mLSTM, PolyNorm (csrc/kernels/seq/gated_block.hip, mlstm.hip,
@@ -459,6 +469,21 @@ class KernelOps:
         """act: False / 0 none, True / 1 squared ReLU, 2: w = [gate rows; up rows], out = silu(gate) * up, 3: the same
         with the gate clamped at ``limit``; ``row_scale`` fp32 [pairs] multiplies each pair's product before it."""
         self._moe_lib.expert_gemm(out, x, w, slots, tile_expert, tile, gather_k, int(act), row_scale, limit)
+
+    # ---- norms before and after every sublayer (csrc/kernels/seq/sandwich.hip)
+    def sandwich_update(self, out, residual, w_next, eps, y=None, w_post=None, mult=1.0, table=None):
+        rows, ids, scale = table if table is not None else (None, None, 1.0)
+        a = a_w = b = b_w = ye = pair_slot = wts = shared = gate = None
+        a_scale = b_scale = 1.0
+        if isinstance(y, tuple) and len(y) == 6:
+            a, a_w, b, b_w, a_scale, b_scale = y
+        elif isinstance(y, tuple):
+            ye, pair_slot, wts, shared, gate = y
+        else:
+            a = y
+        self._delta.sandwich_update(out, residual, w_next, eps, w_post, mult, rows, ids, scale, a, a_w, b, b_w, a_scale,
+                                    b_scale, ye, pair_slot, wts, shared, gate)
+        return out
 
     # ---- residual streams, lightning attention (csrc/kernels/seq/streams.hip, lightning.hip)
     def stream_update(self, out, dst, src, coef, w, eps, y1=None, y2=None):
@@ -658,17 +683,30 @@ class ReferenceOps:
         ref.wkv(out, state, proj, wl, w0, u, norm_w, sp, eps, meta.seq_cu, meta.seq_ctx, meta.seq_state)
 
     def route_topk(self, ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False,
-                   score="softmax"):
-        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+                   score="softmax", group_top2=False):
+        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score, group_top2)
 
     def route_align(self, ids, wts, slots, tile_expert, pair_slot, logits, correction, top, scale, E, nb, tile, groups=1,
-                    keep_groups=1, renorm=False, score="softmax"):
-        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score)
+                    keep_groups=1, renorm=False, score="softmax", group_top2=False):
+        ref.route_topk(ids, wts, logits, correction, top, scale, E, groups, keep_groups, renorm, score, group_top2)
         ref.moe_align(ids.view(-1), nb, tile, slots, tile_expert, pair_slot)
 
-    def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta):
-        ref.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, sp, eps, meta.seq_cu,
-                        meta.seq_ctx, meta.seq_state)
+    def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps, meta):
+        ref.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps,
+                        meta.seq_cu, meta.seq_ctx, meta.seq_state)
+
+    def gated_delta_step(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, w_a2, w_g2, offs, sp, eps, meta):
+        decay = gate = None
+        if sp.channel_decay:
+            low_a, low_g = (proj[:, o:o + w.shape[1]].float() for o, w in ((offs[0], w_a2), (offs[1], w_g2)))
+            decay = torch.nn.functional.linear(low_a, w_a2.float())
+            gate = torch.nn.functional.linear(low_g, w_g2.float())
+        ref.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps,
+                        meta.seq_cu, meta.seq_ctx, meta.seq_state)
+
+    def sandwich_update(self, out, residual, w_next, eps, y=None, w_post=None, mult=1.0, table=None):
+        ref.sandwich_update(out, residual, w_next, eps, y, w_post, mult, table)
+        return out
 
     def delta_rule(self, out, state, proj, wl, a_b, w0, norm_w, sp, eps, meta, out_scale=1.0):
         ref.delta_rule(out, state[0], proj, wl, a_b, w0, norm_w, sp, eps, meta.seq_cu, meta.seq_ctx,

@@ -564,8 +564,9 @@ def attn_prepare(proj, cache, positions, slots, inv_freq, sp, q_norm, k_norm, ep
     over the whole projection, a weight per element; ``sp.head_norm``: over every head - and map -
     of ``dim`` elements, one weight of ``dim`` elements for all) and the rotation; the cache row of
     slots >= 0 gets [keys | values], keys normed and rotated alike, values divided by their per-head
-    root mean square when ``sp.v_norm``. ``sp.yarn``: cos and sin times its amplitude; ``sp.unit_qk``:
-    every rotated query / key head divided by its root mean square."""
+    root mean square when ``sp.v_norm``. ``sp.scaling``: cos and sin times its amplitude; ``sp.unit_qk``:
+    every rotated query / key head divided by its root mean square; ``sp.temp_every`` > 0: the query at
+    position p times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)."""
     T = proj.shape[0]
     nq, nk, nv = sp.q_size, sp.k_size, sp.v_size
     own_kv = sp.kv_from is None
@@ -579,10 +580,13 @@ def attn_prepare(proj, cache, positions, slots, inv_freq, sp, q_norm, k_norm, ep
     q = q.reshape(T, sp.heads * sp.maps, sp.dim)
     if sp.head_norm:
         q = _rows_rms(q, eps) * q_norm.float()
-    amp = sp.yarn.amplitude if sp.yarn is not None else 1.0
+    amp = sp.scaling.amplitude if sp.scaling is not None else 1.0
     q = partial_rope(q, positions, inv_freq, amp)
     if sp.unit_qk:
         q = _rows_rms(q, eps)
+    if sp.temp_every > 0:
+        steps = torch.div(positions + 1, sp.temp_every, rounding_mode="floor").float()
+        q = q * (1.0 + sp.temp_coef * torch.log(steps + 1.0))[:, None, None]
     proj[:, :nq] = q.reshape(T, nq).to(proj.dtype)
     if not own_kv:
         return
@@ -602,7 +606,8 @@ def attn_prepare(proj, cache, positions, slots, inv_freq, sp, q_norm, k_norm, ep
 def window_attention(out, proj, cache, seq_cu, seq_ctx, seq_bt, sp, gate_off, out_scale, lam=0.0, eps=0.0, sink_w=None):
     """Per sequence s (rows cu[s]..cu[s+1]-1 at positions ctx[s]-n .. ctx[s]-1): head h scores
     its prepared query against the cached keys of head h // (heads / kv_heads) with
-    0 <= pos - j < window or j < sp.keep_first; scores s_j = q . k * scale, then
+    0 <= pos - j < window or j < sp.keep_first (``sp.chunk`` > 0: j <= pos in pos's chunk of that many
+    positions); scores s_j = q . k * scale, then
     softcap * tanh(s_j / softcap) (softcap > 0); weights exp(s_j) / (sink + sum exp(s_j)) with
     sink = exp(sink_w[h]) (1 without weights); out[t, h * vdim ..] =
     weighted values * sigmoid(proj[t, gate_off + h]) (gate_off >= 0; ``sp.channel_gate``: element e of the
@@ -620,6 +625,8 @@ def window_attention(out, proj, cache, seq_cu, seq_ctx, seq_bt, sp, gate_off, ou
         ctx = int(seq_ctx[s])
         pos = torch.arange(ctx - (b - a), ctx, device=proj.device)
         lo = 0 if (W <= 0 or sp.keep_first > 0) else max(0, int(pos[0]) - W + 1)
+        if sp.chunk > 0:
+            lo = int(pos[0]) // sp.chunk * sp.chunk
         j = torch.arange(lo, ctx, device=proj.device)
         kv = flat[seq_bt[s].long()[j // bs] * bs + j % bs].float()
         k = kv[:, :G * M * d].view(-1, G, M * d).repeat_interleave(H // G, 1).reshape(-1, H * M, d)
@@ -631,6 +638,8 @@ def window_attention(out, proj, cache, seq_cu, seq_ctx, seq_bt, sp, gate_off, ou
             sc = torch.tanh(sc / sp.softcap) * sp.softcap
         dd = pos[:, None] - j[None]
         ok = (dd >= 0) & (((dd < W) | (j[None] < sp.keep_first)) if W > 0 else (dd >= 0))
+        if sp.chunk > 0:
+            ok &= pos[:, None] // sp.chunk == j[None] // sp.chunk
         sc = sc.masked_fill(~ok, float("-inf"))
         m = sc.max(-1, keepdim=True).values
         sk = 0.0   # the sink's logit: a key without a value
@@ -659,12 +668,16 @@ def _conv_inputs(proj, conv_state, a, b, start, slot, C, taps):
     return torch.cat([prev if start > 0 else torch.zeros_like(prev), x], 0)
 
 
-def gated_delta(y, S, conv_state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps, seq_cu, seq_ctx, seq_state):
-    """proj rows = [q | k | v | beta | decay | gate] pre-activations. Per sequence, from its slot
-    (zero when the step starts at position 0): causal conv + SiLU on q, k, v; unit q (times
-    dim^-1/2) and k; S = g S; u = beta (v - S^T k); S += k u^T; o = S^T q; y = o / rms(o) *
-    norm_w * silu(gate). S [slots, heads, dim, vdim], conv_state [slots, taps - 1, channels]."""
+def gated_delta(y, S, conv_state, proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps, seq_cu, seq_ctx,
+                seq_state):
+    """proj rows = [q | k | v | ...] pre-activations with the decay's, the gate's and beta's columns from ``offs`` on
+    (decay, gate, beta); ``decay`` fp32 [T, heads * dim] and ``gate`` [T, heads * vdim] are the decay's and the gate's
+    pre-activations where they come from bottlenecks (``sp.channel_decay``: a decay per key channel), else None. Per
+    sequence, from its slot (zero when the step starts at position 0): causal conv + SiLU on q, k, v; unit q (times
+    dim^-1/2) and k; S = g S; u = beta (v - S^T k); S += k u^T; o = S^T q; y = o / rms(o) * norm_w * act(gate),
+    act SiLU or sigmoid (``sp.gate_act``). S [slots, heads, dim, vdim], conv_state [slots, taps - 1, channels]."""
     H, G, d, dv, taps = sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.conv
+    off_a, off_g, off_b = offs
     C = sp.conv_channels
     cu = [int(x) for x in seq_cu]
     w = conv_w.float()
@@ -685,19 +698,21 @@ def gated_delta(y, S, conv_state, proj, conv_w, a_log, dt_bias, norm_w, sp, eps,
         q = q * torch.rsqrt(q.pow(2).sum(-1, keepdim=True) + 1e-6) * d ** -0.5
         k = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
         q, k = q.repeat_interleave(H // G, 1), k.repeat_interleave(H // G, 1)
-        p = proj[a:b, C:].float()
-        beta = torch.sigmoid(p[:, :H])
-        g = torch.exp(-torch.exp(a_log.float()) * torch.nn.functional.softplus(p[:, H:2 * H] + dt_bias.float()))
-        gate = p[:, 2 * H:].view(n, H, dv)
+        beta = torch.sigmoid(proj[a:b, off_b:off_b + H].float())
+        pre = (decay[a:b] if decay is not None else proj[a:b, off_a:off_a + H]).float() + dt_bias.float()
+        # [n, heads, dim or 1]
+        g = torch.exp(-torch.exp(a_log.float())[None, :, None] * torch.nn.functional.softplus(pre).view(n, H, -1))
+        gp = (gate[a:b] if gate is not None else proj[a:b, off_g:off_g + H * dv]).float().view(n, H, dv)
+        ga = torch.sigmoid(gp) * (gp if sp.gate_act == "silu" else 1.0)
         st = S[slot].clone() if start > 0 else torch.zeros_like(S[slot])
         o = torch.empty(n, H, dv)
         for t in range(n):
-            st = st * g[t, :, None, None]
+            st = st * g[t][:, :, None]
             u = beta[t, :, None] * (v[t] - torch.einsum("hkv,hk->hv", st, k[t]))
             st = st + k[t, :, :, None] * u[:, None, :]
             o[t] = torch.einsum("hkv,hk->hv", st, q[t])
         S[slot] = st
-        o = _rows_rms(o, eps) * norm_w.float() * (gate * torch.sigmoid(gate))
+        o = _rows_rms(o, eps) * norm_w.float() * ga
         y[a:b] = o.reshape(n, H * dv).to(y.dtype)
 
 
@@ -819,11 +834,13 @@ def wkv(out, S, proj, wl, w0, u, norm_w, sp, eps, seq_cu, seq_ctx, seq_state):
         out[a0:b0] = (_rows_rms(o, eps).reshape(n, N) * norm_w.float() * (g * torch.sigmoid(g))).to(out.dtype)
 
 
-def route_topk(ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False, score="softmax"):
+def route_topk(ids, wts, logits, correction, top, scale, E, groups=1, keep_groups=1, renorm=False, score="softmax",
+               group_top2=False):
     """s = softmax(logits) (fp32, over all router outputs) or, ``score`` = ``sigmoid``, the sigmoid of each; the ``top`` outputs with the largest
     s + correction are chosen (ties: the lower index); wts = s * scale of the chosen, ids = their
     index, outputs >= E (experts without weights) all written as E. ``groups`` > 1: the outputs
-    form equal groups of neighbours, a group scores its largest s + correction, and outputs
+    form equal groups of neighbours, a group scores its largest s + correction (``group_top2``: the
+    sum of its two largest, of s alone without a correction), and outputs
     outside the ``keep_groups`` best groups cannot be chosen. ``renorm``: the chosen s are divided
     by their sum (+ 1e-20) before the scaling. ``correction`` None: chosen by the logits themselves, whose
     order is that of s (a saturated s would tie)."""
@@ -832,6 +849,9 @@ def route_topk(ids, wts, logits, correction, top, scale, E, groups=1, keep_group
     if groups > 1:
         T, n = c.shape
         best = c.view(T, groups, n // groups).max(-1).values
+        if group_top2:
+            of = c if correction is not None else s
+            best = of.reshape(T, groups, n // groups).topk(min(2, n // groups), dim=-1).values.sum(-1)
         kept = torch.argsort(-best, dim=-1, stable=True)[:, :keep_groups]
         allow = torch.zeros_like(best, dtype=torch.bool).scatter_(1, kept, True)
         c = c.masked_fill(~allow.repeat_interleave(n // groups, 1), float("-inf"))
@@ -990,3 +1010,28 @@ def lightning(out, S, proj, decay, norm_w, sp, eps, seq_cu, seq_ctx, seq_state, 
         S[slot] = st
         o = _rows_rms(o.reshape(n, H * dv), eps) * norm_w.float() * torch.sigmoid(gate) * out_scale
         out[a:b] = o.to(out.dtype)
+
+
+# ---------------------------------------------------------------------------------
+# a norm before and a norm after every sublayer
+
+def sandwich_update(out, residual, w_next, eps, y=None, w_post=None, mult=1.0, table=None):
+    """residual (fp32, in place) += mult * y / rms(y) * w_post; out = residual / rms(residual) * w_next. ``y``: the
+    sublayer's result rows; a pair (a, a_w, b, b_w, a_scale, b_scale): a_scale a / rms(a) * a_w + b_scale b / rms(b) * b_w;
+    or a mixture's parts (ye, pair_slot, wts, shared, gate): sum_j wts[t, j] ye[pair_slot[t * top + j]] +
+    sigmoid(gate[t]) shared[t] (gate None: one). ``table`` = (rows, ids, scale): the residual starts as scale * rows[ids]."""
+    if table is not None:
+        rows, ids, scale = table
+        residual.copy_(rows[ids].float() * scale)
+    if isinstance(y, tuple) and len(y) == 6:
+        a, a_w, b, b_w, a_scale, b_scale = y
+        y = a_scale * _rows_rms(a.float(), eps) * a_w.float() + b_scale * _rows_rms(b.float(), eps) * b_w.float()
+    elif isinstance(y, tuple):
+        ye, pair_slot, wts, shared, gate = y
+        T, top = wts.shape
+        y = (ye.float().index_select(0, pair_slot.long().clamp(min=0)).view(T, top, -1) * wts.float().unsqueeze(-1)).sum(1)
+        if shared is not None:
+            y = y + (shared.float() if gate is None else shared.float() * torch.sigmoid(gate.float().view(T, 1)))
+    if y is not None:
+        residual += mult * _rows_rms(y.float(), eps) * w_post.float()
+    out.copy_((_rows_rms(residual, eps) * w_next.float()).to(out.dtype))
