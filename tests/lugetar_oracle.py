@@ -257,7 +257,7 @@ def moe(experts=6, top=2, ff=12, groups=(3, 2), scale=1.3, shared=18):
     return f
 
 
-def make_config(layers, width=28, vocab=90, eps=1e-5, scale=3.0, mult=0.6):
+def make_config(layers, width=28, vocab=90, eps=1e-5, scale=3.0, mult=0.4):
     return {"architecture": "Lugetar", "embedding": {"scale": scale}, "layers": layers, "norm": {"eps": eps},
             "residual_mult": mult, "vocab": vocab, "width": width}
 
