@@ -7,7 +7,8 @@ linear recurrences; its attention has no window), Topezen beside Kemavik (attent
 matrix-valued recurrence and routed experts with a shared expert in both) and beside Kesirax (the
 other design with latent attention), Zinavik beside Topezen (window attention with kept first
 tokens, a matrix-valued recurrence and routed experts in both) and beside Fikizen (the other
-design with parallel mixers). Random-init weights, synthetic prompts, a few layers of each (the per-layer
+design with parallel mixers), Lugetar beside Fikizen (window attention and a gated delta rule in both) and beside
+Zinavik (attention and a matrix-valued recurrence side by side, sigmoid-routed experts with a gated shared one). Random-init weights, synthetic prompts, a few layers of each (the per-layer
 cost is what is compared). ``--layer-models`` picks the models; the ratios are given per pair.
 
 Per size and model, through the engine's own scheduler and step function:
@@ -140,10 +141,34 @@ def zinavik_config(name, s):
                          eos_token_id=(2,), bos_token_id=1)
 
 
+def lugetar_config(name, s):
+    """Four layers: chunked attention and a gated delta rule with channel decays side by side + clamped feed-forward, causal
+    attention with growing queries + routed experts, and the two once more. Each half has half of the heads, as Zinavik's; the
+    chunks are as long as the other designs' windows."""
+    from ..config import (DenseFFSpec, GatedDeltaSpec, HybridLayerSpec, LlamaScaling, LugetarConfig, ParallelMixerSpec,
+                          RoutedMoESpec, WindowAttentionSpec)
+
+    H = s["heads"] // 2
+    left = WindowAttentionSpec(heads=H, kv_heads=max(1, H // 4), dim=128, vdim=128, scale=128 ** -0.5, chunk=s["window"],
+                               rot_dims=128, rot_base=5e5, llama=LlamaScaling(8.0, 8192, 1.0, 4.0), qk_norm=True)
+    right = GatedDeltaSpec(heads=H, kv_heads=H, dim=128, vdim=128, conv=4, channel_decay=True, gate_bottleneck=True,
+                           gate_act="sigmoid")
+    attn = WindowAttentionSpec(heads=s["heads"], kv_heads=max(1, s["heads"] // 4), dim=128, vdim=128, scale=128 ** -0.5,
+                               qk_norm=True, temp_coef=0.1, temp_every=1024)
+    moe = RoutedMoESpec(experts=s["experts"], top=s["top"], ff=s["ff"], scale=1.5, shared_ff=s["ff"], shared_gate=True,
+                        groups=4, keep_groups=2, group_top2=True, score="sigmoid", correction=False)
+    p = HybridLayerSpec(ParallelMixerSpec(left, right, 0.5, 0.5, out_norms=True),
+                        DenseFFSpec(s["dense_ff"] * 2 // 3 // 256 * 256, "clamped_glu", 7.0))
+    return LugetarConfig(name=f"lugetar-{name}", hidden_size=s["width"], vocab_size=s["vocab"],
+                         layers=(p, HybridLayerSpec(attn, moe)) * 2, embed_scale=float(s["width"]) ** 0.5, residual_mult=0.5,
+                         max_position_embeddings=16384, eos_token_id=(2,), bos_token_id=1)
+
+
 MODELS = {"kesirax": kesirax_config, "mixtral": mixtral_config, "fikizen": fikizen_config, "dense": dense_config,
-          "kemavik": kemavik_config, "topezen": topezen_config, "zinavik": zinavik_config}
+          "kemavik": kemavik_config, "topezen": topezen_config, "zinavik": zinavik_config, "lugetar": lugetar_config}
 PAIRS = (("kesirax", "mixtral"), ("fikizen", "dense"), ("kemavik", "fikizen"), ("kemavik", "mixtral"),
-         ("topezen", "kemavik"), ("topezen", "kesirax"), ("zinavik", "topezen"), ("zinavik", "fikizen"))
+         ("topezen", "kemavik"), ("topezen", "kesirax"), ("zinavik", "topezen"), ("zinavik", "fikizen"),
+         ("lugetar", "fikizen"), ("lugetar", "zinavik"))
 
 
 def measure(mcfg, batch, prompt_len, new_tokens, device="cuda", repeats=2):
