@@ -155,9 +155,17 @@ struct GatedDelta {
   float eps;
   bool channel, silu;                   // a decay per key channel; the gate through SiLU (else sigmoid)
   const float* decay; const void* gate; // launch_gated_delta, channel
+  float* chunks;                        // launch_gated_delta: delta_chunk_floats() floats: in chunks (dim <= delta_chunk_max_dim())
   const void *a2, *g2; int ra, rg;      // launch_gated_delta_step, channel: up-projections [heads * dim, ra], [heads * vdim, rg]
 };
 void launch_gated_delta(const GatedDelta& p, float* scratch, bool f32, hipStream_t s);
+// The recurrence in chunks of 16 tokens on the fp32 matrix cores (delta_chunk.hip) from the prepared rows: qk [T, 2 *
+// kv_heads * dim], vv [T, heads * vdim], gg [T, heads * (dim or 1)], bb [T, heads]; o [T, heads * vdim].
+int delta_chunk_max_dim();
+long delta_chunk_floats(int T, int nseq, int heads, int dim, int vdim);
+void launch_delta_chunk(float* o, float* S, float* buf, const float* qk, const float* vv, const float* gg,
+                        const float* bb, const int* seq_cu, const int* seq_ctx, const int* seq_state, int nseq, int T,
+                        int heads, int kv_heads, int dim, int vdim, bool channel, hipStream_t s);
 // The same for steps in which every sequence has ONE row: everything in one launch (two where heads share queries and
 // keys); the decay's and the gate's bottleneck outputs are columns off_a / off_g of proj. dim, vdim <= 256,
 // ra + rg <= gated_delta_step_max_rank().

@@ -19,6 +19,8 @@
 // softplus / exp of the decays and rates. head_norm_gate finishes both: per-head RMS norm of the
 // read-out, weight, SiLU or sigmoid gate, optional scale.
 //
+// Long prompt portions of the gated rule run in chunks on the matrix cores instead (delta_chunk.hip).
+//
 // Steps in which every sequence brings one row run the whole gated rule of a (sequence, head) in one workgroup
 // (gated_delta_step).
 #include "seq_common.h"
@@ -186,14 +188,6 @@ constexpr int kCV = 1;     // state columns per lane (2: half the waves, each tw
 constexpr int kScanThreads = 256;
 static_assert(kCV <= 2, "the read-out store below picks outs[0] / outs[1] by lane");
 constexpr int kCols = kScanThreads / kSeg * kCV;  // state columns per workgroup
-
-// Sum over the 16 lanes of a DPP row; every lane of the row gets it.
-HS_DEVICE float row_sum(float v) {
-  v = dpp_step<0xB1, 0xf, false>(v);   // quad_perm [1, 0, 3, 2]
-  v = dpp_step<0x4E, 0xf, false>(v);   // quad_perm [2, 3, 0, 1]
-  v = dpp_step<0x141, 0xf, false>(v);  // row_half_mirror
-  return dpp_step<0x140, 0xf, false>(v);  // row_mirror
-}
 
 // grid (heads, ceil(vdim / kCols), sequences), four waves: the step's first sequences (its prompt portions, the
 // long ones) are dispatched first and spread over the CUs before the one-token sequences fill in. A state column (one value channel) is held by the 16
@@ -660,15 +654,14 @@ __global__ __launch_bounds__(256) void wkv_step_kernel(
 //   pred_v = sum_k g_k k_k S_kv,  read_v = sum_k g_k q_k S_kv
 // give u_v = beta (v - pred_v) and o_v = read_v + (q . k) u_v, the read-out of the new state S' = g S + k u^T.
 // Thread (r, w) owns columns VEC w .. of rows r, r + R, ...
-constexpr int kStepIt = 16, kStepRank = 1024;
+constexpr int kStepThreads = 512, kStepIt = 8, kStepRank = 1024;
 
-// sum_j w[j] x[j] over a bottleneck; x in LDS
+// sum_j w[j] x[j] over a bottleneck, shared by the 16 lanes of a DPP row (every lane gets it); x in LDS
 template <typename T>
-HS_DEVICE float low_dot(const T* __restrict__ w, const float* x, int n, bool vec) {
+HS_DEVICE float low_dot(const T* __restrict__ w, const float* x, int n, int seg, bool vec) {
   float a = 0.f, b = 0.f;
   if (vec) {
-#pragma unroll 4
-    for (int j = 0; j < n; j += 8) {
+    for (int j = 8 * seg; j < n; j += 128) {
       float v[8];
       Row<T, 8>::ld(w + j, v);
 #pragma unroll
@@ -678,17 +671,17 @@ HS_DEVICE float low_dot(const T* __restrict__ w, const float* x, int n, bool vec
       }
     }
   } else {
-    for (int j = 0; j < n; ++j) a = __builtin_fmaf(ldf<T>(w, j), x[j], a);
+    for (int j = seg; j < n; j += 16) a = __builtin_fmaf(ldf<T>(w, j), x[j], a);
   }
-  return a + b;
+  return row_sum(a + b);
 }
 
 template <typename T, bool CH, int VEC>
-__global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta p, bool own_conv, bool vec_a, bool vec_g) {
+__global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const GatedDelta p, bool own_conv, bool vec_a, bool vec_g) {
   __shared__ float low[CH ? kStepRank : 1];                                 // [decay bottleneck | gate bottleneck]
   __shared__ float xs[3 * 256];                                             // silu(conv): q | k | v
-  __shared__ float sg[256], su[256];                                        // decays, u
-  __shared__ float red[2][1024];                                            // partial sums [r][column]: pred, read
+  __shared__ float sg[256], su[256], sgate[256];                            // decays, u, the gate before its activation
+  __shared__ float red[2][4 * kStepThreads];                                // partial sums [r][column]: pred, read
   __shared__ float sc[16], sn[4];
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int t = p.seq_cu[s];
@@ -698,7 +691,7 @@ __global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta 
   const bool carried = p.seq_ctx[s] - 1 > 0;
   const T* row = (const T*)p.proj + (long)t * p.ld;
   float* Sp = p.S + ((long)p.seq_state[s] * p.heads + h) * dim * vdim;
-  const int W = vdim / VEC, R = 256 / W, r = tid / W, w = tid - r * W;
+  const int W = vdim / VEC, R = kStepThreads / W, r = tid / W, w = tid - r * W;
   const bool active = r < R;
   const bool kept = VEC == 4 && dim <= R * kStepIt;
   f32x4 st[VEC == 4 ? kStepIt : 1];
@@ -713,12 +706,12 @@ __global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta 
     }
   }
   if constexpr (CH) {
-    for (int j = tid; j < p.ra + p.rg; j += 256)
+    for (int j = tid; j < p.ra + p.rg; j += kStepThreads)
       low[j] = j < p.ra ? ldf<T>(row, p.off_a + j) : ldf<T>(row, p.off_g + j - p.ra);
   }
   // the convolution of the head's channels; with heads of their own queries and keys the kept inputs move on here
   float* cs = p.conv_state + (long)p.seq_state[s] * max(hist, 1) * C;
-  for (int i = tid; i < 2 * dim + vdim; i += 256) {
+  for (int i = tid; i < 2 * dim + vdim; i += kStepThreads) {
     const int c = i < dim ? kh * dim + i : i < 2 * dim ? nqk + kh * dim + i - dim : 2 * nqk + h * vdim + i - 2 * dim;
     const float cur = ldf<T>(row, c);
     const float* cw = p.conv_w + (long)c * taps;
@@ -742,19 +735,22 @@ __global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta 
   }
   if constexpr (CH) {
     const float ea = expf(p.a_log[h]);
-    for (int e = tid; e < dim; e += 256) {
+    const int seg = tid & (kSeg - 1);
+#pragma unroll 4
+    for (int e = tid / kSeg; e < dim; e += kStepThreads / kSeg) {
       const long i = (long)h * dim + e;
-      const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, vec_a);
-      sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
+      const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, seg, vec_a);
+      if (seg == 0) sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
+    }
+#pragma unroll 4
+    for (int e = tid / kSeg; e < vdim; e += kStepThreads / kSeg) {
+      const float a = low_dot<T>((const T*)p.g2 + ((long)h * vdim + e) * p.rg, low + p.ra, p.rg, seg, vec_g);
+      if (seg == 0) sgate[e] = a;
     }
   } else {
     const float g = expf(-expf(p.a_log[h]) * softplus_f(ldf<T>(row, p.off_a + h) + p.dt_bias[h]));
-    for (int e = tid; e < dim; e += 256) sg[e] = g;
-  }
-  float gp = 0.f;
-  if (tid < vdim) {
-    if constexpr (CH) gp = low_dot<T>((const T*)p.g2 + ((long)h * vdim + tid) * p.rg, low + p.ra, p.rg, vec_g);
-    else gp = ldf<T>(row, p.off_g + h * vdim + tid);
+    for (int e = tid; e < dim; e += kStepThreads) sg[e] = g;
+    for (int e = tid; e < vdim; e += kStepThreads) sgate[e] = ldf<T>(row, p.off_g + h * vdim + e);
   }
   __syncthreads();
   const float fq = 1.f / sqrtf(sn[0] + 1e-6f) / sqrtf((float)dim), fk = 1.f / sqrtf(sn[1] + 1e-6f);
@@ -802,7 +798,7 @@ __global__ __launch_bounds__(256) void gated_delta_step_kernel(const GatedDelta 
   }
   const float ss = block_sum(tid < vdim ? o * o : 0.f, sc);   // also orders the writes of su before the reads below
   if (tid < vdim) {
-    const float gv = sigmoid_f(gp) * (p.silu ? gp : 1.f);
+    const float gp = sgate[tid], gv = sigmoid_f(gp) * (p.silu ? gp : 1.f);
     stf<T>((T*)p.y, (long)t * p.y_ld + (long)h * vdim + tid, o / sqrtf(ss / (float)vdim + p.eps) * p.norm_w[tid] * gv);
   }
   if (!active) return;
@@ -890,9 +886,9 @@ void gated_delta(const GatedDelta& p, float* scratch, hipStream_t s) {
   const int nqk = p.kv_heads * p.dim, nv = p.heads * p.vdim, ng = CH ? p.heads * p.dim : p.heads;
   const long T_ = p.T;
   float* qk = scratch;            // [T, 2 nqk]
-  float* vv = qk + T_ * 2 * nqk;  // [T, nv]
-  float* gg = vv + T_ * nv;       // [T, ng]
-  float* bb = gg + T_ * ng;       // [T, heads]
+  float* gg = qk + T_ * 2 * nqk;  // [T, ng]
+  float* vv = gg + T_ * ng;       // [T, nv]
+  float* bb = vv + T_ * nv;       // [T, heads]
   float* o = bb + T_ * p.heads;   // [T, nv]
   const int items = 2 * p.kv_heads + (nv + 64 * kPrepCh - 1) / (64 * kPrepCh) + (CH ? p.heads : 1) + 1;
   dim3 pgrid((p.T + kPrepTokens - 1) / kPrepTokens, (items + 3) / 4);
@@ -904,6 +900,10 @@ void gated_delta(const GatedDelta& p, float* scratch, hipStream_t s) {
   if (p.taps == 4) HS_GP(4); else if (p.taps == 3) HS_GP(3); else if (p.taps == 2) HS_GP(2); else HS_GP(0);
 #undef HS_GP
   conv_state_update<T>(p, s);
+  if (p.chunks != nullptr) {
+    launch_delta_chunk(o, p.S, p.chunks, qk, vv, gg, bb, p.seq_cu, p.seq_ctx, p.seq_state, p.nseq, p.T, p.heads, p.kv_heads,
+                       p.dim, p.vdim, CH, s);
+  } else {
   dim3 grid(p.heads, (p.vdim + kCols - 1) / kCols, p.nseq);
   switch (ds_of(p.dim)) {
 #define HS_GD(D)                                                                                                     \
@@ -913,6 +913,7 @@ void gated_delta(const GatedDelta& p, float* scratch, hipStream_t s) {
     break;
     HS_GD(1) HS_GD(2) HS_GD(4) HS_GD(8) HS_GD(16)
 #undef HS_GD
+  }
   }
   const bool own = p.gate != nullptr;   // the gate's rows: the bottleneck's result, or columns of the projection
   head_norm_gate<T>(p.y, p.y_ld, o, own ? p.gate : p.proj, own ? nv : p.ld, own ? 0 : p.off_g, p.norm_w, 0, p.T, p.heads,
@@ -925,8 +926,8 @@ void gated_delta_step(const GatedDelta& p, hipStream_t s) {
   auto ok = [](const void* q, int n) { return n % 8 == 0 && reinterpret_cast<uintptr_t>(q) % 16 == 0; };
   const bool va = ok(p.a2, p.ra), vg = ok(p.g2, p.rg);
   dim3 grid(p.heads, p.nseq);
-  if (p.vdim % 4 == 0) gated_delta_step_kernel<T, CH, 4><<<grid, 256, 0, s>>>(p, own_conv, va, vg);
-  else gated_delta_step_kernel<T, CH, 1><<<grid, 256, 0, s>>>(p, own_conv, va, vg);
+  if (p.vdim % 4 == 0) gated_delta_step_kernel<T, CH, 4><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
+  else gated_delta_step_kernel<T, CH, 1><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
   if (!own_conv) conv_state_update<T>(p, s);   // its readers are other workgroups too: after all of them
 }
 

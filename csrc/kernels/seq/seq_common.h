@@ -16,6 +16,10 @@ template <> struct Row<float, 1> {
   static HS_DEVICE void ld(const float* p, float (&v)[1]) { v[0] = *p; }
   static HS_DEVICE void st(float* p, const float (&v)[1]) { *p = v[0]; }
 };
+template <> struct Row<float, 2> {
+  static HS_DEVICE void ld(const float* p, float (&v)[2]) { const float2 a = *reinterpret_cast<const float2*>(p); v[0] = a.x; v[1] = a.y; }
+  static HS_DEVICE void st(float* p, const float (&v)[2]) { *reinterpret_cast<float2*>(p) = float2{v[0], v[1]}; }
+};
 template <> struct Row<float, 4> {
   static HS_DEVICE void ld(const float* p, float (&v)[4]) {
     const f32x4 a = *reinterpret_cast<const f32x4*>(p);
@@ -67,6 +71,14 @@ template <> struct Row<unsigned short, 8> {
 };
 
 HS_DEVICE float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
+
+// Sum over the 16 lanes of a DPP row; every lane of the row gets it.
+HS_DEVICE float row_sum(float v) {
+  v = dpp_step<0xB1, 0xf, false>(v);   // quad_perm [1, 0, 3, 2]
+  v = dpp_step<0x4E, 0xf, false>(v);   // quad_perm [2, 3, 0, 1]
+  v = dpp_step<0x141, 0xf, false>(v);  // row_half_mirror
+  return dpp_step<0x140, 0xf, false>(v);  // row_mirror
+}
 
 // First key (behind the kept ones) that position pos sees: its window's, its chunk's, or the sequence's first.
 HS_DEVICE int first_key(int pos, int window, int chunk) {

@@ -87,7 +87,7 @@ void gated_delta(at::Tensor& y, at::Tensor& S, at::Tensor& conv_state, const at:
                  const c10::optional<at::Tensor>& gate, const at::Tensor& seq_cu, const at::Tensor& seq_ctx,
                  const at::Tensor& seq_state, at::Tensor& scratch, int64_t heads, int64_t kv_heads, int64_t dim,
                  int64_t vdim, int64_t taps, double eps, int64_t off_a, int64_t off_g, int64_t off_b, bool channel,
-                 bool silu) {
+                 bool silu, const c10::optional<at::Tensor>& chunks) {
   auto p = gated_args(y, S, conv_state, proj, conv_w, a_log, dt_bias, norm_w, seq_cu, seq_ctx, seq_state, heads, kv_heads,
                       dim, vdim, taps, eps, off_a, off_g, off_b, channel, silu);
   CHECK_F32(scratch);
@@ -100,8 +100,19 @@ void gated_delta(at::Tensor& y, at::Tensor& S, at::Tensor& conv_state, const at:
     p.decay = decay->data_ptr<float>();
     p.gate = gate->data_ptr();
   }
+  if (chunks.has_value()) {
+    CHECK_F32(*chunks);
+    TORCH_CHECK(dim <= hipserve::delta_chunk_max_dim() &&
+                chunks->numel() >= hipserve::delta_chunk_floats(p.T, p.nseq, heads, dim, vdim) && p.T / 16 + p.nseq <= 65535,
+                "gated_delta: room for the chunks");
+    p.chunks = chunks->data_ptr<float>();
+  }
   c10::hip::HIPGuardMasqueradingAsCUDA g(proj.device());
   hipserve::launch_gated_delta(p, scratch.data_ptr<float>(), is_f32(proj, "gated_delta"), cur_stream());
+}
+
+int64_t delta_chunk_floats(int64_t T, int64_t nseq, int64_t heads, int64_t dim, int64_t vdim) {
+  return dim > hipserve::delta_chunk_max_dim() ? 0 : hipserve::delta_chunk_floats(T, nseq, heads, dim, vdim);
 }
 
 void gated_delta_step(at::Tensor& y, at::Tensor& S, at::Tensor& conv_state, const at::Tensor& proj,
@@ -313,7 +324,8 @@ TORCH_LIBRARY(hipserve_delta, m) {
   m.def("gated_delta(Tensor(a!) y, Tensor(b!) S, Tensor(c!) conv_state, Tensor proj, Tensor conv_w, Tensor a_log, "
         "Tensor dt_bias, Tensor norm_w, Tensor? decay, Tensor? gate, Tensor seq_cu, Tensor seq_ctx, Tensor seq_state, "
         "Tensor(d!) scratch, int heads, int kv_heads, int dim, int vdim, int taps, float eps, int off_a, int off_g, int off_b, "
-        "bool channel, bool silu) -> ()");
+        "bool channel, bool silu, Tensor(e!)? chunks=None) -> ()");
+  m.def("delta_chunk_floats(int T, int nseq, int heads, int dim, int vdim) -> int", &delta_chunk_floats);
   m.def("gated_delta_step(Tensor(a!) y, Tensor(b!) S, Tensor(c!) conv_state, Tensor proj, Tensor conv_w, Tensor a_log, "
         "Tensor dt_bias, Tensor norm_w, Tensor? a2, Tensor? g2, Tensor seq_cu, Tensor seq_ctx, Tensor seq_state, int heads, "
         "int kv_heads, int dim, int vdim, int taps, float eps, int off_a, int off_g, int off_b, bool channel, bool silu) -> ()");

@@ -51,7 +51,7 @@ LIBS = {
     "seq": ("_C_seq.so", ["kernels/seq/group_norm.hip", "kernels/seq/latent_attention*.hip", "kernels/seq/mingru.hip",
                           "kernels/seq/expert_ffn.hip", "kernels/moe.hip"], "seq_bindings.cpp"),
     "delta": ("_C_delta.so", ["kernels/seq/group_norm.hip", "kernels/seq/window_attention*.hip",
-                              "kernels/seq/delta_scan.hip", "kernels/seq/sandwich.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",
+                              "kernels/seq/delta_scan.hip", "kernels/seq/delta_chunk.hip", "kernels/seq/sandwich.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",
                               "kernels/seq/elementwise.hip", "kernels/moe.hip"], "seq_delta_bindings.cpp"),
     "cell": ("_C_cell.so", ["kernels/seq/gated_block.hip", "kernels/seq/mlstm.hip", "kernels/seq/latent_attention*.hip",
                             "kernels/seq/window_attention*.hip", "kernels/seq/router.hip", "kernels/seq/expert_ffn.hip",

@@ -338,15 +338,25 @@ class KernelOps:
                                            sp.heads, sp.kv_heads, sp.dim, sp.vdim, gate_off, sp.scale, sp.window,
                                            sp.sink, out_scale, *diff)
 
+    # bf16 prompt portions of at least this many rows run the gated delta rule in chunks on the (fp32) matrix cores
+    # (HIPSERVE_DELTA_CHUNK=0: token by token on the scan, as fp32 does)
+    DELTA_CHUNK = os.environ.get("HIPSERVE_DELTA_CHUNK", "1") != "0"
+    DELTA_CHUNK_ROWS = 32
+    DELTA_CHUNK_DTYPES = (torch.bfloat16,)
+
     def gated_delta(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, decay, gate, offs, sp, eps, meta):
         """``decay`` (fp32) / ``gate``: the pre-activations that come from bottlenecks (None: columns of ``proj``);
         ``offs``: the columns of ``proj`` where the decay, the gate and beta (or the bottlenecks) start."""
         T = proj.shape[0]
         scratch = torch.empty(T * (2 * sp.kv_heads * sp.dim + 2 * sp.out_size + sp.heads * (1 + (sp.dim if sp.channel_decay else 1))),
                               device=proj.device, dtype=torch.float32)
+        chunks = None
+        if self.DELTA_CHUNK and proj.dtype in self.DELTA_CHUNK_DTYPES and meta.max_q >= self.DELTA_CHUNK_ROWS:
+            n = self._delta.delta_chunk_floats(T, meta.seq_ctx.shape[0], sp.heads, sp.dim, sp.vdim)   # 0: not for these sizes
+            chunks = torch.empty(n, device=proj.device, dtype=torch.float32) if n else None
         self._delta.gated_delta(y, state[0], state[1], proj, conv_w, a_log, dt_bias, norm_w, decay, gate, meta.seq_cu,
                                 meta.seq_ctx, meta.seq_state, scratch, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.conv, eps,
-                                *offs, sp.channel_decay, sp.gate_act == "silu")
+                                *offs, sp.channel_decay, sp.gate_act == "silu", chunks)
 
     def gated_delta_step(self, y, state, proj, conv_w, a_log, dt_bias, norm_w, w_a2, w_g2, offs, sp, eps, meta):
         """``gated_delta`` for steps in which every sequence has one row (``meta.max_q`` == 1), the bottlenecks'

@@ -229,6 +229,43 @@ def test_channel_delta_alone(target, shape):
             assert bool((t[0] == 7.0).all()) and bool((t[2] == 7.0).all())
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("channel", [True, False])
+@pytest.mark.parametrize("heads,kv,dim,vdim", [(4, 2, 64, 64), (3, 3, 40, 20), (2, 1, 128, 128), (2, 2, 7, 9), (2, 1, 17, 300), (1, 1, 100, 16), (2, 2, 16, 33)])
+def test_delta_chunks_against_the_scan_gpu(dtype, channel, heads, kv, dim, vdim):
+    """The chunked matrix-core kernels against the token-by-token scan, in 32-bit as well: sequences of unequal length
+    (one row, none, a whole number of chunks, one row more), fresh and carried states, strong and weak decays, keys that
+    repeat, write strengths near one."""
+    dev, dt = torch.device("cuda"), getattr(torch, dtype)
+    g = torch.Generator().manual_seed(dim)
+    spec = GatedDeltaSpec(heads, kv, dim, vdim, 4, channel_decay=channel, gate_bottleneck=channel, gate_act="sigmoid" if channel else "silu")
+    mix = make_mixer(spec, 64, EPS, dev, dt, delta_ops(dev))
+    t = mix.init_random(g, 0.1)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    lens, ctx = [70, 1, 0, 16, 33, 5], [70, 9, 4, 16, 80, 5]
+    T = sum(lens)
+    meta, _ = one_seq_meta(1, dev)
+    meta.seq_cu, meta.seq_ctx, meta.seq_state = i32([0] + torch.tensor(lens).cumsum(0).tolist()), i32(ctx), i32([5, 1, 0, 2, 4, 3])
+    meta.max_q = max(lens)
+    start = [torch.randn(s, generator=g).to(dev) for s in mix.state_shapes(7)]
+    h = torch.randn(T, 64, generator=g)
+    h[20:40] = h[20]           # the same key again and again
+    h = h.to(dev, dt)
+    for log_a, beta in ((-1.0, 1.0), (-8.0, 30.0), (4.0, 1.0), (1.0, 30.0)):
+        w = dict(t, A_log=torch.full((heads,), log_a), b=t["b"] * beta)
+        mix.load(lambda k: w[k], "")
+        outs = []
+        for dtypes in ((), (torch.bfloat16, torch.float32)):
+            mix.ops.DELTA_CHUNK_DTYPES = dtypes
+            st = [s.clone() for s in start]
+            outs.append((mix.forward(h, meta, None, st).float(), st))
+        assert bool(torch.isfinite(outs[1][0]).all())
+        for a, b in [(outs[0][0], outs[1][0])] + list(zip(outs[0][1], outs[1][1])):
+            tol = 1e-4 if dtype == "float32" or a.dim() != 2 else 2e-2
+            assert float((a - b).abs().max()) < tol * float(b.abs().max()), (log_a, beta)
+
+
 @pytest.mark.parametrize("target", TARGETS)
 def test_delta_state_taken_turns_and_what_matters(target):
     """Two sequences take turns in two slots, single rows between portions; a lost or mixed-up state or convolution tail
