@@ -142,7 +142,7 @@ void launch_window_attention_mfma(void* out, long out_ld, const void* proj, long
 // columns from off_b on and the decay's / the gate's pre-activations from off_a / off_g on, or from `decay` (fp32
 // [T, heads * dim]: a decay per key channel) and `gate` ([T, heads * vdim], activation type); dt_bias has as many
 // elements as a token has decays. scratch: fp32, T * (2 * kv_heads * dim + 2 * heads * vdim + heads * (1 + decays per
-// head)) floats; the generalized rule's: T * 7 * heads * dim.
+// head)) + 64 floats; the generalized rule's: T * 7 * heads * dim.
 int delta_max_dim();
 int delta_max_taps();
 struct GatedDelta {
@@ -160,7 +160,7 @@ struct GatedDelta {
 };
 void launch_gated_delta(const GatedDelta& p, float* scratch, bool f32, hipStream_t s);
 // The recurrence in chunks of 16 tokens on the fp32 matrix cores (delta_chunk.hip) from the prepared rows: qk [T, 2 *
-// kv_heads * dim], vv [T, heads * vdim], gg [T, heads * (dim or 1)], bb [T, heads]; o [T, heads * vdim].
+// kv_heads * dim], vv [T, heads * vdim], gg [T, heads * (dim or 1)], bb [T, heads]; o [T, heads * vdim] and 64 floats behind it (written, not read).
 int delta_chunk_max_dim();
 long delta_chunk_floats(int T, int nseq, int heads, int dim, int vdim);
 void launch_delta_chunk(float* o, float* S, float* buf, const float* qk, const float* vv, const float* gg,

@@ -219,8 +219,9 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
 template <int TPW, int NW>
 __global__ __launch_bounds__(64 * NW) void delta_chunk_scan_kernel(
     float* __restrict__ o, float* __restrict__ S, float* __restrict__ base, const int* __restrict__ seq_cu,
-    const int* __restrict__ seq_ctx, const int* __restrict__ seq_state, int heads, int dim, int vdim, int VP) {
+    const int* __restrict__ seq_ctx, const int* __restrict__ seq_state, int heads, int dim, int vdim, int VP, long pad) {
   constexpr int DP = 16 * TPW * NW;
+  static_assert(NW == 1 || NW == 2 || NW == 4, "the waves share the four rows of a lane");
   __shared__ __attribute__((aligned(16))) f32x4 part[2][2][NW][64];   // [chunk parity][W S | (G q) S][wave][lane]
   const int s = blockIdx.z, h = blockIdx.x, v0 = 16 * blockIdx.y;
   const int r0 = seq_cu[s], n = seq_cu[s + 1] - r0;
@@ -240,39 +241,45 @@ __global__ __launch_bounds__(64 * NW) void delta_chunk_scan_kernel(
       const int k = 16 * (wave * TPW + b) + 4 * g + r;
       st[b][r] = (carried && k < dim && col < vdim) ? Sp[(long)k * vdim] : 0.f;
     }
-  // a chunk's operands, loaded one chunk ahead
-  f32x4 W[TPW], Q[TPW], K[TPW], E[TPW], U, P;
-  auto fetch = [&](int ci) {
-    const ChunkBuf b = chunk_buf(base, (long)(first + ci) * heads + h, DP, VP);
+  // Two chunks' operands, each loaded two chunks ahead as soon as its registers are free. Loads and stores of the loop are
+  // unconditional (past the end the last chunk is loaded again, rows and columns that do not exist are stored behind
+  // o), so that the wait for an operand never has to cover the younger loads behind it.
+  struct Ops {
+    f32x4 W[TPW], Q[TPW], K[TPW], E[TPW], U, P;
+  } even, odd;
+  auto fetch_products = [&](Ops& x, int ci) {   // what the products with the state take
+    const ChunkBuf b = chunk_buf(base, (long)(first + min(ci, nc - 1)) * heads + h, DP, VP);
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+      const int at = c * DP + 16 * (wave * TPW + i) + 4 * g;
+      x.W[i] = *reinterpret_cast<const f32x4*>(b.W + at);
+      x.Q[i] = *reinterpret_cast<const f32x4*>(b.GQ + at);
+    }
+  };
+  auto fetch_update = [&](Ops& x, int ci) {     // what the state's update and the read-out take
+    const ChunkBuf b = chunk_buf(base, (long)(first + min(ci, nc - 1)) * heads + h, DP, VP);
 #pragma unroll
     for (int i = 0; i < TPW; ++i) {
       const int k0 = 16 * (wave * TPW + i);
-      W[i] = *reinterpret_cast<const f32x4*>(b.W + c * DP + k0 + 4 * g);
-      Q[i] = *reinterpret_cast<const f32x4*>(b.GQ + c * DP + k0 + 4 * g);
-      K[i] = *reinterpret_cast<const f32x4*>(b.KT + (k0 + c) * kC + 4 * g);
-      E[i] = *reinterpret_cast<const f32x4*>(b.GE + k0 + 4 * g);
+      x.K[i] = *reinterpret_cast<const f32x4*>(b.KT + (k0 + c) * kC + 4 * g);
+      x.E[i] = *reinterpret_cast<const f32x4*>(b.GE + k0 + 4 * g);
     }
-    U = *reinterpret_cast<const f32x4*>(b.UT + (long)col * kC + 4 * g);   // col < VP
-    P = *reinterpret_cast<const f32x4*>(b.P + c * kC + 4 * g);
+    x.U = *reinterpret_cast<const f32x4*>(b.UT + (long)col * kC + 4 * g);   // col < VP
+    x.P = *reinterpret_cast<const f32x4*>(b.P + c * kC + 4 * g);
   };
-  fetch(0);
-  for (int ci = 0; ci < nc; ++ci) {
+  auto step = [&](Ops& x, int ci) {
     f32x4 ws = {0.f, 0.f, 0.f, 0.f}, qs = ws;
 #pragma unroll
     for (int b = 0; b < TPW; ++b)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        ws = __builtin_amdgcn_mfma_f32_16x16x4f32(W[b][r], st[b][r], ws, 0, 0, 0);
-        qs = __builtin_amdgcn_mfma_f32_16x16x4f32(Q[b][r], st[b][r], qs, 0, 0, 0);
+        ws = __builtin_amdgcn_mfma_f32_16x16x4f32(x.W[b][r], st[b][r], ws, 0, 0, 0);
+        qs = __builtin_amdgcn_mfma_f32_16x16x4f32(x.Q[b][r], st[b][r], qs, 0, 0, 0);
       }
-    f32x4 kk[TPW], u = U;
-    const f32x4 pp = P;
+    fetch_products(x, ci + 2);
+    f32x4 u = x.U;
 #pragma unroll
-    for (int b = 0; b < TPW; ++b) {
-      kk[b] = K[b];
-      st[b] *= E[b];
-    }
-    if (ci + 1 < nc) fetch(ci + 1);
+    for (int b = 0; b < TPW; ++b) st[b] *= x.E[b];
     f32x4 (*pt)[NW][64] = part[ci & 1];
     if constexpr (NW > 1) {
       pt[0][wave][lane] = ws;
@@ -286,22 +293,33 @@ __global__ __launch_bounds__(64 * NW) void delta_chunk_scan_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int b = 0; b < TPW; ++b) st[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[b][r], u[r], st[b], 0, 0, 0);
-    if (wave == ci % NW) {   // the waves take turns with the read-outs
-      f32x4 oo = qs;
+      for (int b = 0; b < TPW; ++b) st[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.K[b][r], u[r], st[b], 0, 0, 0);
+    f32x4 oo = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(x.P[r], u[r], oo, 0, 0, 0);
+    fetch_update(x, ci + 2);
+#pragma unroll
+    for (int k = 0; k < 4 / NW; ++k) {   // wave w reads out the rows 4 g + w (+ NW ..)
+      const int r = wave + NW * k, i = ci * kC + 4 * g + r;
+      float y = r == 0 ? oo[0] : r == 1 ? oo[1] : r == 2 ? oo[2] : oo[3];
       if constexpr (NW > 1) {
-        oo = pt[1][0][lane];
 #pragma unroll
-        for (int i = 1; i < NW; ++i) oo += pt[1][i][lane];
+        for (int w = 0; w < NW; ++w) y += reinterpret_cast<const float*>(&pt[1][w][lane])[r];
+      } else {
+        y += r == 0 ? qs[0] : r == 1 ? qs[1] : r == 2 ? qs[2] : qs[3];
       }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(pp[r], u[r], oo, 0, 0, 0);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int i = ci * kC + 4 * g + r;
-        if (i < n && col < vdim) o[(long)(r0 + i) * nv + h * vdim + col] = oo[r];
-      }
+      const long at = i < n && col < vdim ? (long)(r0 + i) * nv + h * vdim + col : pad + lane;
+      o[at] = y;
     }
+  };
+  fetch_products(even, 0);
+  fetch_update(even, 0);
+  fetch_products(odd, 1);
+  fetch_update(odd, 1);
+  for (int ci = 0; ci < nc; ci += 2) {
+    step(even, ci);
+    if (ci + 1 >= nc) break;
+    step(odd, ci + 1);
   }
 #pragma unroll
   for (int b = 0; b < TPW; ++b)
@@ -337,7 +355,8 @@ void launch_delta_chunk(float* o, float* S, float* buf, const float* qk, const f
     else                                                                                                               \
       delta_chunk_prepare_kernel<DS, false><<<pgrid, 256, 0, s>>>(buf, qk, vv, gg, bb, seq_cu, nseq, heads, kv_heads, dim, \
                                                                   vdim, VP);                                           \
-    delta_chunk_scan_kernel<TPW, NW><<<sgrid, 64 * NW, 0, s>>>(o, S, buf, seq_cu, seq_ctx, seq_state, heads, dim, vdim, VP); \
+    delta_chunk_scan_kernel<TPW, NW><<<sgrid, 64 * NW, 0, s>>>(o, S, buf, seq_cu, seq_ctx, seq_state, heads, dim, vdim, VP,  \
+                                                               (long)T * heads * vdim);                                \
   } while (0)
   switch (padded(dim)) {
     case 16: HS_DC(1, 1, 1); break;

@@ -97,7 +97,16 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(
   bool carried = false, fresh = true;
   if (s < 0) return;
   end = seq_cu[s + 1];
+  float nxt[kPrepCh];   // the next row's inputs, loaded a row ahead
+#pragma unroll
+  for (int i = 0; i < kPrepCh; ++i) nxt[i] = lane + 64 * i < nc ? ldf<T>(proj, (long)t0 * ld + c0 + lane + 64 * i) : 0.f;
   for (int t = t0; t < t1; ++t) {
+    float row[kPrepCh];
+#pragma unroll
+    for (int i = 0; i < kPrepCh; ++i) {
+      row[i] = nxt[i];
+      if (t + 1 < t1 && lane + 64 * i < nc) nxt[i] = ldf<T>(proj, (long)(t + 1) * ld + c0 + lane + 64 * i);
+    }
     while (t >= end) {   // the next sequence that has rows
       if (++s >= nseq) return;
       end = seq_cu[s + 1];
@@ -129,7 +138,7 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(
       if (64 * i >= nc) continue;
       const int c = c0 + lane + 64 * i;
       if (lane + 64 * i < nc) {
-        const float cur = ldf<T>(proj, (long)t * ld + c);
+        const float cur = row[i];
         float a = 0.f;
         if constexpr (TAPS > 0) {
 #pragma unroll
@@ -736,13 +745,11 @@ __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const Ga
   if constexpr (CH) {
     const float ea = expf(p.a_log[h]);
     const int seg = tid & (kSeg - 1);
-#pragma unroll 4
     for (int e = tid / kSeg; e < dim; e += kStepThreads / kSeg) {
       const long i = (long)h * dim + e;
       const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, seg, vec_a);
       if (seg == 0) sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
     }
-#pragma unroll 4
     for (int e = tid / kSeg; e < vdim; e += kStepThreads / kSeg) {
       const float a = low_dot<T>((const T*)p.g2 + ((long)h * vdim + e) * p.rg, low + p.ra, p.rg, seg, vec_g);
       if (seg == 0) sgate[e] = a;

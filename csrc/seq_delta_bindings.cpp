@@ -91,7 +91,7 @@ void gated_delta(at::Tensor& y, at::Tensor& S, at::Tensor& conv_state, const at:
   auto p = gated_args(y, S, conv_state, proj, conv_w, a_log, dt_bias, norm_w, seq_cu, seq_ctx, seq_state, heads, kv_heads,
                       dim, vdim, taps, eps, off_a, off_g, off_b, channel, silu);
   CHECK_F32(scratch);
-  TORCH_CHECK(scratch.numel() >= (long)p.T * (2 * kv_heads * dim + 2 * heads * vdim + heads * (1 + (channel ? dim : 1))));
+  TORCH_CHECK(scratch.numel() >= (long)p.T * (2 * kv_heads * dim + 2 * heads * vdim + heads * (1 + (channel ? dim : 1))) + 64);
   TORCH_CHECK(channel == decay.has_value() && channel == gate.has_value(), "gated_delta: bottlenecks' results");
   if (channel) {
     CHECK_F32(*decay); CHECK_CONTIG(*gate);

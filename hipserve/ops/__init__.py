@@ -348,7 +348,7 @@ class KernelOps:
         """``decay`` (fp32) / ``gate``: the pre-activations that come from bottlenecks (None: columns of ``proj``);
         ``offs``: the columns of ``proj`` where the decay, the gate and beta (or the bottlenecks) start."""
         T = proj.shape[0]
-        scratch = torch.empty(T * (2 * sp.kv_heads * sp.dim + 2 * sp.out_size + sp.heads * (1 + (sp.dim if sp.channel_decay else 1))),
+        scratch = torch.empty(T * (2 * sp.kv_heads * sp.dim + 2 * sp.out_size + sp.heads * (1 + (sp.dim if sp.channel_decay else 1))) + 64,
                               device=proj.device, dtype=torch.float32)
         chunks = None
         if self.DELTA_CHUNK and proj.dtype in self.DELTA_CHUNK_DTYPES and meta.max_q >= self.DELTA_CHUNK_ROWS:
