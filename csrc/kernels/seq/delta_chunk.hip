@@ -229,7 +229,7 @@ __global__ __launch_bounds__(64 * NW) void delta_chunk_scan_kernel(
   int first = 0;   // the sequence's first chunk in the step
   for (int i = 0; i < s; ++i) first += (seq_cu[i + 1] - seq_cu[i] + kC - 1) / kC;
   const int nc = (n + kC - 1) / kC;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 15, g = lane >> 4;
   const int col = v0 + c, nv = heads * vdim;
   const bool carried = seq_ctx[s] - n > 0;
   float* Sp = S + ((long)seq_state[s] * heads + h) * dim * vdim + col;
@@ -316,6 +316,7 @@ __global__ __launch_bounds__(64 * NW) void delta_chunk_scan_kernel(
   fetch_update(even, 0);
   fetch_products(odd, 1);
   fetch_update(odd, 1);
+  __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0): the loop's own waits then count the loop's loads only
   for (int ci = 0; ci < nc; ci += 2) {
     step(even, ci);
     if (ci + 1 >= nc) break;

@@ -149,16 +149,18 @@ class LayerListModel:
 
     def step_workspace_bytes(self, tokens: int, seqs: int) -> int:
         el = torch.finfo(self.dtype).bits // 8
-        wide = 0
+        wide = scratch = 0
         for lw in self.layers:
             if lw is None:
                 continue
+            for m in (lw.mixer, getattr(lw.mixer, "left", None), getattr(lw.mixer, "right", None)):
+                scratch = max(scratch, getattr(m, "scratch_floats", 0))
             n = 3 * _proj_width(lw.mixer)
             if lw.mlp is not None:
                 f = lw.mlp.spec
                 n = max(n, 2 * f.ff * getattr(f, "top", 1) * 2 + 2 * getattr(f, "shared_ff", 0))
             wide = max(wide, n)
-        return tokens * (wide * (el + 4) + 12 * self.cfg.hidden_size) + seqs * self.cfg.vocab_size * 12
+        return tokens * (wide * (el + 4) + 4 * scratch + 12 * self.cfg.hidden_size) + seqs * self.cfg.vocab_size * 12
 
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
         """32-bit logits = head . hidden."""

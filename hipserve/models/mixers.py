@@ -525,6 +525,12 @@ class GatedDelta:
     def out_size(self) -> int:
         return self.spec.out_size
 
+    @property
+    def scratch_floats(self) -> int:
+        """32-bit scratch of a step per token: the prepared rows, the read-outs and the chunks' operands."""
+        s = self.spec
+        return 2 * s.conv_channels + s.heads * (2 * s.dim + 1) + s.heads * (4 * max(s.dim, 16) + max(s.vdim, 16) + 16)
+
     def state_shapes(self, slots: int):
         s = self.spec
         return [(slots, s.heads, s.dim, s.vdim), (slots, max(s.conv - 1, 1), s.conv_channels)]
