@@ -685,8 +685,21 @@ HS_DEVICE float low_dot(const T* __restrict__ w, const float* x, int n, int seg,
   return row_sum(a + b);
 }
 
-template <typename T, bool CH, int VEC>
+// The same from weights that were loaded before x was there: lane seg holds w[8 seg .. 8 seg + 7] (n <= 128).
+HS_DEVICE float low_dot8(const u16x8 w, const float* x, int n, int seg) {
+  float a = 0.f;
+  if (8 * seg < n) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) a = __builtin_fmaf(bf16_to_f32(w[i]), x[8 * seg + i], a);
+  }
+  return row_sum(a);
+}
+
+// EARLY (bf16, ranks of a multiple of 8 up to 128, head sizes up to 128): the up-projections' weights are loaded with the state.
+template <typename T, bool CH, int VEC, bool EARLY>
 __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const GatedDelta p, bool own_conv, bool vec_a, bool vec_g) {
+  static_assert(!EARLY || (CH && sizeof(T) == 2), "early weights are bf16 bottlenecks");
+  constexpr int kEarly = EARLY ? 128 / (kStepThreads / kSeg) : 1;   // rows of each up-projection per lane row
   __shared__ float low[CH ? kStepRank : 1];                                 // [decay bottleneck | gate bottleneck]
   __shared__ float xs[3 * 256];                                             // silu(conv): q | k | v
   __shared__ float sg[256], su[256], sgate[256];                            // decays, u, the gate before its activation
@@ -712,6 +725,17 @@ __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const Ga
         st[i] = f32x4{0.f, 0.f, 0.f, 0.f};
         if (active && k < dim && carried) st[i] = *reinterpret_cast<const f32x4*>(Sp + (long)k * vdim + 4 * w);
       }
+    }
+  }
+  const int seg = tid & (kSeg - 1);
+  u16x8 wa[kEarly], wg[kEarly];
+  if constexpr (EARLY) {
+#pragma unroll
+    for (int i = 0; i < kEarly; ++i) {
+      const int e = tid / kSeg + i * (kStepThreads / kSeg);
+      wa[i] = wg[i] = u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      if (e < dim && 8 * seg < p.ra) wa[i] = *reinterpret_cast<const u16x8*>((const T*)p.a2 + ((long)h * dim + e) * p.ra + 8 * seg);
+      if (e < vdim && 8 * seg < p.rg) wg[i] = *reinterpret_cast<const u16x8*>((const T*)p.g2 + ((long)h * vdim + e) * p.rg + 8 * seg);
     }
   }
   if constexpr (CH) {
@@ -744,7 +768,15 @@ __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const Ga
   }
   if constexpr (CH) {
     const float ea = expf(p.a_log[h]);
-    const int seg = tid & (kSeg - 1);
+    if constexpr (EARLY) {
+#pragma unroll
+      for (int i = 0; i < kEarly; ++i) {
+        const int e = tid / kSeg + i * (kStepThreads / kSeg);
+        const float a = low_dot8(wa[i], low, p.ra, seg), b = low_dot8(wg[i], low + p.ra, p.rg, seg);
+        if (seg == 0 && e < dim) sg[e] = expf(-ea * softplus_f(a + p.dt_bias[(long)h * dim + e]));
+        if (seg == 0 && e < vdim) sgate[e] = b;
+      }
+    } else {
     for (int e = tid / kSeg; e < dim; e += kStepThreads / kSeg) {
       const long i = (long)h * dim + e;
       const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, seg, vec_a);
@@ -753,6 +785,7 @@ __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const Ga
     for (int e = tid / kSeg; e < vdim; e += kStepThreads / kSeg) {
       const float a = low_dot<T>((const T*)p.g2 + ((long)h * vdim + e) * p.rg, low + p.ra, p.rg, seg, vec_g);
       if (seg == 0) sgate[e] = a;
+    }
     }
   } else {
     const float g = expf(-expf(p.a_log[h]) * softplus_f(ldf<T>(row, p.off_a + h) + p.dt_bias[h]));
@@ -933,8 +966,13 @@ void gated_delta_step(const GatedDelta& p, hipStream_t s) {
   auto ok = [](const void* q, int n) { return n % 8 == 0 && reinterpret_cast<uintptr_t>(q) % 16 == 0; };
   const bool va = ok(p.a2, p.ra), vg = ok(p.g2, p.rg);
   dim3 grid(p.heads, p.nseq);
-  if (p.vdim % 4 == 0) gated_delta_step_kernel<T, CH, 4><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
-  else gated_delta_step_kernel<T, CH, 1><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
+  bool early = false;
+  if constexpr (CH && sizeof(T) == 2) {
+    early = va && vg && p.ra <= 128 && p.rg <= 128 && p.dim <= 128 && p.vdim <= 128 && p.vdim % 4 == 0;
+    if (early) gated_delta_step_kernel<T, CH, 4, true><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
+  }
+  if (!early && p.vdim % 4 == 0) gated_delta_step_kernel<T, CH, 4, false><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
+  else if (!early) gated_delta_step_kernel<T, CH, 1, false><<<grid, kStepThreads, 0, s>>>(p, own_conv, va, vg);
   if (!own_conv) conv_state_update<T>(p, s);   // its readers are other workgroups too: after all of them
 }
 

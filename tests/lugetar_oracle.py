@@ -279,10 +279,11 @@ def make_weights(cfg, seed=0, gain=1.0, rank=11):
                 p + "k.norm": 1.5 + rnd(kk, std=0.3), p + "o": mat(Wd, m["heads"] * m["vdim"])}
 
     def delta(m, p):
+        rank_g = rank + (8 if rank % 8 == 0 else 2)   # the two bottlenecks differ in width
         qk, v, dec, taps = m["kv_heads"] * m["dim"], m["heads"] * m["vdim"], m["heads"] * m["dim"], m["conv"]
         t = {p + "b": mat(m["heads"], Wd, 1.5), p + "A_log": rnd(m["heads"], std=0.5) - 1.5,
              p + "dt_bias": rnd(dec, std=0.7), p + "norm": 1 + rnd(m["vdim"], std=0.2), p + "a1": mat(rank, Wd),
-             p + "a2": mat(dec, rank, 1.5), p + "g1": mat(rank + 2, Wd), p + "g2": mat(v, rank + 2, 2.0), p + "o": mat(Wd, v)}
+             p + "a2": mat(dec, rank, 1.5), p + "g1": mat(rank_g, Wd), p + "g2": mat(v, rank_g, 2.0), p + "o": mat(Wd, v)}
         for n, c in (("q", qk), ("k", qk), ("v", v)):
             t[p + n], t[p + n + ".conv"] = mat(c, Wd, 1.5), rnd(c, taps, std=0.7)
         return t
