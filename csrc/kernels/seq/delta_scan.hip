@@ -777,15 +777,15 @@ __global__ __launch_bounds__(kStepThreads) void gated_delta_step_kernel(const Ga
         if (seg == 0 && e < vdim) sgate[e] = b;
       }
     } else {
-    for (int e = tid / kSeg; e < dim; e += kStepThreads / kSeg) {
-      const long i = (long)h * dim + e;
-      const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, seg, vec_a);
-      if (seg == 0) sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
-    }
-    for (int e = tid / kSeg; e < vdim; e += kStepThreads / kSeg) {
-      const float a = low_dot<T>((const T*)p.g2 + ((long)h * vdim + e) * p.rg, low + p.ra, p.rg, seg, vec_g);
-      if (seg == 0) sgate[e] = a;
-    }
+      for (int e = tid / kSeg; e < dim; e += kStepThreads / kSeg) {
+        const long i = (long)h * dim + e;
+        const float a = low_dot<T>((const T*)p.a2 + i * p.ra, low, p.ra, seg, vec_a);
+        if (seg == 0) sg[e] = expf(-ea * softplus_f(a + p.dt_bias[i]));
+      }
+      for (int e = tid / kSeg; e < vdim; e += kStepThreads / kSeg) {
+        const float a = low_dot<T>((const T*)p.g2 + ((long)h * vdim + e) * p.rg, low + p.ra, p.rg, seg, vec_g);
+        if (seg == 0) sgate[e] = a;
+      }
     }
   } else {
     const float g = expf(-expf(p.a_log[h]) * softplus_f(ldf<T>(row, p.off_a + h) + p.dt_bias[h]));
@@ -944,16 +944,16 @@ void gated_delta(const GatedDelta& p, float* scratch, hipStream_t s) {
     launch_delta_chunk(o, p.S, p.chunks, qk, vv, gg, bb, p.seq_cu, p.seq_ctx, p.seq_state, p.nseq, p.T, p.heads, p.kv_heads,
                        p.dim, p.vdim, CH, s);
   } else {
-  dim3 grid(p.heads, (p.vdim + kCols - 1) / kCols, p.nseq);
-  switch (ds_of(p.dim)) {
+    dim3 grid(p.heads, (p.vdim + kCols - 1) / kCols, p.nseq);
+    switch (ds_of(p.dim)) {
 #define HS_GD(D)                                                                                                     \
   case D:                                                                                                            \
     gated_delta_scan_kernel<D, CH><<<grid, kScanThreads, 0, s>>>(o, p.S, qk, vv, gg, bb, p.seq_cu, p.seq_ctx,          \
                                                                  p.seq_state, p.heads, p.kv_heads, p.dim, p.vdim);    \
     break;
-    HS_GD(1) HS_GD(2) HS_GD(4) HS_GD(8) HS_GD(16)
+      HS_GD(1) HS_GD(2) HS_GD(4) HS_GD(8) HS_GD(16)
 #undef HS_GD
-  }
+    }
   }
   const bool own = p.gate != nullptr;   // the gate's rows: the bottleneck's result, or columns of the projection
   head_norm_gate<T>(p.y, p.y_ld, o, own ? p.gate : p.proj, own ? nv : p.ld, own ? 0 : p.off_g, p.norm_w, 0, p.T, p.heads,
